@@ -4,12 +4,16 @@
 * ``cera_amd/lib/libcera_host.so`` -- CPU host layer: quantizers, GGUF, synthetic models (g++)
 * ``cera_amd/lib/libcera_hip_llama.so`` + ``cera_amd/lib/cera-hip`` -- the Model-trait layer
   above the C-ABI and its command-line driver (g++)
+* ``cera_amd/lib/libcera_hip_layered.so`` + ``cera_amd/lib/cera-trace`` -- the trace runner with
+  only the kernels of the models it loads, linked from the same objects
 """
 from __future__ import annotations
 
+import hashlib
 import os
 import shutil
 import subprocess
+import sys
 from pathlib import Path
 
 PKG = Path(__file__).resolve().parent
@@ -19,9 +23,13 @@ HIP_LIB = LIB_DIR / "libcera_hip.so"
 HOST_LIB = LIB_DIR / "libcera_host.so"
 LLAMA_LIB = LIB_DIR / "libcera_hip_llama.so"
 CLI_BIN = LIB_DIR / "cera-hip"
+LAYERED_LIB = LIB_DIR / "libcera_hip_layered.so"
+TRACE_BIN = LIB_DIR / "cera-trace"
 HSACO = LIB_DIR / "cera_hip_gfx950.hsaco"
 
 HIP_SRCS = sorted((PKG / "csrc").glob("*.hip"))
+# what the layered float models need of csrc/
+LAYERED_SRCS = [PKG / "csrc" / f"{n}.hip" for n in ("ctx", "model_api", "layered", "dense", "sigmoid_attn", "conv_norm")]
 HOST_SRCS = sorted((PKG / "host").glob("*.cpp"))
 
 # -ffp-contract=off: the parity target never fuses a*b+c implicitly; FMAs in
@@ -47,40 +55,42 @@ def hipcc_path() -> str:
     raise RuntimeError("hipcc not found")
 
 
-def build_hip(verbose: bool = False, jobs: int = 8) -> Path:
-    """Compile every csrc/*.hip to an object (in parallel) and link the C-ABI library."""
+def _run(cmd, verbose: bool, what: str) -> None:
+    r = subprocess.run(cmd, capture_output=True, text=True)
+    if verbose or r.returncode:
+        print(" ".join(cmd), file=sys.stderr)
+        print(r.stdout + r.stderr, file=sys.stderr)
+    if r.returncode:
+        raise RuntimeError(what)
+
+
+def compile_hip(srcs, verbose: bool = False, jobs: int = 8) -> list[str]:
+    """Compile HIP sources to objects in parallel; returns their paths."""
     from concurrent.futures import ThreadPoolExecutor
 
     LIB_DIR.mkdir(exist_ok=True)
     obj_dir = LIB_DIR / "obj"
     obj_dir.mkdir(exist_ok=True)
-    srcs = sorted((PKG / "csrc").glob("*.hip"))
-    hipcc = hipcc_path()
     flags = [f for f in HIPCC_FLAGS if f != "-shared"]
 
-    def compile_one(src: Path):
+    def compile_one(src: Path) -> str:
         obj = obj_dir / (src.stem + ".o")
-        cmd = [hipcc, *flags, f"-I{ROOT / 'include'}", f"-I{PKG / 'csrc'}", "-c", str(src), "-o", str(obj)]
-        r = subprocess.run(cmd, capture_output=True, text=True)
-        return src, obj, cmd, r
+        _run([hipcc_path(), *flags, f"-I{ROOT / 'include'}", f"-I{PKG / 'csrc'}", "-c", str(src), "-o", str(obj)],
+             verbose, f"hipcc failed on {src.name}")
+        return str(obj)
 
-    objs = []
     with ThreadPoolExecutor(max_workers=jobs) as ex:
-        for src, obj, cmd, r in ex.map(compile_one, srcs):
-            if verbose or r.returncode:
-                print(" ".join(cmd))
-                print(r.stdout + r.stderr)
-            if r.returncode:
-                raise RuntimeError(f"hipcc failed on {src.name}")
-            objs.append(str(obj))
-    cmd = [hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", str(HIP_LIB)]
-    r = subprocess.run(cmd, capture_output=True, text=True)
-    if verbose or r.returncode:
-        print(" ".join(cmd))
-        print(r.stdout + r.stderr)
-    if r.returncode:
-        raise RuntimeError("hipcc link failed")
-    return HIP_LIB
+        return list(ex.map(compile_one, srcs))
+
+
+def link_hip(objs, out: Path, verbose: bool = False) -> Path:
+    _run([hipcc_path(), "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", str(out)], verbose, "hipcc link failed")
+    return out
+
+
+def build_hip(verbose: bool = False, jobs: int = 8) -> Path:
+    """Compile every csrc/*.hip to an object (in parallel) and link the C-ABI library."""
+    return link_hip(compile_hip(sorted((PKG / "csrc").glob("*.hip")), verbose, jobs), HIP_LIB, verbose)
 
 
 def build_hsaco(verbose: bool = False) -> Path:
@@ -121,20 +131,61 @@ def build_backend(verbose: bool = False) -> Path:
               f"-I{ROOT / 'include'}", f"-I{PKG / 'host'}", f"-I{PKG / 'backend'}"]
     link = [f"-L{LIB_DIR}", "-lcera_hip", "-lcera_host", "-Wl,-rpath,$ORIGIN"]
     b = PKG / "backend"
-    gguf = str(PKG / "host" / "gguf.cpp")  # C++ classes are not exported by the host library: compile them in
+    # C++ classes are not exported by the host library: compile them in
+    host = [str(PKG / "host" / f) for f in ("gguf.cpp", "json.cpp", "safetensors.cpp")]
+    models = [str(b / f) for f in ("hip_device_model.cpp", "hip_llama.cpp", "hip_layered.cpp", "load_dir.cpp", "load_model.cpp")]
     cmds = [
-        [*common, "-shared", str(b / "hip_llama.cpp"), str(b / "hip_llama_capi.cpp"), gguf, "-o", str(LLAMA_LIB),
-         *link],
-        [*common, str(b / "cli.cpp"), str(b / "hip_llama.cpp"), gguf, "-o", str(CLI_BIN), *link],
+        [*common, "-shared", *models, str(b / "hip_llama_capi.cpp"), *host, "-o", str(LLAMA_LIB), *link],
+        [*common, str(b / "cli.cpp"), str(b / "trace.cpp"), *models, *host, "-o", str(CLI_BIN), *link],
     ]
     for cmd in cmds:
-        r = subprocess.run(cmd, capture_output=True, text=True)
-        if verbose or r.returncode:
-            print(" ".join(cmd))
-            print(r.stdout + r.stderr)
-        if r.returncode:
-            raise RuntimeError("g++ failed building the backend layer")
+        _run(cmd, verbose, "g++ failed building the backend layer")
     return LLAMA_LIB
+
+
+def _trace_sources() -> list[Path]:
+    """Every file the trace runner is built from (headers of the same directories included)."""
+    files = list(LAYERED_SRCS) + sorted((PKG / "csrc").glob("*.h")) + sorted((ROOT / "include").glob("*.h"))
+    return files + sorted((PKG / "host").glob("*.[ch]*")) + sorted((PKG / "backend").glob("*.[ch]*")) + [Path(__file__)]
+
+
+def _trace_stamp() -> str:
+    h = hashlib.sha256()
+    for f in _trace_sources():
+        h.update(f.name.encode() + b"\0" + f.read_bytes())
+    return h.hexdigest()
+
+
+def build_trace(verbose: bool = False, objs=None, jobs: int = 8) -> Path:
+    """The trace runner (cera-trace) and the library it runs on.  ``objs``: objects of LAYERED_SRCS
+    when they are compiled already."""
+    stamp = _trace_stamp()
+    if objs is None:
+        objs = compile_hip(LAYERED_SRCS, verbose, jobs)
+    link_hip(objs, LAYERED_LIB, verbose)
+    b, host = PKG / "backend", PKG / "host"
+    srcs = [b / "trace_run.cpp", b / "trace.cpp", b / "hip_device_model.cpp", b / "hip_layered.cpp", b / "load_dir.cpp",
+            host / "json.cpp", host / "safetensors.cpp"]
+    _run(["g++", "-O2", "-std=c++17", "-fPIC", "-pthread", "-Wall", "-Wextra", "-fvisibility=hidden", f"-I{ROOT / 'include'}",
+          f"-I{host}", f"-I{b}", *map(str, srcs), "-o", str(TRACE_BIN), f"-L{LIB_DIR}", "-lcera_hip_layered", "-lcera_host",
+          "-Wl,-rpath,$ORIGIN"], verbose, "g++ failed building the trace runner")
+    (LIB_DIR / "cera-trace.stamp").write_text(stamp)
+    return TRACE_BIN
+
+
+def ensure_trace() -> Path:
+    """The trace runner, built first when it is missing or its sources have changed since."""
+    import fcntl
+
+    LIB_DIR.mkdir(exist_ok=True)
+    with open(LIB_DIR / ".trace.lock", "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        stamp = LIB_DIR / "cera-trace.stamp"
+        built = all(p.exists() for p in (TRACE_BIN, LAYERED_LIB, HOST_LIB, stamp))
+        if not built or stamp.read_text() != _trace_stamp():
+            build_host()
+            build_trace()
+    return TRACE_BIN
 
 
 def build_all(verbose: bool = False) -> None:
@@ -142,6 +193,7 @@ def build_all(verbose: bool = False) -> None:
     build_hip(verbose)
     build_hsaco(verbose)
     build_backend(verbose)
+    build_trace(verbose, [str(LIB_DIR / "obj" / (p.stem + ".o")) for p in LAYERED_SRCS])
 
 
 if __name__ == "__main__":

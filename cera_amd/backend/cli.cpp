@@ -4,7 +4,11 @@
 //   cera-hip inspect --model m.gguf
 //   cera-hip run     --model m.gguf [--prompt-len 512] [--n-predict 256] [--seed S]
 //                    [--ubatch 512] [--ctx 1024] [--device 0] [--tokens-out FILE] [--per-token-prefill]
-//                    [--kv f32|f16]
+//                    [--kv f32|f16] [--dtype bf16|f32]
+//   cera-hip trace   --model DIR --out DIR [--dtype bfloat16|float32] [--max-tokens N]
+//
+// --model of `run` is a GGUF file or a directory with config.json and model.safetensors (--dtype is
+// for the latter).  `trace` replays given requests from standard input (trace.h).
 //
 // `run` is the workload `cera bench` times (cera-cli/src/main.rs:932-938 for the
 // protocol): a prompt of uniform random token ids is prefilled in `ubatch`
@@ -20,7 +24,9 @@
 #include <thread>
 
 #include "cera_host.h"
-#include "hip_llama.h"
+#include "gguf.h"
+#include "load_model.h"
+#include "trace.h"
 
 namespace {
 
@@ -125,15 +131,18 @@ int cmd_inspect(const Args& a) {
 }
 
 int cmd_run(const Args& a) {
-    std::string err;
-    auto g = cera::GgufFile::open(a.str("model", ""), &err);
-    if (!g) { std::fprintf(stderr, "%s\n", err.c_str()); return 1; }
     const size_t n_prompt = a.num("prompt-len", 512), n_predict = a.num("n-predict", 256), ubatch = a.num("ubatch", 512);
     const size_t ctx = a.num("ctx", std::max<size_t>(1024, n_prompt + n_predict));
+    const std::string dtype = a.str("dtype", "bf16");
+    if (dtype != "bf16" && dtype != "f32") { std::fprintf(stderr, "--dtype must be bf16 or f32\n"); return 1; }
     double t0 = now_s();
     std::unique_ptr<cera::Model> model;
     try {
-        model = cera::load_model_hip(*g, ctx, static_cast<int>(a.num("device", 0)));
+        cera::LoadOptions opt;
+        opt.context_size = ctx;
+        opt.device = static_cast<int>(a.num("device", 0));
+        opt.f32 = dtype == "f32";
+        model = cera::load_model(a.str("model", ""), opt);
     } catch (const std::exception& e) {
         std::fprintf(stderr, "load failed: %s\n", e.what());
         return 1;
@@ -168,9 +177,7 @@ int cmd_run(const Args& a) {
             auto r = model->forward_prefill_chunked(prompt.data(), n_prompt, 0, st, ubatch, cancel);
             logits = std::move(*r.second);
         }
-        uint32_t next = 0;
-        for (size_t i = 1; i < logits.size(); ++i)
-            if (logits[i] > logits[next]) next = static_cast<uint32_t>(i);
+        const uint32_t next = cera::argmax_token(logits);
         double t2 = now_s();
         out.push_back(next);
         while (out.size() < n_predict) out.push_back(model->forward_greedy(&out.back(), 1, st.seq_len, st));
@@ -204,10 +211,11 @@ int cmd_run(const Args& a) {
 
 int main(int argc, char** argv) {
     if (argc < 2) {
-        std::fprintf(stderr, "usage: cera-hip gen|inspect|run [options]\n");
+        std::fprintf(stderr, "usage: cera-hip gen|inspect|run|trace [options]\n");
         return 2;
     }
     std::string cmd = argv[1];
+    if (cmd == "trace") return cera::trace_main(argc, argv, 2);
     Args a = parse(argc, argv, 2);
     if (cmd == "gen") return cmd_gen(a);
     if (cmd == "inspect") return cmd_inspect(a);

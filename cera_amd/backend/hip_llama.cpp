@@ -1,8 +1,6 @@
 // HipLlamaModel over the C-ABI of cera_hip.h.  Reference lines: see hip_llama.h.
 #include "hip_llama.h"
 
-#include "cera_host.h"
-
 #include <algorithm>
 #include <cmath>
 #include <cstring>
@@ -39,43 +37,7 @@ cera_hip_tensor as_tensor(const GgufFile& g, const std::string& name) {
     return t;
 }
 
-size_t argmax(const std::vector<float>& v) {  // cera/src/sampler.rs:20-30
-    size_t best = 0;
-    float bv = -INFINITY;
-    for (size_t i = 0; i < v.size(); ++i)
-        if (v[i] > bv) { bv = v[i]; best = i; }
-    return best;
-}
-
 }  // namespace
-
-// ---- trait defaults (cera/src/model/mod.rs:207-220, 303-332, 494-497) ----
-
-std::vector<float> Model::forward_prefill(const uint32_t* tokens, size_t n, size_t start_pos, InferenceState& state) {
-    std::vector<float> logits;
-    for (size_t i = 0; i < n; ++i) logits = forward(tokens + i, 1, start_pos + i, state);
-    return logits;
-}
-
-uint32_t Model::forward_greedy(const uint32_t* tokens, size_t n, size_t pos, InferenceState& state) {
-    return static_cast<uint32_t>(argmax(forward(tokens, n, pos, state)));
-}
-
-std::pair<size_t, std::optional<std::vector<float>>> Model::forward_prefill_chunked(
-    const uint32_t* tokens, size_t n, size_t start_pos, InferenceState& state, size_t ubatch,
-    const std::atomic<bool>& cancel) {
-    if (ubatch == 0) ubatch = std::max<size_t>(n, 1);
-    size_t consumed = 0;
-    std::optional<std::vector<float>> last;
-    while (consumed < n) {
-        size_t len = std::min(ubatch, n - consumed);
-        last = forward_prefill(tokens + consumed, len, start_pos + consumed, state);
-        consumed += len;
-        // polled after the chunk, so a cancel raised before the call still advances by one chunk
-        if (cancel.load(std::memory_order_relaxed) && consumed < n) break;
-    }
-    return {consumed, std::move(last)};
-}
 
 // ---- HipLlamaModel ----
 
@@ -211,82 +173,12 @@ std::unique_ptr<HipLlamaModel> HipLlamaModel::from_gguf(const GgufFile& g, size_
     hc.logit_scale = c.scalars.logit;
     hc.rope_freqs = rope_freqs.empty() ? nullptr : rope_freqs.data();
 
-    if (cera_hip_ctx_create(device, nullptr, &self->ctx_) != CERA_HIP_OK)
-        bail(std::string("hip context: ") + cera_hip_last_error(nullptr));
+    self->open_context(device);
     if (cera_hip_model_create(self->ctx_, &hc, &embd, untied ? &output : nullptr, output_norm.data(), layers.data(),
                               &self->model_) != CERA_HIP_OK)
         bail(std::string("hip model: ") + cera_hip_last_error(self->ctx_));
     return self;
 }
-
-HipLlamaModel::~HipLlamaModel() {
-    if (model_) cera_hip_model_destroy(model_);
-    if (ctx_) cera_hip_ctx_destroy(ctx_);
-}
-
-void HipLlamaModel::device_panic(const char* what) const {
-    throw BackendError(std::string(what) + ": " + cera_hip_last_error(ctx_));
-}
-
-std::vector<float> HipLlamaModel::forward(const uint32_t* tokens, size_t n, size_t pos, InferenceState& state) {
-    if (n != 1) bail("HipLlamaModel forward expects single token");
-    if (tokens[0] >= config_.vocab_size)
-        bail("token_id " + std::to_string(tokens[0]) + " out of range (vocab_size=" + std::to_string(config_.vocab_size) + ")");
-    std::vector<float> logits(config_.vocab_size);
-    if (cera_hip_forward(model_, tokens[0], static_cast<uint32_t>(pos), logits.data()) != CERA_HIP_OK)
-        device_panic("forward");
-    state.seq_len = cera_hip_seq_len(model_);
-    return logits;
-}
-
-std::vector<float> HipLlamaModel::forward_prefill(const uint32_t* tokens, size_t n, size_t start_pos,
-                                                  InferenceState& state) {
-    if (n == 0) bail("forward_prefill requires at least one token");
-    if (start_pos != state.seq_len)
-        bail("forward_prefill: start_pos (" + std::to_string(start_pos) + ") must equal state.seq_len (" +
-             std::to_string(state.seq_len) + ")");
-    std::vector<float> logits(config_.vocab_size);
-    if (cera_hip_forward_prefill(model_, tokens, static_cast<uint32_t>(n), static_cast<uint32_t>(start_pos),
-                                 logits.data()) != CERA_HIP_OK)
-        device_panic("forward_prefill");
-    state.seq_len = cera_hip_seq_len(model_);
-    return logits;
-}
-
-std::vector<float> HipLlamaModel::forward_prefill_logits_all(const uint32_t* tokens, size_t n, size_t start_pos,
-                                                             InferenceState& state) {
-    if (n == 0) bail("forward_prefill_logits_all requires at least one token");
-    if (start_pos != state.seq_len)
-        bail("forward_prefill_logits_all: start_pos (" + std::to_string(start_pos) + ") must equal state.seq_len (" +
-             std::to_string(state.seq_len) + ")");
-    std::vector<float> logits(n * config_.vocab_size);
-    if (cera_hip_forward_prefill_logits_all(model_, tokens, static_cast<uint32_t>(n), static_cast<uint32_t>(start_pos),
-                                            logits.data()) != CERA_HIP_OK)
-        device_panic("forward_prefill_logits_all");
-    state.seq_len = cera_hip_seq_len(model_);
-    return logits;
-}
-
-uint32_t HipLlamaModel::forward_greedy(const uint32_t* tokens, size_t n, size_t pos, InferenceState& state) {
-    if (n != 1) bail("HipLlamaModel forward_greedy expects single token");
-    uint32_t next = 0;
-    if (cera_hip_forward_greedy(model_, tokens[0], static_cast<uint32_t>(pos), &next) != CERA_HIP_OK)
-        device_panic("forward_greedy");
-    state.seq_len = cera_hip_seq_len(model_);
-    return next;
-}
-
-void HipLlamaModel::truncate_kv(InferenceState& state, size_t len) {
-    if (len > state.seq_len)
-        bail("truncate_kv: len (" + std::to_string(len) + ") exceeds seq_len (" + std::to_string(state.seq_len) + ")");
-    if (cera_hip_truncate_kv(model_, static_cast<uint32_t>(len)) != CERA_HIP_OK) device_panic("truncate_kv");
-    state.seq_len = len;
-}
-
-// The trait defaults panic with unimplemented!(): a backend without device-resident state has
-// nothing to snapshot (cera/src/model/mod.rs:521-533).
-StateSnapshot Model::snapshot_state() { throw BackendError("snapshot_state not supported by this backend"); }
-void Model::restore_state(const StateSnapshot&) { throw BackendError("restore_state not supported by this backend"); }
 
 void HipLlamaModel::shift_kv(InferenceState& state, size_t n_keep, size_t shift) {
     // the reference asserts these in all builds (cera/src/kv_cache.rs:1110-1116)
@@ -308,93 +200,9 @@ KvCompression HipLlamaModel::kv_compression() const {
     return cera_hip_kv_type(model_) == CERA_HIP_KV_F16 ? KvCompression::F16 : KvCompression::None;
 }
 
-// the integer-only converters of the host library (the reference's, cera/src/quant.rs:48-164)
-static uint16_t half_bits(float v) { return cera_f32_to_f16(v); }
-static float half_value(uint16_t b) { return cera_f16_to_f32(b); }
-
-StateSnapshot HipLlamaModel::snapshot_state() {
-    StateSnapshot snap;
-    snap.seq_len = cera_hip_seq_len(model_);
-    const bool f16 = kv_compression() == KvCompression::F16;
-    const size_t elems = snap.seq_len * config_.n_kv_heads * config_.head_dim;
-    std::vector<float> k(elems), v(elems);
-    snap.layers.resize(config_.n_layers);
-    for (size_t l = 0; l < config_.n_layers; ++l) {
-        LayerSnapshot& L = snap.layers[l];
-        L.f16 = f16;
-        if (elems && cera_hip_read_kv(model_, static_cast<uint32_t>(l), k.data(), v.data()) != CERA_HIP_OK)
-            device_panic("snapshot_state");
-        if (!f16) {
-            L.k_data.assign(reinterpret_cast<uint8_t*>(k.data()), reinterpret_cast<uint8_t*>(k.data() + elems));
-            L.v_data.assign(reinterpret_cast<uint8_t*>(v.data()), reinterpret_cast<uint8_t*>(v.data() + elems));
-        } else {  // the cache's own half bits: read_kv widened them exactly
-            L.k_data.resize(elems * 2);
-            L.v_data.resize(elems * 2);
-            for (size_t i = 0; i < elems; ++i) {
-                const uint16_t kb = half_bits(k[i]), vb = half_bits(v[i]);
-                std::memcpy(L.k_data.data() + 2 * i, &kb, 2);
-                std::memcpy(L.v_data.data() + 2 * i, &vb, 2);
-            }
-        }
-    }
-    return snap;
-}
-
-void HipLlamaModel::restore_state(const StateSnapshot& snap) {
-    const bool f16 = kv_compression() == KvCompression::F16;
-    const size_t elems = snap.seq_len * config_.n_kv_heads * config_.head_dim;
-    const size_t bytes = elems * (f16 ? 2 : 4);
-    if (snap.layers.size() != config_.n_layers) bail("restore_state: snapshot has " + std::to_string(snap.layers.size()) +
-                                                     " layers, model has " + std::to_string(config_.n_layers));
-    if (snap.seq_len > config_.max_seq_len) bail("restore_state: snapshot is longer than the context");
-    for (const LayerSnapshot& L : snap.layers) {
-        // the cross-mode gate: an f16 snapshot never loads into an f32 cache or the reverse
-        if (L.f16 != f16) bail("restore_state: snapshot and model disagree on the KV cache element type");
-        if (L.k_data.size() != bytes || L.v_data.size() != bytes)
-            bail("restore_state: layer byte length does not match seq_len * kv_dim * element size");
-    }
-    std::vector<float> k(elems), v(elems);
-    for (size_t l = 0; l < config_.n_layers; ++l) {
-        const LayerSnapshot& L = snap.layers[l];
-        if (!f16) {
-            std::memcpy(k.data(), L.k_data.data(), bytes);
-            std::memcpy(v.data(), L.v_data.data(), bytes);
-        } else {
-            for (size_t i = 0; i < elems; ++i) {
-                uint16_t kb, vb;
-                std::memcpy(&kb, L.k_data.data() + 2 * i, 2);
-                std::memcpy(&vb, L.v_data.data() + 2 * i, 2);
-                k[i] = half_value(kb);
-                v[i] = half_value(vb);
-            }
-        }
-        if (cera_hip_write_kv(model_, static_cast<uint32_t>(l), k.data(), v.data(), static_cast<uint32_t>(snap.seq_len)) !=
-            CERA_HIP_OK)
-            device_panic("restore_state");
-    }
-    if (cera_hip_set_seq_len(model_, static_cast<uint32_t>(snap.seq_len)) != CERA_HIP_OK) device_panic("restore_state");
-}
-
 void HipLlamaModel::set_reference_order(uint32_t mode) {
     if (cera_hip_set_reference_order(model_, mode) != CERA_HIP_OK)
         bail(std::string("set_reference_order: ") + cera_hip_last_error(ctx_));
-}
-
-uint64_t HipLlamaModel::gpu_memory_bytes() const { return cera_hip_memory_bytes(model_); }
-
-std::string HipLlamaModel::device_name() const {
-    char name[256] = {0};
-    uint32_t cu = 0;
-    uint64_t hbm = 0;
-    if (cera_hip_device_info(ctx_, name, &cu, &hbm) != CERA_HIP_OK) return "unknown";
-    return std::string(name) + " (" + std::to_string(cu) + " CUs, " + std::to_string(hbm >> 30) + " GiB)";
-}
-
-std::unique_ptr<Model> load_model_hip(const GgufFile& gguf, size_t context_size, int device) {
-    std::string arch = gguf.get_str("general.architecture").value_or("unknown");
-    if (arch == "qwen2" || arch == "qwen3" || arch == "llama" || arch == "granite")
-        return HipLlamaModel::from_gguf(gguf, context_size, device);
-    bail("unsupported architecture for hip: " + arch);
 }
 
 }  // namespace cera

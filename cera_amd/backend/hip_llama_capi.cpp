@@ -3,14 +3,14 @@
 #include <algorithm>
 
 #include <chrono>
-#include <cmath>
 #include <cstring>
 
 #include "hip_llama.h"
+#include "load_model.h"
 
 struct cera_llama {
-    std::unique_ptr<cera::GgufFile> gguf;
-    std::unique_ptr<cera::HipLlamaModel> model;
+    std::unique_ptr<cera::Model> model;
+    cera::HipLlamaModel* llama = nullptr;   // the same model, when it is a llama
     cera::InferenceState state;
     std::atomic<bool> cancel{false};
     std::string err;
@@ -47,24 +47,25 @@ double now_s() {
 extern "C" {
 
 cera_llama* cera_llama_open(const char* path, uint64_t context_size, int device, char* err, uint64_t err_len) {
+    return cera_llama_open_dtype(path, context_size, device, 0, err, err_len);
+}
+cera_llama* cera_llama_open_dtype(const char* path, uint64_t context_size, int device, int f32, char* err, uint64_t err_len) {
     if (!path) {
         set_err(err, err_len, "null path");
         return nullptr;
     }
     std::unique_ptr<cera_llama> h(new cera_llama());
-    std::string e;
-    h->gguf = cera::GgufFile::open(path, &e);
-    if (!h->gguf) {
-        set_err(err, err_len, e);
-        return nullptr;
-    }
     try {
-        h->model = cera::HipLlamaModel::from_gguf(*h->gguf, context_size, device);
+        cera::LoadOptions opt;
+        opt.context_size = context_size;
+        opt.device = device;
+        opt.f32 = f32 != 0;
+        h->model = cera::load_model(path, opt);
+        h->llama = dynamic_cast<cera::HipLlamaModel*>(h->model.get());
     } catch (const std::exception& ex) {
         set_err(err, err_len, ex.what());
         return nullptr;
     }
-    // the weights are in HBM now; the mapping is only needed for metadata afterwards
     return h.release();
 }
 void cera_llama_close(cera_llama* h) { delete h; }
@@ -83,7 +84,7 @@ int cera_llama_get_config(const cera_llama* h, cera_llama_config* out) {
     out->max_seq_len = c.max_seq_len;
     out->rope_theta = c.rope_theta;
     out->rms_norm_eps = c.rms_norm_eps;
-    out->rope_type = h->model->rope_type() == cera::RopeType::Norm ? 1u : 0u;
+    out->rope_type = !h->llama || h->llama->rope_type() == cera::RopeType::Norm ? 1u : 0u;
     return 0;
 }
 uint64_t cera_llama_seq_len(const cera_llama* h) { return h->state.seq_len; }
@@ -159,7 +160,7 @@ uint64_t cera_llama_snapshot_seq_len(const cera_llama_snapshot* s) { return s ? 
 uint64_t cera_llama_snapshot_bytes(const cera_llama_snapshot* s) {
     uint64_t n = 0;
     if (s)
-        for (const auto& L : s->snap.layers) n += L.k_data.size() + L.v_data.size();
+        for (const auto& L : s->snap.layers) n += L.k_data.size() + L.v_data.size() + L.conv_data.size();
     return n;
 }
 int cera_llama_restore_state(cera_llama* h, const cera_llama_snapshot* s) {
@@ -179,12 +180,7 @@ int cera_llama_generate_greedy(cera_llama* h, const uint32_t* prompt, uint64_t n
         h->state = cera::InferenceState{};   // a generation starts with a new state, as Session::generate does
         double t0 = now_s();
         auto r = h->model->forward_prefill_chunked(prompt, n_prompt, 0, h->state, ubatch, never);
-        const std::vector<float>& l = *r.second;
-        size_t best = 0;
-        float bv = -INFINITY;
-        for (size_t i = 0; i < l.size(); ++i)
-            if (l[i] > bv) { bv = l[i]; best = i; }
-        out[0] = static_cast<uint32_t>(best);
+        out[0] = cera::argmax_token(*r.second);
         double t1 = now_s();
         for (uint64_t i = 1; i < n_new; ++i) out[i] = h->model->forward_greedy(&out[i - 1], 1, h->state.seq_len, h->state);
         double t2 = now_s();
@@ -195,9 +191,8 @@ int cera_llama_generate_greedy(cera_llama* h, const uint32_t* prompt, uint64_t n
 
 int cera_llama_set_reference_order(cera_llama* h, int on) {
     return guarded(h, [&] {
-        auto* hm = dynamic_cast<cera::HipLlamaModel*>(h->model.get());
-        if (!hm) throw cera::BackendError("set_reference_order: not a hip model");
-        hm->set_reference_order(on < 0 ? 0u : static_cast<uint32_t>(on));
+        if (!h->llama) throw cera::BackendError("set_reference_order: not a llama");
+        h->llama->set_reference_order(on < 0 ? 0u : static_cast<uint32_t>(on));
     });
 }
 

@@ -1,4 +1,4 @@
-/* C face of HipLlamaModel (hip_llama.h) for callers without C++: the ctypes
+/* C face of the Model trait over the model registry (load_model.h) for callers without C++: the ctypes
  * tests and the bench driver.  One handle = one loaded model + its
  * InferenceState + a cancel flag.  Every call returns 0 on success and -1 on
  * failure with the reason readable through cera_llama_last_error (the C++
@@ -22,6 +22,10 @@ typedef struct {
 
 CERA_LLAMA_API cera_llama* cera_llama_open(const char* gguf_path, uint64_t context_size, int device, char* err,
                                            uint64_t err_len);
+/* path: a GGUF file, or a directory with config.json and model.safetensors; f32 != 0 runs the latter's
+ * model in f32 instead of bf16. */
+CERA_LLAMA_API cera_llama* cera_llama_open_dtype(const char* path, uint64_t context_size, int device, int f32, char* err,
+                                                 uint64_t err_len);
 CERA_LLAMA_API void cera_llama_close(cera_llama*);
 CERA_LLAMA_API const char* cera_llama_last_error(const cera_llama*);
 CERA_LLAMA_API int cera_llama_get_config(const cera_llama*, cera_llama_config* out);

@@ -1,0 +1,113 @@
+// Kernels of conv_norm.h.  Everything here is f32 up to the store of an output row.
+#include "bf16.hip.h"
+#include "conv_norm.h"
+
+namespace {
+
+__device__ __forceinline__ float bf16_at(const uint16_t* p, uint64_t i) { return __builtin_bit_cast(float, static_cast<uint32_t>(p[i]) << 16); }
+
+__global__ __launch_bounds__(256) void embed_pos_kernel(const uint16_t* __restrict__ embed, const uint16_t* __restrict__ pos,
+                                                        const uint32_t* __restrict__ tokens, uint32_t token, uint32_t start,
+                                                        uint32_t width, uint64_t ld, float* __restrict__ x, float* __restrict__ x0) {
+    const uint32_t t = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
+    if (c >= ld) return;
+    const uint64_t tok = tokens ? tokens[t] : token;
+    const float v = c < width ? bf16_at(embed, tok * width + c) + bf16_at(pos, static_cast<uint64_t>(start + t) * width + c) : 0.0f;
+    x[t * ld + c] = v;
+    x0[t * ld + c] = v;
+}
+
+// Eight rows per workgroup: first 1 / rms of those rows and of the taps - 1 before them (recomputed, so
+// that workgroups need nothing from each other), then the channels, four per thread.
+constexpr int ROWS = 8;
+template <typename T>
+__global__ __launch_bounds__(256) void norm_conv_kernel(NormConv a) {
+    __shared__ float inv[ROWS + CONV_MAX_TAPS];
+    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int back = a.taps ? static_cast<int>(a.taps) - 1 : 0, t0 = static_cast<int>(blockIdx.x) * ROWS;
+    const int t_end = min(t0 + ROWS, static_cast<int>(a.n));
+    for (int t = t0 - back + static_cast<int>(wave); t < t_end; t += 4) {
+        if (t < 0) continue;
+        const float* const row = a.x + static_cast<uint64_t>(t) * a.ld;
+        float ss = 0.0f;
+        for (uint32_t c = lane * 4; c < a.ld; c += 256) {
+            const float4 v = *reinterpret_cast<const float4*>(row + c);
+            ss = fmaf(v.x, v.x, ss); ss = fmaf(v.y, v.y, ss); ss = fmaf(v.z, v.z, ss); ss = fmaf(v.w, v.w, ss);
+        }
+        ss = wave_sum(ss);
+        const float r = 1.0f / sqrtf(ss / static_cast<float>(a.width) + a.eps);
+        if (lane == 0) {
+            inv[t - t0 + back] = r;
+            if (a.inv && t >= t0) a.inv[t] = r;
+        }
+    }
+    __syncthreads();
+    for (uint32_t c = (blockIdx.y * 256 + threadIdx.x) * 4; c < a.ld; c += gridDim.y * 1024) {
+        const float4 w = *reinterpret_cast<const float4*>(a.w + c);
+        auto h_at = [&](int t) -> float4 {
+            if (t < 0) {
+                const int64_t p = static_cast<int64_t>(a.start) + t;
+                if (p < 0) return make_float4(0.f, 0.f, 0.f, 0.f);
+                return *reinterpret_cast<const float4*>(a.ring.rows + static_cast<uint64_t>(p & (a.ring.depth - 1)) * a.ring.ld + c);
+            }
+            const float4 v = *reinterpret_cast<const float4*>(a.x + static_cast<uint64_t>(t) * a.ld + c);
+            const float s = inv[t - t0 + back];
+            return make_float4(v.x * s * w.x, v.y * s * w.y, v.z * s * w.z, v.w * s * w.w);
+        };
+        for (int t = t0; t < t_end; ++t) {
+            const float4 h = h_at(t);
+            float4 ya = h, yb = h;
+            for (int j = 0; j < static_cast<int>(a.taps); ++j) {
+                const float4 g = j == back ? h : h_at(t - back + j);
+                const float4 ka = *reinterpret_cast<const float4*>(a.wa + static_cast<uint64_t>(j) * a.ld + c);
+                ya.x = fmaf(ka.x, g.x, ya.x); ya.y = fmaf(ka.y, g.y, ya.y); ya.z = fmaf(ka.z, g.z, ya.z); ya.w = fmaf(ka.w, g.w, ya.w);
+                if (a.wb) {
+                    const float4 kb = *reinterpret_cast<const float4*>(a.wb + static_cast<uint64_t>(j) * a.ld + c);
+                    yb.x = fmaf(kb.x, g.x, yb.x); yb.y = fmaf(kb.y, g.y, yb.y); yb.z = fmaf(kb.z, g.z, yb.z); yb.w = fmaf(kb.w, g.w, yb.w);
+                }
+            }
+            const uint64_t at = static_cast<uint64_t>(t) * a.ld + c;
+            ElemOps<T>::store4(static_cast<T*>(a.out_a) + at, ya.x, ya.y, ya.z, ya.w);
+            if (a.out_b) ElemOps<T>::store4(static_cast<T*>(a.out_b) + at, yb.x, yb.y, yb.z, yb.w);
+        }
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void concat2_kernel(const float* __restrict__ a, const float* __restrict__ b, uint64_t ld, T* __restrict__ out) {
+    const uint64_t c = (static_cast<uint64_t>(blockIdx.x) * 256 + threadIdx.x) * 4, t = blockIdx.y;
+    if (c >= 2 * ld) return;
+    const float4 v = *reinterpret_cast<const float4*>(c < ld ? a + t * ld + c : b + t * ld + (c - ld));
+    ElemOps<T>::store4(out + t * 2 * ld + c, v.x, v.y, v.z, v.w);
+}
+
+}  // namespace
+
+cera_hip_status cera_launch_embed_pos(cera_hip_ctx* ctx, const void* embed, const void* pos, const uint32_t* tokens, uint32_t token,
+                                      uint32_t n, uint32_t start, uint32_t width, uint64_t ld, float* x, float* x0) {
+    hipLaunchKernelGGL(embed_pos_kernel, dim3(static_cast<uint32_t>((ld + 255) / 256), n), dim3(256), 0, ctx->stream,
+                       static_cast<const uint16_t*>(embed), static_cast<const uint16_t*>(pos), tokens, token, start, width, ld, x, x0);
+    HIP_TRY(ctx, hipGetLastError());
+    return CERA_HIP_OK;
+}
+
+cera_hip_status cera_launch_norm_conv(cera_hip_ctx* ctx, const NormConv& a, bool f32) {
+    if (a.ld % 4 || a.taps > CONV_MAX_TAPS || (a.taps > 1 && (!a.ring.rows || a.ring.depth < a.taps)) || (a.out_b && !a.wb && a.taps))
+        return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "norm_conv: bad shape");
+    const uint32_t groups = (a.n + ROWS - 1) / ROWS;
+    // few rows: the channels are spread over workgroups as well (each recomputes its rows' norms)
+    const uint32_t cols = static_cast<uint32_t>((a.ld + 1023) / 1024);
+    const dim3 grid(groups, groups * cols <= 4 * ctx->n_cu ? cols : 1);
+    if (f32) hipLaunchKernelGGL(norm_conv_kernel<float>, grid, dim3(256), 0, ctx->stream, a);
+    else hipLaunchKernelGGL(norm_conv_kernel<__bf16>, grid, dim3(256), 0, ctx->stream, a);
+    HIP_TRY(ctx, hipGetLastError());
+    return CERA_HIP_OK;
+}
+
+cera_hip_status cera_launch_concat2(cera_hip_ctx* ctx, const float* a, const float* b, uint32_t n, uint64_t ld, void* out, bool f32) {
+    const dim3 grid(static_cast<uint32_t>((2 * ld / 4 + 255) / 256), n);
+    if (f32) hipLaunchKernelGGL(concat2_kernel<float>, grid, dim3(256), 0, ctx->stream, a, b, ld, static_cast<float*>(out));
+    else hipLaunchKernelGGL(concat2_kernel<__bf16>, grid, dim3(256), 0, ctx->stream, a, b, ld, static_cast<__bf16*>(out));
+    HIP_TRY(ctx, hipGetLastError());
+    return CERA_HIP_OK;
+}

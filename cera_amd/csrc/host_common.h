@@ -75,6 +75,8 @@ cera_hip_status cera_fail(cera_hip_ctx* ctx, cera_hip_status st, const std::stri
 
 // element / byte geometry of a GGML type; false when there is no kernel for it
 bool cera_type_geometry(uint32_t t, uint32_t* block_elems, uint32_t* block_bytes);
+// type, shape and byte count of a caller's tensor; *row_bytes: bytes of one row
+cera_hip_status cera_check_tensor(cera_hip_ctx* ctx, const cera_hip_tensor* t, uint64_t* row_bytes);
 cera_hip_status cera_scratch(cera_hip_ctx* ctx, int slot, uint64_t nbytes, void** out);
 // kernel `name` of the context's loaded code object, nullptr when there is no module or no such kernel
 hipFunction_t cera_module_fn(cera_hip_ctx* ctx, const std::string& name);

@@ -17,8 +17,28 @@ struct LayerDev {
     void *kc = nullptr, *vc = nullptr;  // [n_kv_heads][max_seq_len][head_dim], f32 or half (model->kv_f16)
 };
 
+// What a model family does for the model-level entry points (model_api.hip).  The caller holds the
+// model's locks and has checked tokens and positions.
+struct CeraModelOps {
+    // one token at `pos`; its logits are left in m->logits when wanted.  The caller advances seq_len.
+    cera_hip_status (*decode)(cera_hip_model* m, uint32_t token, uint32_t pos, bool want_logits);
+    // n tokens from start_pos on, advancing m->seq_len; logits (host) of the last / of every position
+    cera_hip_status (*prefill)(cera_hip_model* m, const uint32_t* tokens, uint32_t n, uint32_t start_pos, float* last_logits);
+    cera_hip_status (*prefill_all)(cera_hip_model* m, const uint32_t* tokens, uint32_t n, uint32_t start_pos, float* logits_all);
+    // fails when the state at `len` is gone (nullable: every shorter length can be taken up again)
+    cera_hip_status (*truncate)(cera_hip_model* m, uint32_t len);
+    cera_hip_status (*read_kv)(cera_hip_model* m, uint32_t layer, float* k_out, float* v_out);
+    cera_hip_status (*write_kv)(cera_hip_model* m, uint32_t layer, const float* k, const float* v, uint32_t n_pos);
+    // convolution state of a layer (nullable: the family has none)
+    cera_hip_status (*read_conv)(cera_hip_model* m, uint32_t layer, float* rows);
+    cera_hip_status (*write_conv)(cera_hip_model* m, uint32_t layer, const float* rows, uint32_t n_pos);
+    void (*destroy)(cera_hip_model* m);
+};
+
 struct cera_hip_model {
     cera_hip_ctx* ctx = nullptr;
+    const CeraModelOps* ops = nullptr;
+    struct CeraLayered* layered = nullptr;   // the layered family's state (layered.h); the llama fields below are then unused
     cera_hip_config cfg{};
     cera_hip_dtensor *embd = nullptr, *output = nullptr;
     float* output_norm = nullptr;

@@ -15,6 +15,9 @@
 #include "host_common.h"
 #include "model.h"
 
+// the entry points of this file that only a llama has
+static cera_hip_status llama_only(cera_hip_model* m, const char* what);
+
 // ---------------------------------------------------------------------------
 static cera_hip_status dev_alloc(cera_hip_ctx* ctx, uint64_t bytes, void** out, uint64_t* total) {
     *out = nullptr;
@@ -147,6 +150,11 @@ static void free_model(cera_hip_model* m) {
     delete m;
 }
 
+static const CeraModelOps* llama_ops();
+static cera_hip_status llama_only(cera_hip_model* m, const char* what) {
+    if (m->ops == llama_ops()) return CERA_HIP_OK;
+    return cera_fail(m->ctx, CERA_HIP_ERR_ARGUMENT, std::string(what) + ": not available for this model family");
+}
 static bool gemv_type_ok(uint32_t t) {
     return t == CERA_HIP_Q4_0 || t == CERA_HIP_Q4_1 || t == CERA_HIP_Q8_0 || t == CERA_HIP_Q4_K ||
            t == CERA_HIP_Q5_K || t == CERA_HIP_Q6_K;
@@ -211,6 +219,7 @@ extern "C" cera_hip_status cera_hip_model_create(cera_hip_ctx* ctx, const cera_h
     cera_hip_model* m = new (std::nothrow) cera_hip_model();
     if (!m) return cera_fail(ctx, CERA_HIP_ERR_OOM, "host allocation failed");
     m->ctx = ctx;
+    m->ops = llama_ops();
     m->cfg = c;
     m->cfg.rope_freqs = nullptr;
     m->layers.resize(c.n_layers);
@@ -307,7 +316,6 @@ extern "C" cera_hip_status cera_hip_model_create(cera_hip_ctx* ctx, const cera_h
     return CERA_HIP_OK;
 }
 
-extern "C" void cera_hip_model_destroy(cera_hip_model* m) { free_model(m); }
 extern "C" uint64_t cera_hip_decode_copy_reserve_bytes(const cera_hip_config* cfg) { return cfg ? cera_copy_reserve_bytes(*cfg) : 0; }
 extern "C" uint64_t cera_hip_decode_copy_plan(const uint64_t* copy_bytes, uint32_t n, uint64_t free_bytes, uint64_t reserve_bytes,
                                               uint8_t* take) {
@@ -316,26 +324,18 @@ extern "C" uint64_t cera_hip_decode_copy_plan(const uint64_t* copy_bytes, uint32
 extern "C" cera_hip_status cera_hip_drop_decode_copies(cera_hip_model* m, uint64_t* freed_bytes) {
     if (!m) return CERA_HIP_ERR_ARGUMENT;
     ModelLock lk(m);
+    CERA_TRY(llama_only(m, "drop_decode_copies"));
     const uint64_t f = cera_model_drop_decode_copies(m);
     if (freed_bytes) *freed_bytes = f;
     return CERA_HIP_OK;
 }
-extern "C" uint32_t cera_hip_seq_len(const cera_hip_model* m) { return m ? m->seq_len : 0; }
-extern "C" uint64_t cera_hip_memory_bytes(const cera_hip_model* m) { return m ? m->bytes : 0; }
-
-extern "C" cera_hip_status cera_hip_truncate_kv(cera_hip_model* m, uint32_t len) {
-    if (!m) return CERA_HIP_ERR_ARGUMENT;
-    ModelLock lk(m);
-    if (len < m->seq_len) m->seq_len = len;  // rows past len are simply overwritten later
-    return CERA_HIP_OK;
-}
-
 // LlamaModel::shift_kv -> InferenceState::shift_kv_with_rope (cera/src/model/llama.rs:1727-1738,
 // cera/src/kv_cache.rs:1091-1310): drop cache cells [n_keep, n_keep + shift), move the tail down
 // and re-rotate its K rows by R(-shift) so their encoded position matches their new index.
 extern "C" cera_hip_status cera_hip_shift_kv(cera_hip_model* m, uint32_t n_keep, uint32_t shift) {
     if (!m) return CERA_HIP_ERR_ARGUMENT;
     ModelLock lk(m);
+    CERA_TRY(llama_only(m, "shift_kv"));
     cera_hip_ctx* ctx = m->ctx;
     const cera_hip_config& c = m->cfg;
     if (shift == 0) return cera_fail(ctx, CERA_HIP_ERR_ARGUMENT, "shift_kv: shift must be > 0");
@@ -409,47 +409,6 @@ extern "C" cera_hip_status cera_hip_shift_kv(cera_hip_model* m, uint32_t n_keep,
     return CERA_HIP_OK;
 }
 
-// Prefix-cache snapshots (Model::snapshot_state / restore_state, cera/src/model/mod.rs:507-533;
-// layer layout LayerSnapshot::Attention, cera/src/kv_cache.rs:1382-1396): a layer's K and V as
-// time-major [n_pos][kv_dim] f32, the CPU state's own layout.  cera_hip_read_kv is the snapshot
-// side; this is the restore side.  Call it for every layer, then cera_hip_set_seq_len.
-extern "C" cera_hip_status cera_hip_write_kv(cera_hip_model* m, uint32_t layer, const float* k, const float* v,
-                                             uint32_t n_pos) {
-    if (!m || (n_pos && (!k || !v)) || layer >= m->cfg.n_layers) return CERA_HIP_ERR_ARGUMENT;
-    ModelLock lk(m);
-    const cera_hip_config& c = m->cfg;
-    if (n_pos > c.max_seq_len) return cera_fail(m->ctx, CERA_HIP_ERR_POSITION, "write_kv: more positions than max_seq_len");
-    const uint64_t per_head = static_cast<uint64_t>(c.max_seq_len) * c.head_dim;
-    const uint64_t kv_dim = static_cast<uint64_t>(c.n_kv_heads) * c.head_dim;
-    std::vector<float> hk(static_cast<uint64_t>(n_pos) * c.head_dim), hv(hk.size());
-    std::vector<kv_half> h16;
-    const uint64_t esz = m->kv_f16 ? sizeof(kv_half) : sizeof(float);
-    auto put = [&](void* cache, uint32_t h, const std::vector<float>& rows) -> cera_hip_status {
-        char* dst = static_cast<char*>(cache) + h * per_head * esz;
-        if (!m->kv_f16) return cera_hip_upload(m->ctx, dst, rows.data(), rows.size() * 4);
-        h16.resize(rows.size());
-        for (size_t i = 0; i < rows.size(); ++i) h16[i] = static_cast<kv_half>(rows[i]);   // round to nearest even
-        return cera_hip_upload(m->ctx, dst, h16.data(), h16.size() * sizeof(kv_half));
-    };
-    for (uint32_t h = 0; h < c.n_kv_heads && n_pos; ++h) {
-        for (uint32_t t = 0; t < n_pos; ++t) {
-            std::memcpy(hk.data() + static_cast<uint64_t>(t) * c.head_dim, k + t * kv_dim + h * c.head_dim, c.head_dim * 4);
-            std::memcpy(hv.data() + static_cast<uint64_t>(t) * c.head_dim, v + t * kv_dim + h * c.head_dim, c.head_dim * 4);
-        }
-        CERA_TRY(put(m->layers[layer].kc, h, hk));
-        CERA_TRY(put(m->layers[layer].vc, h, hv));
-    }
-    return CERA_HIP_OK;
-}
-
-extern "C" cera_hip_status cera_hip_set_seq_len(cera_hip_model* m, uint32_t len) {
-    if (!m) return CERA_HIP_ERR_ARGUMENT;
-    ModelLock lk(m);
-    if (len > m->cfg.max_seq_len) return cera_fail(m->ctx, CERA_HIP_ERR_POSITION, "set_seq_len: beyond max_seq_len");
-    m->seq_len = len;
-    return CERA_HIP_OK;
-}
-
 // Model::configure_kv_compression for the modes this backend has (cera/src/model/mod.rs:557-592,
 // KvCompression::{None, F16}, cera/src/kv_cache.rs:88-98): called before the first forward pass;
 // the first call wins, the same mode again is a no-op, a different one a conflict.  Switching
@@ -457,6 +416,7 @@ extern "C" cera_hip_status cera_hip_set_seq_len(cera_hip_model* m, uint32_t len)
 extern "C" cera_hip_status cera_hip_configure_kv(cera_hip_model* m, uint32_t kv_type) {
     if (!m) return CERA_HIP_ERR_ARGUMENT;
     ModelLock lk(m);
+    CERA_TRY(llama_only(m, "configure_kv"));
     cera_hip_ctx* ctx = m->ctx;
     if (kv_type > CERA_HIP_KV_F16) return cera_fail(ctx, CERA_HIP_ERR_ARGUMENT, "configure_kv: unknown cache type");
     const bool want_f16 = kv_type == CERA_HIP_KV_F16;
@@ -493,6 +453,7 @@ extern "C" cera_hip_status cera_hip_configure_kv(cera_hip_model* m, uint32_t kv_
 extern "C" cera_hip_status cera_hip_set_reference_order(cera_hip_model* m, uint32_t on) {
     if (!m) return CERA_HIP_ERR_ARGUMENT;
     ModelLock lk(m);
+    CERA_TRY(llama_only(m, "set_reference_order"));
     if (m->seq_len != 0) return cera_fail(m->ctx, CERA_HIP_ERR_POSITION, "set_reference_order: the cache already holds positions");
     std::string why;
     if (on && !cera_model_ref_order_supported(m, &why))
@@ -694,27 +655,6 @@ static cera_hip_status decode_step(cera_hip_model* m, uint32_t token, uint32_t p
     return CERA_HIP_OK;
 }
 
-// A call at position 0 starts a fresh sequence: callers hand a new InferenceState to every
-// generate(), and a device-resident backend resets its own counter then, as the reference's do
-// (cera/src/model/metal_lfm2.rs:4091-4096, gpu_lfm2.rs:3755-3762).  Cached rows are simply
-// overwritten.
-static cera_hip_status begin_at(cera_hip_model* m, uint32_t pos) {
-    if (m->kv_broken) return cera_fail(m->ctx, CERA_HIP_ERR_DEVICE, "the model's KV cache is unusable (a cache re-allocation failed)");
-    if (pos == 0) m->seq_len = 0;
-    return CERA_HIP_OK;
-}
-
-static cera_hip_status check_step(cera_hip_model* m, uint32_t token, uint32_t pos) {
-    CERA_TRY(begin_at(m, pos));
-    if (token >= m->cfg.vocab)
-        return cera_fail(m->ctx, CERA_HIP_ERR_ARGUMENT, "token id " + std::to_string(token) + " out of range (vocab " + std::to_string(m->cfg.vocab) + ")");
-    if (pos != m->seq_len)
-        return cera_fail(m->ctx, CERA_HIP_ERR_POSITION, "pos " + std::to_string(pos) + " != seq_len " + std::to_string(m->seq_len));
-    if (pos >= m->cfg.max_seq_len)
-        return cera_fail(m->ctx, CERA_HIP_ERR_POSITION, "context full: pos " + std::to_string(pos) + " >= max_seq_len " + std::to_string(m->cfg.max_seq_len));
-    return CERA_HIP_OK;
-}
-
 // Kernel arguments are captured at launch, so (unlike an async copy from a
 // stack variable) the values cannot change under a launch that is still queued.
 static __global__ void set_token_pos_kernel(uint32_t* scalars, uint32_t token, uint32_t pos) {
@@ -725,63 +665,6 @@ static cera_hip_status set_token_pos(cera_hip_model* m, uint32_t token, uint32_t
     hipLaunchKernelGGL(set_token_pos_kernel, dim3(1), dim3(1), 0, m->ctx->stream, m->scalars, token, pos);
     HIP_TRY(m->ctx, hipGetLastError());
     return CERA_HIP_OK;
-}
-
-extern "C" cera_hip_status cera_hip_forward(cera_hip_model* m, uint32_t token, uint32_t pos, float* logits) {
-    if (!m || !logits) return CERA_HIP_ERR_ARGUMENT;
-    ModelLock lk(m);
-    CERA_TRY(check_step(m, token, pos));
-    CERA_TRY(decode_step(m, token, pos, true));
-    CERA_TRY(cera_hip_download(m->ctx, logits, m->logits, static_cast<uint64_t>(m->cfg.vocab) * 4));
-    m->seq_len = pos + 1;
-    return CERA_HIP_OK;
-}
-
-extern "C" cera_hip_status cera_hip_forward_greedy(cera_hip_model* m, uint32_t token, uint32_t pos, uint32_t* next) {
-    if (!m || !next) return CERA_HIP_ERR_ARGUMENT;
-    ModelLock lk(m);
-    CERA_TRY(check_step(m, token, pos));
-    CERA_TRY(decode_step(m, token, pos, true));
-    // the argmax kernel writes the token into pinned host memory itself: no copy launch behind it
-    uint32_t *word_host, *word_dev;
-    CERA_TRY(cera_pinned_word(m->ctx, &word_host, &word_dev));
-    CERA_TRY(cera_launch_argmax(m->ctx, m->logits, m->cfg.vocab, m->scalars + 2, word_dev));
-    HIP_TRY(m->ctx, hipStreamSynchronize(m->ctx->stream));
-    *next = *static_cast<volatile uint32_t*>(word_host);
-    m->seq_len = pos + 1;
-    return CERA_HIP_OK;
-}
-
-extern "C" cera_hip_status cera_hip_forward_prefill(cera_hip_model* m, const uint32_t* tokens, uint32_t n,
-                                                    uint32_t start_pos, float* last_logits) {
-    if (!m || !tokens || !last_logits) return CERA_HIP_ERR_ARGUMENT;
-    if (n == 0) return cera_fail(m->ctx, CERA_HIP_ERR_ARGUMENT, "forward_prefill requires at least one token");
-    ModelLock lk(m);
-    CERA_TRY(begin_at(m, start_pos));
-    if (start_pos != m->seq_len)
-        return cera_fail(m->ctx, CERA_HIP_ERR_POSITION, "forward_prefill: start_pos " + std::to_string(start_pos) +
-                                                            " must equal seq_len " + std::to_string(m->seq_len));
-    if (static_cast<uint64_t>(start_pos) + n > m->cfg.max_seq_len)
-        return cera_fail(m->ctx, CERA_HIP_ERR_POSITION, "forward_prefill: prompt does not fit max_seq_len");
-    for (uint32_t i = 0; i < n; ++i)
-        if (tokens[i] >= m->cfg.vocab) return cera_fail(m->ctx, CERA_HIP_ERR_ARGUMENT, "token id out of range");
-    return cera_model_prefill(m, tokens, n, start_pos, last_logits);
-}
-
-extern "C" cera_hip_status cera_hip_forward_prefill_logits_all(cera_hip_model* m, const uint32_t* tokens, uint32_t n,
-                                                               uint32_t start_pos, float* logits_all) {
-    if (!m || !tokens || !logits_all) return CERA_HIP_ERR_ARGUMENT;
-    if (n == 0) return cera_fail(m->ctx, CERA_HIP_ERR_ARGUMENT, "forward_prefill_logits_all requires at least one token");
-    ModelLock lk(m);
-    CERA_TRY(begin_at(m, start_pos));
-    if (start_pos != m->seq_len)
-        return cera_fail(m->ctx, CERA_HIP_ERR_POSITION, "forward_prefill_logits_all: start_pos " + std::to_string(start_pos) +
-                                                            " must equal seq_len " + std::to_string(m->seq_len));
-    if (static_cast<uint64_t>(start_pos) + n > m->cfg.max_seq_len)
-        return cera_fail(m->ctx, CERA_HIP_ERR_POSITION, "forward_prefill_logits_all: tokens do not fit max_seq_len");
-    for (uint32_t i = 0; i < n; ++i)
-        if (tokens[i] >= m->cfg.vocab) return cera_fail(m->ctx, CERA_HIP_ERR_ARGUMENT, "token id out of range");
-    return cera_model_prefill_logits_all(m, tokens, n, start_pos, logits_all);
 }
 
 // one decode step with the logits copied out (the per-token route of the all-logits call)
@@ -803,9 +686,32 @@ cera_hip_status cera_model_prefill_per_token(cera_hip_model* m, const uint32_t* 
     return cera_hip_download(m->ctx, last_logits, m->logits, static_cast<uint64_t>(m->cfg.vocab) * 4);
 }
 
-extern "C" cera_hip_status cera_hip_read_kv(cera_hip_model* m, uint32_t layer, float* k_out, float* v_out) {
-    if (!m || !k_out || !v_out || layer >= m->cfg.n_layers) return CERA_HIP_ERR_ARGUMENT;
-    ModelLock lk(m);
+static cera_hip_status write_kv(cera_hip_model* m, uint32_t layer, const float* k, const float* v, uint32_t n_pos) {
+    const cera_hip_config& c = m->cfg;
+    const uint64_t per_head = static_cast<uint64_t>(c.max_seq_len) * c.head_dim;
+    const uint64_t kv_dim = static_cast<uint64_t>(c.n_kv_heads) * c.head_dim;
+    std::vector<float> hk(static_cast<uint64_t>(n_pos) * c.head_dim), hv(hk.size());
+    std::vector<kv_half> h16;
+    const uint64_t esz = m->kv_f16 ? sizeof(kv_half) : sizeof(float);
+    auto put = [&](void* cache, uint32_t h, const std::vector<float>& rows) -> cera_hip_status {
+        char* dst = static_cast<char*>(cache) + h * per_head * esz;
+        if (!m->kv_f16) return cera_hip_upload(m->ctx, dst, rows.data(), rows.size() * 4);
+        h16.resize(rows.size());
+        for (size_t i = 0; i < rows.size(); ++i) h16[i] = static_cast<kv_half>(rows[i]);   // round to nearest even
+        return cera_hip_upload(m->ctx, dst, h16.data(), h16.size() * sizeof(kv_half));
+    };
+    for (uint32_t h = 0; h < c.n_kv_heads && n_pos; ++h) {
+        for (uint32_t t = 0; t < n_pos; ++t) {
+            std::memcpy(hk.data() + static_cast<uint64_t>(t) * c.head_dim, k + t * kv_dim + h * c.head_dim, c.head_dim * 4);
+            std::memcpy(hv.data() + static_cast<uint64_t>(t) * c.head_dim, v + t * kv_dim + h * c.head_dim, c.head_dim * 4);
+        }
+        CERA_TRY(put(m->layers[layer].kc, h, hk));
+        CERA_TRY(put(m->layers[layer].vc, h, hv));
+    }
+    return CERA_HIP_OK;
+}
+
+static cera_hip_status read_kv(cera_hip_model* m, uint32_t layer, float* k_out, float* v_out) {
     const cera_hip_config& c = m->cfg;
     const uint64_t per_head = static_cast<uint64_t>(c.max_seq_len) * c.head_dim;
     std::vector<float> hk(static_cast<uint64_t>(m->seq_len) * c.head_dim), hv(hk.size());
@@ -832,10 +738,11 @@ extern "C" cera_hip_status cera_hip_read_kv(cera_hip_model* m, uint32_t layer, f
     return CERA_HIP_OK;
 }
 
-extern "C" cera_hip_status cera_hip_read_hidden(cera_hip_model* m, float* hidden_out) {
-    if (!m || !hidden_out) return CERA_HIP_ERR_ARGUMENT;
-    ModelLock lk(m);
-    return cera_hip_download(m->ctx, hidden_out, m->hidden, static_cast<uint64_t>(m->cfg.hidden) * 4);
+// what the model-level entry points (model_api.hip) call for a llama
+static const CeraModelOps* llama_ops() {
+    static const CeraModelOps ops = {decode_step, cera_model_prefill, cera_model_prefill_logits_all, nullptr, read_kv, write_kv,
+                                     nullptr, nullptr, free_model};
+    return &ops;
 }
 
 // cpu::rope / cpu::rope_norm on host buffers (test entry point).

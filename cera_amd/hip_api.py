@@ -35,6 +35,7 @@ SYMBOLS = [
     "cera_hip_set_reference_order", "cera_hip_reference_order",
     "cera_hip_rmsnorm_q8_0", "cera_hip_attn_decode_step", "cera_hip_attn_decode_dev_noalloc", "cera_hip_gemm_block_dots",
     "cera_hip_ffn_gate_up_fused", "cera_hip_qkv_fused",
+    "cera_hip_layered_create", "cera_hip_read_conv", "cera_hip_write_conv",
 ]
 
 
@@ -65,6 +66,30 @@ class Config(C.Structure):
                 ("rope_theta", C.c_float), ("rms_eps", C.c_float), ("embed_scale", C.c_float),
                 ("residual_scale", C.c_float), ("attn_scale", C.c_float), ("logit_scale", C.c_float),
                 ("rope_freqs", C.c_void_p)]
+
+
+class AttnSpec(C.Structure):
+    """cera_hip_attn_spec."""
+    _fields_ = [("heads", C.c_uint32), ("kv_heads", C.c_uint32), ("dim", C.c_uint32), ("vdim", C.c_uint32),
+                ("scale", C.c_float), ("chunk", C.c_uint32), ("rot_dims", C.c_uint32), ("yarn", C.c_uint32),
+                ("rot_base", C.c_double), ("yarn_factor", C.c_double), ("yarn_original", C.c_double),
+                ("yarn_fast", C.c_double), ("yarn_slow", C.c_double)]
+
+
+class LayeredLayer(C.Structure):
+    """cera_hip_layered_layer."""
+    _fields_ = [("attn", AttnSpec), ("ff", C.c_uint32), ("_reserved", C.c_uint32), ("norm", C.c_void_p),
+                ("conv_attn", C.c_void_p), ("conv_ffn", C.c_void_p), ("score_bias", C.c_void_p)] + \
+               [(n, Tensor) for n in ("q", "k", "v", "head_gate", "o", "ffn_gate", "ffn_up", "ffn_down")]
+
+
+class LayeredConfig(C.Structure):
+    """cera_hip_layered_config."""
+    _fields_ = [(n, C.c_uint32) for n in ("n_layers", "width", "vocab", "max_seq_len", "conv_taps", "loop_start",
+                                          "loop_stop", "loop_times")] + \
+               [("eps", C.c_float), ("residual_mult", C.c_float), ("f32", C.c_uint32), ("_reserved", C.c_uint32)] + \
+               [(n, Tensor) for n in ("embed", "pos", "head", "loop_in")] + \
+               [("loop_step", C.c_void_p), ("final_norm", C.c_void_p)]
 
 
 class GemvOp(C.Structure):
@@ -158,6 +183,8 @@ def load_library() -> C.CDLL:
         "cera_hip_ffn_gate_up_fused": (i32, [vp, vp, vp, vp, vp, f32, vp, vp]),
         "cera_hip_qkv_fused": (i32, [vp, vp, vp, vp, vp, f32, vp, vp]),
         "cera_hip_gemm_block_dots": (i32, [vp, C.POINTER(Tensor), vp, u64, vp, vp]),
+        "cera_hip_layered_create": (i32, [vp, C.POINTER(LayeredConfig), C.POINTER(LayeredLayer), pp]),
+        "cera_hip_read_conv": (i32, [vp, u32, vp]), "cera_hip_write_conv": (i32, [vp, u32, vp, u32]),
         "cera_hip_rmsnorm_q8_0": (i32, [vp, vp, vp, u64, f32, vp, vp, vp]),
         "cera_hip_attn_decode_step": (i32, [vp, vp, vp, vp, vp, vp, u32, u32, u32, u32, f32, u32, vp, f32, u32,
                                             vp, vp, vp, vp, vp]),
@@ -702,3 +729,50 @@ class Model:
         if getattr(self, "h", None):
             self.ctx.lib.cera_hip_model_destroy(self.h)
             self.h = None
+
+
+class LayeredModel(Model):
+    """cera_hip_layered_create over arrays: ``cfg`` as a Nafevik config.json, ``weights`` by tensor name --
+    uint16 bf16 bits [out, in] for matrices, float32 for vectors."""
+
+    def __init__(self, ctx: Context, cfg: dict, weights: dict, max_seq_len: int, f32: bool = False):
+        self.ctx, self.cfg = ctx, dict(cfg)
+        keep = []
+
+        def mat(name):
+            a = weights[name]
+            assert a.dtype == np.uint16 and a.flags["C_CONTIGUOUS"], name
+            return Tensor(BF16, 0, a.shape[0], a.shape[1], a.ctypes.data, a.nbytes)
+
+        def vec(name):
+            a = np.ascontiguousarray(weights[name], np.float32)
+            keep.append(a)
+            return a.ctypes.data
+
+        c = LayeredConfig(len(cfg["layers"]), cfg["width"], cfg["vocab"], max_seq_len, cfg["canon"]["taps"])
+        c.eps, c.residual_mult, c.f32 = cfg["norm"]["eps"], cfg["residual_mult"], int(f32)
+        c.embed, c.pos, c.head, c.final_norm = mat("embed"), mat("pos"), mat("head"), vec("final.norm")
+        if cfg.get("loop"):
+            c.loop_start, c.loop_stop, c.loop_times = (cfg["loop"][k] for k in ("start", "stop", "times"))
+            c.loop_in, c.loop_step = mat("loop.in"), vec("loop.step")
+        layers = (LayeredLayer * c.n_layers)()
+        for i, spec in enumerate(cfg["layers"]):
+            Y, p, m = layers[i], f"l{i}.", spec["mixer"]
+            a = Y.attn
+            a.heads, a.kv_heads, a.dim, a.vdim, a.scale = m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["scale"]
+            a.chunk = (m.get("mask") or {}).get("size", 0)
+            rot = m.get("rot")
+            if rot:
+                a.rot_dims, a.rot_base = rot["dims"], rot["base"]
+                if rot.get("scaling"):
+                    a.yarn = 1
+                    for k in ("factor", "original", "fast", "slow"):
+                        setattr(a, "yarn_" + k, rot["scaling"][k])
+            Y.norm, Y.conv_attn, Y.score_bias = vec(p + "norm1"), vec(p + "canon1"), vec(p + "mix.pb")
+            Y.q, Y.k, Y.v, Y.head_gate, Y.o = (mat(p + "mix." + n) for n in ("q", "k", "v", "g", "o"))
+            if spec.get("mlp"):
+                Y.ff, Y.conv_ffn = spec["mlp"]["ff"], vec(p + "canon2")
+                Y.ffn_gate, Y.ffn_up, Y.ffn_down = (mat(p + "mlp." + n) for n in ("gate", "up", "down"))
+        h = C.c_void_p()
+        ctx.check(ctx.lib.cera_hip_layered_create(ctx.h, C.byref(c), layers, C.byref(h)))
+        self.h, self.vocab, self.hidden = h, c.vocab, c.width

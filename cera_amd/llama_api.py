@@ -11,7 +11,7 @@ import numpy as np
 
 from . import _build
 
-LLAMA_SYMBOLS = ["cera_llama_open", "cera_llama_close", "cera_llama_last_error", "cera_llama_get_config",
+LLAMA_SYMBOLS = ["cera_llama_open", "cera_llama_open_dtype", "cera_llama_close", "cera_llama_last_error", "cera_llama_get_config",
                  "cera_llama_seq_len", "cera_llama_gpu_memory_bytes", "cera_llama_forward",
                  "cera_llama_forward_greedy", "cera_llama_forward_prefill", "cera_llama_forward_prefill_logits_all", "cera_llama_forward_prefill_chunked",
                  "cera_llama_set_cancel", "cera_llama_truncate_kv", "cera_llama_supports_kv_shift", "cera_llama_f16_kv_supported", "cera_llama_configure_kv_compression", "cera_llama_shift_kv",
@@ -38,6 +38,7 @@ def lib() -> C.CDLL:
         vp, cp, u64, u32 = C.c_void_p, C.c_char_p, C.c_uint64, C.c_uint32
         sig = {
             "cera_llama_open": (vp, [cp, u64, C.c_int, cp, u64]),
+            "cera_llama_open_dtype": (vp, [cp, u64, C.c_int, C.c_int, cp, u64]),
             "cera_llama_close": (None, [vp]),
             "cera_llama_last_error": (cp, [vp]),
             "cera_llama_get_config": (C.c_int, [vp, C.POINTER(LlamaConfigC)]),
@@ -100,9 +101,10 @@ class Snapshot:
 class HipLlama:
     """One loaded model + its InferenceState (position counter) + cancel flag."""
 
-    def __init__(self, gguf_path: str, context_size: int = 1024, device: int = 0):
+    def __init__(self, path: str, context_size: int = 1024, device: int = 0, f32: bool = False):
+        """``path``: a GGUF file, or a directory with config.json + model.safetensors (``f32`` is for the latter)."""
         err = C.create_string_buffer(1024)
-        self.h = lib().cera_llama_open(str(gguf_path).encode(), context_size, device, err, 1024)
+        self.h = lib().cera_llama_open_dtype(str(path).encode(), context_size, device, int(f32), err, 1024)
         if not self.h:
             raise BackendError(err.value.decode())
         c = LlamaConfigC()

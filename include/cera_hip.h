@@ -469,6 +469,51 @@ CERA_HIP_API cera_hip_status cera_hip_model_create(cera_hip_ctx*, const cera_hip
                                                    const cera_hip_tensor* output /* nullable => tied */,
                                                    const float* output_norm, const cera_hip_layer* layers,
                                                    cera_hip_model** out);
+/* ---- layered float models -------------------------------------------------
+ * A decoder described layer by layer: bfloat16 weights, RMS norms, one norm per layer read by an
+ * attention mixer and a feed-forward side by side (x += residual_mult * (mixer + feed-forward)),
+ * each reading its input through a short causal convolution; attention with unnormalised sigmoid
+ * weights inside chunks of positions and a gate per head; learned position vectors; a range of layers
+ * that runs several times over.  Every size and constant is a field.  The Nafevik architecture is
+ * one such model (its config.json reader is HipLayeredModel, cera_amd/backend/hip_layered.h).
+ * All the model-level calls below take the handle; those that only a llama has (configure_kv,
+ * shift_kv, set_reference_order, drop_decode_copies) fail with CERA_HIP_ERR_ARGUMENT. */
+typedef struct {
+    uint32_t heads, kv_heads, dim, vdim; /* dim: query / key size, vdim: value size; each at most 256 */
+    float scale;                         /* score = q . k * scale + score_bias[head] */
+    uint32_t chunk;                      /* positions per attention chunk; 0: the whole sequence */
+    uint32_t rot_dims;                   /* leading dimensions rotated in adjacent pairs; 0: none */
+    uint32_t yarn;                       /* 1: the frequencies are blended as below */
+    double rot_base;
+    double yarn_factor, yarn_original, yarn_fast, yarn_slow;
+} cera_hip_attn_spec;
+/* Matrices are bf16 tensors (ggml_type CERA_HIP_BF16), [m = outputs][k = inputs]; vectors f32. */
+typedef struct {
+    cera_hip_attn_spec attn;
+    uint32_t ff;                       /* feed-forward width; 0: the layer has none */
+    uint32_t _reserved;
+    const float* norm;                 /* [width] */
+    const float *conv_attn, *conv_ffn; /* [width][conv_taps]; the second null without a feed-forward */
+    const float* score_bias;           /* [heads] */
+    cera_hip_tensor q, k, v, head_gate, o;
+    cera_hip_tensor ffn_gate, ffn_up, ffn_down;
+} cera_hip_layered_layer;
+typedef struct {
+    uint32_t n_layers, width, vocab, max_seq_len;
+    uint32_t conv_taps;
+    uint32_t loop_start, loop_stop, loop_times; /* layers [start, stop) run `times` times in a row; times 0: no loop */
+    float eps, residual_mult;
+    uint32_t f32;                        /* 0: matrix products and activations in bf16; 1: everything in f32 */
+    uint32_t _reserved;
+    cera_hip_tensor embed, pos, head;    /* [vocab][width], [positions][width], [vocab][width] */
+    cera_hip_tensor loop_in;             /* [width][2 width]: reads the residual, then the embedding output */
+    const float* loop_step;              /* [loop_times][width], added after loop_in in each pass */
+    const float* final_norm;             /* [width] */
+} cera_hip_layered_config;
+/* Builds the model in HBM.  cera_hip_read_kv / _write_kv / _read_conv / _write_conv number its
+ * layers in execution order, every pass of the loop counted. */
+CERA_HIP_API cera_hip_status cera_hip_layered_create(cera_hip_ctx*, const cera_hip_layered_config*,
+                                                     const cera_hip_layered_layer* layers, cera_hip_model** out);
 CERA_HIP_API void cera_hip_model_destroy(cera_hip_model*);
 /* Model::forward (cera/src/model/mod.rs:200-606; LlamaModel::forward,
  * cera/src/model/llama.rs:1585-1605): one token at `pos` -> vocab logits.
@@ -548,6 +593,10 @@ CERA_HIP_API cera_hip_status cera_hip_read_kv(cera_hip_model*, uint32_t layer, f
  * which "sets internal seq_len" as the trait method does. */
 CERA_HIP_API cera_hip_status cera_hip_write_kv(cera_hip_model*, uint32_t layer, const float* k, const float* v,
                                                uint32_t n_pos);
+/* The convolution half of a layer's snapshot: the last conv_taps - 1 normalised rows [taps - 1][width],
+ * oldest first (zeros before the sequence's start).  No-ops for a family without convolutions. */
+CERA_HIP_API cera_hip_status cera_hip_read_conv(cera_hip_model*, uint32_t layer, float* rows);
+CERA_HIP_API cera_hip_status cera_hip_write_conv(cera_hip_model*, uint32_t layer, const float* rows, uint32_t n_pos);
 CERA_HIP_API cera_hip_status cera_hip_set_seq_len(cera_hip_model*, uint32_t len);
 /* Test hook: final normed hidden state of the last forward (f32[hidden]). */
 CERA_HIP_API cera_hip_status cera_hip_read_hidden(cera_hip_model*, float* hidden_out);

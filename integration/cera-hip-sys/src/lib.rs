@@ -89,6 +89,70 @@ pub struct cera_hip_tensor {
     pub nbytes: u64,
 }
 
+/// One layer's attention in a layered float model (sizes, score scale, chunked mask, rotation).
+#[repr(C)]
+#[derive(Clone, Copy, Debug)]
+pub struct cera_hip_attn_spec {
+    pub heads: u32,
+    pub kv_heads: u32,
+    pub dim: u32,
+    pub vdim: u32,
+    pub scale: f32,
+    pub chunk: u32,
+    pub rot_dims: u32,
+    pub yarn: u32,
+    pub rot_base: f64,
+    pub yarn_factor: f64,
+    pub yarn_original: f64,
+    pub yarn_fast: f64,
+    pub yarn_slow: f64,
+}
+
+/// Weights of one layer of a layered float model: bf16 matrices, `f32` vectors (host).
+#[repr(C)]
+#[derive(Clone, Copy, Debug)]
+pub struct cera_hip_layered_layer {
+    pub attn: cera_hip_attn_spec,
+    pub ff: u32,
+    pub _reserved: u32,
+    pub norm: *const f32,
+    pub conv_attn: *const f32,
+    pub conv_ffn: *const f32,
+    pub score_bias: *const f32,
+    pub q: cera_hip_tensor,
+    pub k: cera_hip_tensor,
+    pub v: cera_hip_tensor,
+    pub head_gate: cera_hip_tensor,
+    pub o: cera_hip_tensor,
+    pub ffn_gate: cera_hip_tensor,
+    pub ffn_up: cera_hip_tensor,
+    pub ffn_down: cera_hip_tensor,
+}
+
+/// A layered float model: sizes, loop, and the weights outside the layers.
+#[repr(C)]
+#[derive(Clone, Copy, Debug)]
+pub struct cera_hip_layered_config {
+    pub n_layers: u32,
+    pub width: u32,
+    pub vocab: u32,
+    pub max_seq_len: u32,
+    pub conv_taps: u32,
+    pub loop_start: u32,
+    pub loop_stop: u32,
+    pub loop_times: u32,
+    pub eps: f32,
+    pub residual_mult: f32,
+    pub f32: u32,
+    pub _reserved: u32,
+    pub embed: cera_hip_tensor,
+    pub pos: cera_hip_tensor,
+    pub head: cera_hip_tensor,
+    pub loop_in: cera_hip_tensor,
+    pub loop_step: *const f32,
+    pub final_norm: *const f32,
+}
+
 /// Per-layer weights. The norm / bias vectors are host `f32`; the optional ones are null when
 /// the architecture has none (biases: Qwen2, per-head QK norms: Qwen3).
 #[repr(C)]
@@ -636,6 +700,23 @@ pub fn cera_hip_ctx_create(
         k: *const f32,
         v: *const f32,
         n_pos: u32,
+    ) -> cera_hip_status;
+    pub fn cera_hip_read_conv(
+        model: *mut cera_hip_model,
+        layer: u32,
+        rows: *mut f32,
+    ) -> cera_hip_status;
+    pub fn cera_hip_write_conv(
+        model: *mut cera_hip_model,
+        layer: u32,
+        rows: *const f32,
+        n_pos: u32,
+    ) -> cera_hip_status;
+    pub fn cera_hip_layered_create(
+        ctx: *mut cera_hip_ctx,
+        cfg: *const cera_hip_layered_config,
+        layers: *const cera_hip_layered_layer,
+        out: *mut *mut cera_hip_model,
     ) -> cera_hip_status;
     pub fn cera_hip_set_seq_len(model: *mut cera_hip_model, len: u32) -> cera_hip_status;
     pub fn cera_hip_read_hidden(

@@ -72,7 +72,8 @@ def test_extern_block_matches_the_header():
 
 def test_struct_fields_match_the_header():
     src = re.sub(r"/\*.*?\*/", "", HEADER, flags=re.S)
-    for struct in ("cera_hip_tensor", "cera_hip_layer", "cera_hip_config", "cera_hip_gemv_op", "cera_hip_decode_op"):
+    for struct in ("cera_hip_tensor", "cera_hip_layer", "cera_hip_config", "cera_hip_gemv_op", "cera_hip_decode_op",
+                   "cera_hip_attn_spec", "cera_hip_layered_layer", "cera_hip_layered_config"):
         body = re.search(r"typedef struct \{([^}]*)\} " + struct + ";", src).group(1)
         c_fields = []
         for decl in body.split(";"):
@@ -144,7 +145,7 @@ def test_patch_touches_the_expected_files():
 
 def test_patch_applies_to_the_reference_tree():
     ref = Path("/root/reference")
-    if not ref.exists():
+    if not (ref / "cera").exists():
         pytest.skip("the reference tree is not present on this machine")
     n = 0
     for f, start, old in _hunks(PATCH):
