@@ -246,6 +246,98 @@ def measure_e2e(seed: int, n_thr: int):
             "all_logits_short_batch": short}
 
 
+# Layer sizes of `--design`: an 8B-, a 3B- and a 1B-class layer, eight of them.
+DESIGN_SIZES = {
+    "8b": dict(width=4096, ff=14336, heads=32, kv_heads=8, dim=128),
+    "3b": dict(width=3072, ff=8192, heads=24, kv_heads=8, dim=128),
+    "1b": dict(width=2048, ff=8192, heads=32, kv_heads=8, dim=64),
+}
+DESIGN_LAYERS, DESIGN_VOCAB, DESIGN_CTX = 8, 32000, 4096
+
+
+def nafevik_model(ctx, hip_api, size, rng, f32=False):
+    """A random-init Nafevik of DESIGN_LAYERS layers, the last six of them a loop run once (chunks of 2048,
+    four taps): (model, weight bytes a decode step reads).  The layers share host arrays, not HBM."""
+    W, FF, Hq, G, D = (size[k] for k in ("width", "ff", "heads", "kv_heads", "dim"))
+    def mat(m, k, sigma=0.02):
+        w = rng.standard_normal((m, k), dtype=np.float32) * np.float32(sigma)
+        return (w.view(np.uint32) >> 16).astype(np.uint16)
+    def vec(*shape):
+        return (0.1 * rng.standard_normal(shape)).astype(np.float32)
+    layer = {"norm1": 1 + vec(W), "canon1": vec(W, 4), "canon2": vec(W, 4), "mix.pb": vec(Hq) - 4, "mix.q": mat(Hq * D, W), "mix.k": mat(G * D, W),
+             "mix.v": mat(G * D, W), "mix.g": mat(Hq, W), "mix.o": mat(W, Hq * D), "mlp.gate": mat(FF, W), "mlp.up": mat(FF, W), "mlp.down": mat(W, FF)}
+    spec = {"type": "attention", "mlp": {"kind": "dense", "ff": FF},
+            "mixer": {"heads": Hq, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": 2048},
+                      "rot": {"dims": D, "base": 50000.0, "scaling": {"factor": 8.0, "original": 1024, "fast": 32.0, "slow": 1.0}}}}
+    cfg = {"width": W, "vocab": DESIGN_VOCAB, "canon": {"taps": 4}, "norm": {"eps": 1e-6}, "residual_mult": 0.7, "max_positions": DESIGN_CTX,
+           "layers": [spec] * DESIGN_LAYERS, "loop": {"start": 2, "stop": DESIGN_LAYERS, "times": 1}}
+    weights = {f"l{i}.{k}": v for i in range(DESIGN_LAYERS) for k, v in layer.items()}
+    weights.update({"embed": mat(DESIGN_VOCAB, W, 1.0), "pos": mat(DESIGN_CTX, W), "head": mat(DESIGN_VOCAB, W), "final.norm": 1 + vec(W),
+                    "loop.in": mat(W, 2 * W), "loop.step": vec(1, W)})
+    nbytes = DESIGN_LAYERS * sum(v.nbytes for v in layer.values() if v.dtype == np.uint16) + weights["head"].nbytes + weights["loop.in"].nbytes
+    return hip_api.LayeredModel(ctx, cfg, weights, DESIGN_CTX, f32), nbytes
+
+
+def llama_model(ctx, hip_api, H, size, quant, seed, n_thr):
+    """The llama of the same layer sizes in a GGUF type mix."""
+    from cera_amd import synth
+    cfg = dict(n_layers=1, hidden=size["width"], ffn=size["ff"], n_heads=size["heads"], n_kv_heads=size["kv_heads"], head_dim=size["dim"],
+               vocab=DESIGN_VOCAB, max_seq_len=DESIGN_CTX, rope_type=1, rope_theta=500000.0, rms_eps=1e-5)
+    type_of = synth.q4_k_m_type if quant == "q4_k_m" else (lambda name: H.Q8_0)
+    w = synth.make_llama(cfg, seed, type_of=type_of, n_threads=n_thr)
+    for i in range(1, DESIGN_LAYERS):
+        w.update({k.replace("blk.0.", f"blk.{i}."): v for k, v in w.items() if k.startswith("blk.0.")})
+    cfg["n_layers"] = DESIGN_LAYERS
+    nbytes = sum(v[3].nbytes for k, v in w.items() if isinstance(v, tuple) and not k.startswith("token_embd"))
+    return hip_api.Model(ctx, cfg, w), nbytes
+
+
+def measure_design(ctx, hip_api, H, args, n_thr):
+    """Prefill and decode rates of a Nafevik and of the llama of equal layer sizes, in turn, random weights."""
+    rng = np.random.default_rng(args.seed)
+    out = []
+    for name in args.design_sizes.split(","):
+        size = DESIGN_SIZES[name]
+        flops = 2 * DESIGN_LAYERS * (size["width"] * (2 * size["heads"] + 2 * size["kv_heads"]) * size["dim"] + 3 * size["width"] * size["ff"])
+        models = [("nafevik_bf16", *nafevik_model(ctx, hip_api, size, rng))]
+        for quant in args.design_llama.split(",") if args.design_llama else []:
+            models.append((f"llama_{quant}", *llama_model(ctx, hip_api, H, size, quant, args.seed, n_thr)))
+        best = {m[0]: {} for m in models}
+        toks = rng.integers(0, DESIGN_VOCAB, 2048).astype(np.uint32)
+        for rep in range(args.design_reps + 1):   # the first turn is warm-up; the models take turns
+            for label, m, nbytes in models:
+                res = {}
+                for n in (32, 512, 2048):
+                    t0 = time.perf_counter()
+                    m.forward_prefill(toks[:n], 0)
+                    res[f"prefill_{n}_tok_s"] = n / (time.perf_counter() - t0)
+                for at in (512, 1900):
+                    if at == 512:
+                        m.forward_prefill(toks[:512], 0)
+                    else:
+                        m.forward_prefill(toks[:1900], 0)
+                    t, steps = int(toks[0]), 64
+                    t = m.forward_greedy(t, at)
+                    t0 = time.perf_counter()
+                    for i in range(1, steps):
+                        t = m.forward_greedy(t, at + i)
+                    res[f"decode_at_{at}_tok_s"] = (steps - 1) / (time.perf_counter() - t0)
+                if rep:
+                    for k, v in res.items():
+                        best[label][k] = max(best[label].get(k, 0.0), v)
+                print(f"{name} {label} turn {rep}: " + ", ".join(f"{k} {v:.0f}" for k, v in res.items()), file=sys.stderr, flush=True)
+        for label, m, nbytes in models:
+            r = {k: round(v, 1) for k, v in best[label].items()}
+            r["weight_bytes_per_step"] = nbytes
+            r["decode_weight_GB/s"] = round(best[label]["decode_at_512_tok_s"] * nbytes / 1e9, 1)
+            r["decode_frac_of_hbm_peak"] = round(r["decode_weight_GB/s"] / HBM_PEAK_GBS, 4)
+            r["prefill_2048_TFLOP/s"] = round(best[label]["prefill_2048_tok_s"] * flops / 1e12, 1)
+            out.append({"size": name, "model": label, **r})
+            m.close()
+    return {"design": args.design, "layers": DESIGN_LAYERS, "vocab": DESIGN_VOCAB, "sizes": DESIGN_SIZES, "data": "synthetic, random-init weights",
+            "statistic": f"best of {args.design_reps} turns, host API calls included", "results": out}
+
+
 def reference_decode_threads(physical, logical):
     """The decode pool width cera picks for a bandwidth-bound model (more than 2.5 MB of weights per pool
     dispatch, which an 8B model is): physical + physical / 4 capped at 24, never above the detected
@@ -279,6 +371,12 @@ def main() -> int:
                     help="run only a 1 GiB copy kernel, a few launches of each per-layer GEMV kernel, decode attention at "
                          "131072 and 8192 keys and the two prefill GEMMs at 2048 tokens, for a hardware-counter pass under "
                          "rocprofv3 --pmc; prints no JSON")
+    ap.add_argument("--design", choices=["nafevik"],
+                    help="instead of the workload above: prefill and decode rates of this model design with random weights at a few "
+                         "layer sizes, beside the llama of equal size; prints one JSON line")
+    ap.add_argument("--design-sizes", default=",".join(DESIGN_SIZES), help="of " + ", ".join(DESIGN_SIZES))
+    ap.add_argument("--design-llama", default="q4_k_m,q8_0", help="type mixes of the llama beside it (empty: none)")
+    ap.add_argument("--design-reps", type=int, default=3)
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build measures one GPU only (the hot path has no multi-GPU part); "
@@ -292,6 +390,9 @@ def main() -> int:
     dev_name, n_cu, hbm = ctx.device_info()
     rng = np.random.default_rng(args.seed)
     n_thr = min(16, os.cpu_count() or 1)
+    if args.design:
+        print(json.dumps(measure_design(ctx, hip_api, H, args, n_thr)))
+        return 0
     eps = 1e-5
 
     # ---- synthetic weights: one properly quantized layer + head, cloned on device

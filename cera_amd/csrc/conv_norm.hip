@@ -1,4 +1,6 @@
 // Kernels of conv_norm.h.  Everything here is f32 up to the store of an output row.
+#include <algorithm>
+
 #include "bf16.hip.h"
 #include "conv_norm.h"
 
@@ -17,16 +19,21 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(const uint16_t* __restri
     x0[t * ld + c] = v;
 }
 
-// Eight rows per workgroup: first 1 / rms of those rows and of the taps - 1 before them (recomputed, so
-// that workgroups need nothing from each other), then the channels, four per thread.
-constexpr int ROWS = 8;
-template <typename T>
-__global__ __launch_bounds__(256) void norm_conv_kernel(NormConv a) {
-    __shared__ float inv[ROWS + CONV_MAX_TAPS];
+// A workgroup takes `rows` consecutive rows: first 1 / rms of those rows and of the taps - 1 before them
+// (recomputed, so that workgroups need nothing from each other), one row per wavefront; then the channels,
+// four per thread, walking down the rows.  TAPS > 0: the window of rows and the taps' weights stay in
+// registers; 0: any number of taps, re-reading the window.
+constexpr int NC_WAVES = 16, NC_MAX_ROWS = 16;
+__device__ __forceinline__ void fma4(float4& y, const float4& k, const float4& g) {
+    y.x = fmaf(k.x, g.x, y.x); y.y = fmaf(k.y, g.y, y.y); y.z = fmaf(k.z, g.z, y.z); y.w = fmaf(k.w, g.w, y.w);
+}
+template <typename T, int TAPS>
+__global__ __launch_bounds__(NC_WAVES * 64) void norm_conv_kernel(NormConv a, int rows) {
+    __shared__ float inv[NC_MAX_ROWS + CONV_MAX_TAPS];
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    const int back = a.taps ? static_cast<int>(a.taps) - 1 : 0, t0 = static_cast<int>(blockIdx.x) * ROWS;
-    const int t_end = min(t0 + ROWS, static_cast<int>(a.n));
-    for (int t = t0 - back + static_cast<int>(wave); t < t_end; t += 4) {
+    const int taps = TAPS ? TAPS : static_cast<int>(a.taps), back = taps ? taps - 1 : 0;
+    const int t0 = static_cast<int>(blockIdx.x) * rows, t_end = min(t0 + rows, static_cast<int>(a.n));
+    for (int t = t0 - back + static_cast<int>(wave); t < t_end; t += NC_WAVES) {
         if (t < 0) continue;
         const float* const row = a.x + static_cast<uint64_t>(t) * a.ld;
         float ss = 0.0f;
@@ -42,7 +49,7 @@ __global__ __launch_bounds__(256) void norm_conv_kernel(NormConv a) {
         }
     }
     __syncthreads();
-    for (uint32_t c = (blockIdx.y * 256 + threadIdx.x) * 4; c < a.ld; c += gridDim.y * 1024) {
+    for (uint32_t c = threadIdx.x * 4; c < a.ld; c += NC_WAVES * 256) {
         const float4 w = *reinterpret_cast<const float4*>(a.w + c);
         auto h_at = [&](int t) -> float4 {
             if (t < 0) {
@@ -54,21 +61,43 @@ __global__ __launch_bounds__(256) void norm_conv_kernel(NormConv a) {
             const float s = inv[t - t0 + back];
             return make_float4(v.x * s * w.x, v.y * s * w.y, v.z * s * w.z, v.w * s * w.w);
         };
-        for (int t = t0; t < t_end; ++t) {
-            const float4 h = h_at(t);
-            float4 ya = h, yb = h;
-            for (int j = 0; j < static_cast<int>(a.taps); ++j) {
-                const float4 g = j == back ? h : h_at(t - back + j);
-                const float4 ka = *reinterpret_cast<const float4*>(a.wa + static_cast<uint64_t>(j) * a.ld + c);
-                ya.x = fmaf(ka.x, g.x, ya.x); ya.y = fmaf(ka.y, g.y, ya.y); ya.z = fmaf(ka.z, g.z, ya.z); ya.w = fmaf(ka.w, g.w, ya.w);
-                if (a.wb) {
-                    const float4 kb = *reinterpret_cast<const float4*>(a.wb + static_cast<uint64_t>(j) * a.ld + c);
-                    yb.x = fmaf(kb.x, g.x, yb.x); yb.y = fmaf(kb.y, g.y, yb.y); yb.z = fmaf(kb.z, g.z, yb.z); yb.w = fmaf(kb.w, g.w, yb.w);
-                }
-            }
+        auto store = [&](int t, const float4& ya, const float4& yb) {
             const uint64_t at = static_cast<uint64_t>(t) * a.ld + c;
             ElemOps<T>::store4(static_cast<T*>(a.out_a) + at, ya.x, ya.y, ya.z, ya.w);
             if (a.out_b) ElemOps<T>::store4(static_cast<T*>(a.out_b) + at, yb.x, yb.y, yb.z, yb.w);
+        };
+        if constexpr (TAPS > 0) {
+            float4 ka[TAPS], kb[TAPS], h[TAPS];
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) {
+                ka[j] = *reinterpret_cast<const float4*>(a.wa + static_cast<uint64_t>(j) * a.ld + c);
+                kb[j] = a.wb ? *reinterpret_cast<const float4*>(a.wb + static_cast<uint64_t>(j) * a.ld + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+            }
+#pragma unroll
+            for (int j = 0; j + 1 < TAPS; ++j) h[j + 1] = h_at(t0 - back + j);
+            for (int t = t0; t < t_end; ++t) {
+#pragma unroll
+                for (int j = 0; j + 1 < TAPS; ++j) h[j] = h[j + 1];
+                h[TAPS - 1] = h_at(t);
+                float4 ya = h[TAPS - 1], yb = ya;
+#pragma unroll
+                for (int j = 0; j < TAPS; ++j) {
+                    fma4(ya, ka[j], h[j]);
+                    fma4(yb, kb[j], h[j]);
+                }
+                store(t, ya, yb);
+            }
+        } else {
+            for (int t = t0; t < t_end; ++t) {
+                const float4 h = h_at(t);
+                float4 ya = h, yb = h;
+                for (int j = 0; j < taps; ++j) {
+                    const float4 g = j == back ? h : h_at(t - back + j);
+                    fma4(ya, *reinterpret_cast<const float4*>(a.wa + static_cast<uint64_t>(j) * a.ld + c), g);
+                    if (a.wb) fma4(yb, *reinterpret_cast<const float4*>(a.wb + static_cast<uint64_t>(j) * a.ld + c), g);
+                }
+                store(t, ya, yb);
+            }
         }
     }
 }
@@ -94,12 +123,20 @@ cera_hip_status cera_launch_embed_pos(cera_hip_ctx* ctx, const void* embed, cons
 cera_hip_status cera_launch_norm_conv(cera_hip_ctx* ctx, const NormConv& a, bool f32) {
     if (a.ld % 4 || a.taps > CONV_MAX_TAPS || (a.taps > 1 && (!a.ring.rows || a.ring.depth < a.taps)) || (a.out_b && !a.wb && a.taps))
         return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "norm_conv: bad shape");
-    const uint32_t groups = (a.n + ROWS - 1) / ROWS;
-    // few rows: the channels are spread over workgroups as well (each recomputes its rows' norms)
-    const uint32_t cols = static_cast<uint32_t>((a.ld + 1023) / 1024);
-    const dim3 grid(groups, groups * cols <= 4 * ctx->n_cu ? cols : 1);
-    if (f32) hipLaunchKernelGGL(norm_conv_kernel<float>, grid, dim3(256), 0, ctx->stream, a);
-    else hipLaunchKernelGGL(norm_conv_kernel<__bf16>, grid, dim3(256), 0, ctx->stream, a);
+    // one workgroup per CU, more rows each beyond that
+    const int rows = static_cast<int>(std::min<uint32_t>(NC_MAX_ROWS, std::max<uint32_t>(1, (a.n + ctx->n_cu - 1) / ctx->n_cu)));
+    const dim3 grid((a.n + rows - 1) / rows), block(NC_WAVES * 64);
+    auto go = [&](auto tag) {
+        using T = decltype(tag);
+        switch (a.taps) {
+            case 2: hipLaunchKernelGGL((norm_conv_kernel<T, 2>), grid, block, 0, ctx->stream, a, rows); break;
+            case 3: hipLaunchKernelGGL((norm_conv_kernel<T, 3>), grid, block, 0, ctx->stream, a, rows); break;
+            case 4: hipLaunchKernelGGL((norm_conv_kernel<T, 4>), grid, block, 0, ctx->stream, a, rows); break;
+            default: hipLaunchKernelGGL((norm_conv_kernel<T, 0>), grid, block, 0, ctx->stream, a, rows); break;
+        }
+    };
+    if (f32) go(float{});
+    else go(static_cast<__bf16>(0.0f));
     HIP_TRY(ctx, hipGetLastError());
     return CERA_HIP_OK;
 }

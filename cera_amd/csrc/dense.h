@@ -2,6 +2,7 @@
 // activations and a streaming GEMV for one, with the small operations around them folded in.
 #pragma once
 #include "host_common.h"
+#include "sigmoid_attn.h"   // SAttnPartials
 
 constexpr uint32_t DENSE_PAD = 64;   // K is padded with zeros to whole 128-byte lines of bf16
 static inline uint64_t dense_pad(uint64_t k) { return (k + DENSE_PAD - 1) / DENSE_PAD * DENSE_PAD; }
@@ -34,12 +35,14 @@ cera_hip_status cera_launch_dense_gemm(cera_hip_ctx* ctx, const DenseMat& w, con
 // One token.  Where its activations come from:
 struct DenseIn {
     // RAW: element-type vector [kp].  NORM: x f32 [kp], normalised over its first n_mean entries.
+    // MERGE: as RAW, but the first heads * vdim elements are the sum of attention's partial results, gated.
     // CONCAT: x | x2, f32 [kp / 2] each.  Pad columns of x, x2, scale, add and plain are zero.
-    enum Kind { RAW = 0, NORM = 1, CONCAT = 2 } kind = RAW;
+    enum Kind { RAW = 0, NORM = 1, CONCAT = 2, MERGE = 3 } kind = RAW;
     const void* x = nullptr;
     const float* x2 = nullptr;
     uint32_t n_mean = 0;
     float eps = 0;
+    SAttnPartials merge;
     // NORM: staged value of channel c is x[c] * inv * scale[c] + (add ? add[c] : 0)
     const float *scale_a = nullptr, *add_a = nullptr, *scale_b = nullptr, *add_b = nullptr;
     // NORM: also h[c] = x[c] * inv * plain[c] into h_out (nullable), by one workgroup
@@ -47,7 +50,7 @@ struct DenseIn {
     float* h_out = nullptr;
 };
 // y = W_a . in_a, and in the same launch y_b = W_b . in_b (wb nullable).  The two may have different
-// NORM scale / add vectors; RAW and CONCAT share the one input.  *launched = false when the input
+// NORM scale / add vectors; the other kinds share the one input.  *launched = false when the input
 // does not fit the workgroup's LDS (the caller then takes the GEMM route).
 cera_hip_status cera_launch_dense_gemv(cera_hip_ctx* ctx, const DenseIn& in, const DenseMat& wa, const DenseOut& oa,
                                        const DenseMat* wb, const DenseOut* ob, bool f32, bool* launched);

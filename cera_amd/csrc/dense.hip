@@ -6,7 +6,7 @@
 // operand: a lane then holds four consecutive output rows of one token, which the epilogue stores
 // as one vector.  The f32 variant stages both operands as f32 and runs on v_mfma_f32_16x16x4_f32.
 //
-// GEMV: a wavefront streams four rows at a time, 16 bytes per lane per row and step, against the
+// GEMV: a wavefront streams up to four rows at a time, 16 bytes per lane per row and step, against the
 // activation vector in LDS; the workgroup prepares that vector itself (row norm, convolution of the
 // current token, concatenation), so those need no launch of their own.
 #include <algorithm>
@@ -264,12 +264,14 @@ struct GemvDArgs {
     DenseIn in;
     const __bf16 *wa, *wb;
     uint32_t rows_a, rows_b, kp, stage_len;   // stage_len: LDS elements, kp rounded up to a whole step of the wavefront
-    uint32_t blocks_a, groups_a, groups_b, blocks_b;   // groups of four rows
+    uint32_t blocks_a, groups_a, groups_b, blocks_b;   // groups of R rows
     DenseOut oa, ob;
 };
 
-constexpr int GEMV_WAVES = 8, GEMV_ROWS = 4, GEMV_U = 2;
-constexpr uint32_t GEMV_STEP = 64 * 8 * GEMV_U;
+constexpr int GEMV_WAVES = 8;
+// A wavefront has R rows in flight, U steps of 64 16-byte chunks each: 8 KB per wavefront either way.
+template <int R> constexpr int GEMV_U = 8 / R;
+template <int R> constexpr uint32_t GEMV_STEP = 64 * 8 * GEMV_U<R>;
 
 // Fills the workgroup's activation vector xs[0, stage_len).
 template <typename T, int KIND>
@@ -278,8 +280,41 @@ __device__ __forceinline__ void gemv_stage(const GemvDArgs& a, bool second, bool
     if (KIND == DenseIn::RAW) {
         const T* x = static_cast<const T*>(in.x);
         constexpr uint32_t V = 16 / sizeof(T);
+#pragma unroll 4
         for (uint32_t i = threadIdx.x * V; i < a.stage_len; i += GEMV_WAVES * 64 * V)
             *reinterpret_cast<uint4*>(xs + i) = i < a.kp ? *reinterpret_cast<const uint4*>(x + i) : make_uint4(0, 0, 0, 0);
+    } else if (KIND == DenseIn::MERGE) {
+        const T* x = static_cast<const T*>(in.x);
+        const SAttnPartials& m = in.merge;
+        const uint32_t cols = m.heads * m.vdim, cols_p = (cols + DENSE_PAD - 1) / DENSE_PAD * DENSE_PAD;
+        const uint64_t slice = static_cast<uint64_t>(m.heads) * m.vdim_p;
+        constexpr uint32_t V = 16 / sizeof(T);
+#pragma unroll 4
+        for (uint32_t i = cols_p + threadIdx.x * V; i < a.stage_len; i += GEMV_WAVES * 64 * V)
+            *reinterpret_cast<uint4*>(xs + i) = i < a.kp ? *reinterpret_cast<const uint4*>(x + i) : make_uint4(0, 0, 0, 0);
+#pragma unroll 2
+        for (uint32_t i = threadIdx.x * 4; i < cols_p; i += GEMV_WAVES * 256) {
+            if (i + 4 <= cols && m.vdim % 4 == 0) {
+                const uint32_t h = i / m.vdim;
+                const float* p = m.part + h * m.vdim_p + (i - h * m.vdim);
+                f32x4 s = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll 4
+                for (uint32_t z = 1; z < m.splits; ++z) s += *reinterpret_cast<const f32x4*>(p + z * slice);
+                const float g = sigmoid_f32(m.gate[h]);
+                ElemOps<T>::store4(xs + i, s.x * g, s.y * g, s.z * g, s.w * g);
+            } else {
+#pragma unroll
+                for (uint32_t e = i; e < i + 4; ++e) {
+                    float s = 0.0f;
+                    if (e < cols) {
+                        const uint32_t h = e / m.vdim;
+                        for (uint32_t z = 0; z < m.splits; ++z) s += m.part[z * slice + h * m.vdim_p + (e - h * m.vdim)];
+                        s *= sigmoid_f32(m.gate[h]);
+                    }
+                    xs[e] = ElemOps<T>::from(s);
+                }
+            }
+        }
     } else if (KIND == DenseIn::CONCAT) {
         const float* x = static_cast<const float*>(in.x);
         const uint32_t half = a.kp / 2;
@@ -298,7 +333,7 @@ __device__ __forceinline__ void gemv_stage(const GemvDArgs& a, bool second, bool
         }
         ss = wave_sum(ss);
         if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
-        __syncthreads();
+        lds_barrier();
         float tot = 0.0f;
 #pragma unroll
         for (int i = 0; i < GEMV_WAVES; ++i) tot += red[i];
@@ -318,83 +353,131 @@ __device__ __forceinline__ void gemv_stage(const GemvDArgs& a, bool second, bool
             ElemOps<T>::store4(xs + i, o.x, o.y, o.z, o.w);
         }
     }
-    __syncthreads();
+    lds_barrier();
 }
 
-// groups [g0, g1) of four rows of one matrix; SWIGLU: a group is two gate rows and their two up rows
-template <typename T>
-__device__ __forceinline__ void gemv_rows(const __bf16* __restrict__ w, uint32_t rows, uint32_t kp, uint32_t stage_len, const DenseOut& o,
-                                          uint32_t g0, uint32_t g1, const T* xs) {
-    const uint32_t lane = threadIdx.x & 63, last = kp / 8 - 1;
-    const bool swiglu = o.epi == DENSE_SWIGLU;
-    for (uint32_t g = g0 + (threadIdx.x >> 6); g < g1; g += GEMV_WAVES) {
-        uint32_t row[GEMV_ROWS];
-        const __bf16* p[GEMV_ROWS];
+// One wavefront's walk over its groups of R rows (g, g + GEMV_WAVES, ... below g1) of one matrix, a step of
+// U * 64 16-byte chunks at a time; SWIGLU: a group is R / 2 gate rows and their up rows.  Two step buffers
+// alternate, the next step's loads -- of the next group too -- going out before the current one is multiplied.
+template <typename T, int R> struct GemvWalk {
+    static constexpr int U = GEMV_U<R>, H = R > 1 ? R / 2 : 1;
+    typedef uint4 Buf[U][R];
+    const __bf16* w;
+    uint32_t rows, kp, stage_len, g1, lane, last;
+    bool swiglu;
+    uint32_t lg, lk;            // group and step the next load takes
+    const __bf16* p[R];
+    float acc[R];
+
+    __device__ __forceinline__ void set_rows() {
 #pragma unroll
-        for (int r = 0; r < GEMV_ROWS; ++r) {
+        for (int r = 0; r < R; ++r) {
+            uint32_t row = lg * R + r;
             if (swiglu) {
-                const uint32_t i = g * 2 + (r & 1);
-                row[r] = (i >> 4) * 32 + (i & 15) + (r & 2) * 8;
-            } else {
-                row[r] = g * 4 + r;
+                const uint32_t i = lg * H + r % H;
+                row = (i >> 4) * 32 + (i & 15) + (r >= H && R > 1 ? 16 : 0);
             }
-            p[r] = w + static_cast<uint64_t>(min(row[r], rows - 1)) * kp;
+            p[r] = w + static_cast<uint64_t>(min(row, rows - 1)) * kp;
         }
-        float acc[GEMV_ROWS] = {0.f, 0.f, 0.f, 0.f};
-        for (uint32_t k = 0; k < stage_len; k += GEMV_STEP) {
-            uint4 wv[GEMV_U][GEMV_ROWS];
+    }
+    __device__ __forceinline__ void begin(const __bf16* w_, uint32_t rows_, uint32_t kp_, uint32_t stage_len_, bool swiglu_, uint32_t g, uint32_t g1_) {
+        w = w_; rows = rows_; kp = kp_; stage_len = stage_len_; swiglu = R > 1 && swiglu_; g1 = g1_;
+        lane = threadIdx.x & 63; last = kp / 8 - 1;
+        lg = g; lk = 0;
+        if (lg < g1) set_rows();
 #pragma unroll
-            for (int u = 0; u < GEMV_U; ++u)
+        for (int r = 0; r < R; ++r) acc[r] = 0.0f;
+    }
+    __device__ __forceinline__ bool load(Buf& b) {
+        if (lg >= g1) return false;
 #pragma unroll
-                for (int r = 0; r < GEMV_ROWS; ++r)   // past the row's end: its last chunk again, against zeros
-                    wv[u][r] = ld_u128_nt(p[r] + min(k / 8 + u * 64 + lane, last) * 8);
+        for (int u = 0; u < U; ++u)
 #pragma unroll
-            for (int u = 0; u < GEMV_U; ++u) {
-                const typename ElemOps<T>::X8 xv = ElemOps<T>::ld8(xs + k + (u * 64 + lane) * 8);
-#pragma unroll
-                for (int r = 0; r < GEMV_ROWS; ++r) acc[r] = ElemOps<T>::dot8(wv[u][r], xv, acc[r]);
-            }
+            for (int r = 0; r < R; ++r)   // past the row's end: its last chunk again, against zeros
+                b[u][r] = ld_u128_nt(p[r] + min(lk / 8 + u * 64 + lane, last) * 8);
+        lk += GEMV_STEP<R>;
+        if (lk >= stage_len) {
+            lk = 0;
+            lg += GEMV_WAVES;
+            if (lg < g1) set_rows();
         }
+        return true;
+    }
+    // multiplies a step of group g at k; at the group's last step reduces and stores, and moves on
+    __device__ __forceinline__ void use(const Buf& b, uint32_t& g, uint32_t& k, const T* xs, const DenseOut& o) {
 #pragma unroll
-        for (int r = 0; r < GEMV_ROWS; ++r) acc[r] = wave_sum(acc[r]);
+        for (int u = 0; u < U; ++u) {
+            const typename ElemOps<T>::X8 xv = ElemOps<T>::ld8(xs + k + (u * 64 + lane) * 8);
+#pragma unroll
+            for (int r = 0; r < R; ++r) acc[r] = ElemOps<T>::dot8(b[u][r], xv, acc[r]);
+        }
+        k += GEMV_STEP<R>;
+        if (k < stage_len) return;
+        k = 0;
+#pragma unroll
+        for (int r = 0; r < R; ++r) acc[r] = wave_sum(acc[r]);
         if (swiglu) {
-            const uint32_t i = g * 2 + lane;
-            if (lane < 2 && i < o.rows)
-                static_cast<T*>(o.out)[i] = ElemOps<T>::from(dense_silu_mul(lane ? acc[1] : acc[0], lane ? acc[3] : acc[2]));
+            const uint32_t i = g * H + lane;
+            float gt = acc[0], up = acc[R > 1 ? H : 0];
+#pragma unroll
+            for (int r = 1; r < H; ++r)
+                if (lane == static_cast<uint32_t>(r)) { gt = acc[r]; up = acc[H + r]; }
+            if (lane < static_cast<uint32_t>(H) && i < o.rows) static_cast<T*>(o.out)[i] = ElemOps<T>::from(dense_silu_mul(gt, up));
         } else {
-            const uint32_t i = g * 4 + lane;
-            if (lane < 4 && i < rows) {
-                const float y = lane < 2 ? (lane ? acc[1] : acc[0]) : (lane == 2 ? acc[2] : acc[3]);
+            const uint32_t i = g * R + lane;
+            float y = acc[0];
+#pragma unroll
+            for (int r = 1; r < R; ++r)
+                if (lane == static_cast<uint32_t>(r)) y = acc[r];
+            if (lane < static_cast<uint32_t>(R) && i < rows) {
                 float* out = static_cast<float*>(o.out) + i;
                 if (o.epi == DENSE_ADD) *out = fmaf(o.mult, y, *out);
                 else *out = o.bias ? y + o.bias[i] : y;
             }
         }
+#pragma unroll
+        for (int r = 0; r < R; ++r) acc[r] = 0.0f;
+        g += GEMV_WAVES;
     }
-}
+};
 
-template <typename T, int KIND>
+template <typename T, int KIND, int R>
 __global__ __launch_bounds__(GEMV_WAVES * 64) void dense_gemv_kernel(GemvDArgs a) {
     extern __shared__ __align__(16) unsigned char smem[];
     __shared__ float red[GEMV_WAVES];
     T* const xs = reinterpret_cast<T*>(smem);
     const bool second = blockIdx.x >= a.blocks_a;
-    gemv_stage<T, KIND>(a, second, KIND == DenseIn::NORM && a.in.h_out && blockIdx.x == 0, xs, red);
     const uint32_t groups = second ? a.groups_b : a.groups_a, blocks = second ? a.blocks_b : a.blocks_a;
     const uint32_t b = second ? blockIdx.x - a.blocks_a : blockIdx.x;
     // the first `groups % blocks` workgroups take one group more
     const uint32_t each = groups / blocks, more = groups % blocks;
     const uint32_t g0 = b * each + min(b, more), g1 = g0 + each + (b < more ? 1 : 0);
-    if (second) gemv_rows<T>(a.wb, a.rows_b, a.kp, a.stage_len, a.ob, g0, g1, xs);
-    else gemv_rows<T>(a.wa, a.rows_a, a.kp, a.stage_len, a.oa, g0, g1, xs);
+    const DenseOut& o = second ? a.ob : a.oa;
+    GemvWalk<T, R> walk;
+    typename GemvWalk<T, R>::Buf w0, w1;
+    uint32_t g = g0 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), k = 0;
+    walk.begin(second ? a.wb : a.wa, second ? a.rows_b : a.rows_a, a.kp, a.stage_len, o.epi == DENSE_SWIGLU, g, g1);
+    // the first weights are on their way while the activation vector is prepared
+    bool more0 = walk.load(w0);
+    gemv_stage<T, KIND>(a, second, KIND == DenseIn::NORM && a.in.h_out && blockIdx.x == 0, xs, red);
+    while (more0) {
+        const bool more1 = walk.load(w1);
+        walk.use(w0, g, k, xs, o);
+        if (!more1) break;
+        more0 = walk.load(w0);
+        walk.use(w1, g, k, xs, o);
+    }
 }
 
 constexpr uint64_t GEMV_LDS_MAX = 60 * 1024;
 
 }  // namespace
 
-static uint64_t gemv_lds(uint64_t kp, bool f32) { return (kp + GEMV_STEP - 1) / GEMV_STEP * GEMV_STEP * (f32 ? 4 : 2); }
-bool cera_dense_gemv_fits(uint64_t kp, bool f32) { return gemv_lds(kp, f32) <= GEMV_LDS_MAX; }
+static uint64_t gemv_stage_len(uint64_t kp, int r) {
+    const uint64_t step = 64ull * 8 * (8 / r);
+    return (kp + step - 1) / step * step;
+}
+bool cera_dense_gemv_fits(uint64_t kp, bool f32) { return gemv_stage_len(kp, 1) * (f32 ? 4 : 2) <= GEMV_LDS_MAX; }
 
 cera_hip_status cera_launch_dense_gemm(cera_hip_ctx* ctx, const DenseMat& w, const void* x, uint64_t ldx, uint32_t n,
                                        const DenseOut& o, bool f32) {
@@ -451,13 +534,19 @@ cera_hip_status cera_launch_dense_gemv(cera_hip_ctx* ctx, const DenseIn& in, con
     GemvDArgs a{};
     a.in = in;
     a.wa = static_cast<const __bf16*>(wa.w); a.rows_a = wa.rows; a.kp = wa.kp; a.oa = oa;
-    a.stage_len = (wa.kp + GEMV_STEP - 1) / GEMV_STEP * GEMV_STEP;
-    const uint64_t lds = gemv_lds(wa.kp, f32);
-    if (lds > GEMV_LDS_MAX) return CERA_HIP_OK;
-    a.groups_a = oa.epi == DENSE_SWIGLU ? wa.rows / 4 : (wa.rows + 3) / 4;
+    if (!cera_dense_gemv_fits(wa.kp, f32)) return CERA_HIP_OK;
+    // fewer rows per wavefront (and a longer run of each) where four would leave CUs without work
+    const bool pairs = oa.epi == DENSE_SWIGLU || (wb && ob->epi == DENSE_SWIGLU);
+    const uint64_t all_rows = static_cast<uint64_t>(wa.rows) + (wb ? wb->rows : 0);
+    int r = 4;
+    if (all_rows < 8ull * GEMV_WAVES * ctx->n_cu && wa.kp >= 1024) r = 2;
+    if (all_rows < 4ull * GEMV_WAVES * ctx->n_cu && wa.kp >= 2048 && !pairs) r = 1;
+    a.stage_len = static_cast<uint32_t>(gemv_stage_len(wa.kp, r));
+    const uint64_t lds = a.stage_len * (f32 ? 4ull : 2ull);
+    a.groups_a = oa.epi == DENSE_SWIGLU ? wa.rows / r : (wa.rows + r - 1) / r;
     if (wb) {
         a.wb = static_cast<const __bf16*>(wb->w); a.rows_b = wb->rows; a.ob = *ob;
-        a.groups_b = ob->epi == DENSE_SWIGLU ? wb->rows / 4 : (wb->rows + 3) / 4;
+        a.groups_b = ob->epi == DENSE_SWIGLU ? wb->rows / r : (wb->rows + r - 1) / r;
     }
     // about two workgroups per CU, shared between the matrices by their rows; no workgroup without a group
     const uint32_t total = a.groups_a + a.groups_b;
@@ -465,14 +554,21 @@ cera_hip_status cera_launch_dense_gemv(cera_hip_ctx* ctx, const DenseIn& in, con
     a.blocks_a = std::max(1u, std::min(a.groups_a, wb ? static_cast<uint32_t>(static_cast<uint64_t>(want) * a.groups_a / total) : want));
     a.blocks_b = wb ? std::max(1u, std::min(a.groups_b, want > a.blocks_a ? want - a.blocks_a : 1u)) : 0;
     const dim3 grid(a.blocks_a + a.blocks_b), block(GEMV_WAVES * 64);
-    auto go = [&](auto tag) {
+    auto go = [&](auto tag, auto rows) {
         using T = decltype(tag);
-        if (in.kind == DenseIn::RAW) hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::RAW>), grid, block, lds, ctx->stream, a);
-        else if (in.kind == DenseIn::NORM) hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::NORM>), grid, block, lds, ctx->stream, a);
-        else hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::CONCAT>), grid, block, lds, ctx->stream, a);
+        constexpr int R = decltype(rows)::value;
+        if (in.kind == DenseIn::RAW) hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::RAW, R>), grid, block, lds, ctx->stream, a);
+        else if (in.kind == DenseIn::MERGE) hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::MERGE, R>), grid, block, lds, ctx->stream, a);
+        else if (in.kind == DenseIn::NORM) hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::NORM, R>), grid, block, lds, ctx->stream, a);
+        else hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::CONCAT, R>), grid, block, lds, ctx->stream, a);
     };
-    if (f32) go(float{});
-    else go(static_cast<__bf16>(0.0f));
+    auto by_rows = [&](auto tag) {
+        if (r == 4) go(tag, std::integral_constant<int, 4>{});
+        else if (r == 2) go(tag, std::integral_constant<int, 2>{});
+        else go(tag, std::integral_constant<int, 1>{});
+    };
+    if (f32) by_rows(float{});
+    else by_rows(static_cast<__bf16>(0.0f));
     HIP_TRY(ctx, hipGetLastError());
     *launched = true;
     return CERA_HIP_OK;

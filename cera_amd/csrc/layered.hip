@@ -4,7 +4,8 @@
 // Decode, per layer, three launches: [norm, both input convolutions, Q|K|V|gate and gate|up
 // with SwiGLU] - [rotation, append, attention, head gates; the convolutions' history for the next
 // token beside it] - [O and down as one product over the two inputs side by side, added to the
-// residual].  A long key range adds one launch that sums the partial results.
+// residual; it also adds up attention's partial results over key ranges].  A very long key range adds
+// a launch for that sum.
 #include <algorithm>
 #include <cmath>
 #include <cstring>
@@ -192,9 +193,10 @@ cera_hip_status decode(cera_hip_model* m, uint32_t token, uint32_t pos, bool wan
         of.epi = DENSE_SWIGLU; of.rows = W.ff;
         of.out = static_cast<char*>(g.cat) + W.att_p * g.esz;
         CERA_TRY(gemv(in, W.qkvg, oq, W.ff ? &W.gate_up : nullptr, &of));
-        CERA_TRY(cera_launch_sattn_step(ctx, W.shape, step_pass(g, W, R, pos), R.ring, R.hist, g.f32));
         DenseIn raw;
         raw.x = g.cat;
+        CERA_TRY(cera_launch_sattn_step(ctx, W.shape, step_pass(g, W, R, pos), R.ring, R.hist, &raw.merge, g.f32));
+        if (raw.merge.part) raw.kind = DenseIn::MERGE;
         DenseOut add;
         add.epi = DENSE_ADD; add.out = g.x; add.mult = g.cfg.residual_mult; add.rows = width;
         CERA_TRY(gemv(raw, W.down, add));

@@ -56,7 +56,15 @@ struct ConvHist {
     uint32_t taps = 0;
     float *a = nullptr, *b = nullptr;
 };
+// merge (nullable): receives partial results over key ranges that the consumer of the output adds up and gates
+// itself -- or part == nullptr when the launch has already written p.out.
+constexpr uint32_t SATTN_MERGE_SPLITS = 8;
+struct SAttnPartials {
+    const float* part = nullptr;   // [splits][heads][vdim_p]
+    const float* gate = nullptr;   // [heads], before the sigmoid
+    uint32_t splits = 0, heads = 0, vdim = 0, vdim_p = 0;
+};
 cera_hip_status cera_launch_sattn_step(cera_hip_ctx* ctx, const SAttnShape& s, const SAttnPass& p, const ConvRing& ring,
-                                       const ConvHist& hist, bool f32);
+                                       const ConvHist& hist, SAttnPartials* merge, bool f32);
 // the history sums alone, for the token at `pos`
 cera_hip_status cera_launch_conv_hist(cera_hip_ctx* ctx, const ConvRing& ring, const ConvHist& hist, uint32_t pos);

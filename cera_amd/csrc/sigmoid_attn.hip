@@ -57,39 +57,50 @@ template <int DK, int VT, int CT> struct Tile<__bf16, DK, VT, CT> {
             if ((DK || kd < static_cast<int>(nk)) && live) q[ct][kd] = *reinterpret_cast<const bf16x8*>(row + kd * 32 + g * 8);
         }
     }
-    // kb: first key of the block; lo / hi: the visible range of this lane's column; inside: the whole block is
-    // visible to every column of the wavefront
-    __device__ __forceinline__ void block(const __bf16* kbase, const __bf16* vbase, uint32_t cap, uint32_t kb, uint32_t nk,
-                                          uint32_t nv, uint32_t dim_p, const uint32_t (&lo)[CT], const uint32_t (&hi)[CT],
-                                          bool inside, float scale, const float (&bias)[CT], uint32_t lane) {
+    // A block's K rows go into registers ahead of its turn.
+    bf16x8 ka[MK], kc[MK];
+    __device__ __forceinline__ void load_k(const __bf16* kbase, uint32_t kb, uint32_t nk, uint32_t dim_p, uint32_t lane) {
         const uint32_t r = lane & 15, g = lane >> 4;
         const __bf16* const k0 = kbase + static_cast<uint64_t>(kb + (r >> 2) * 8 + (r & 3)) * dim_p + g * 8;
         const __bf16* const k1 = k0 + 4 * static_cast<uint64_t>(dim_p);
-        const __bf16* const v0 = vbase + static_cast<uint64_t>(r) * cap + kb + g * 8;
-        bf16x8 ka[MK], kc[MK], va[MV];
 #pragma unroll
         for (int kd = 0; kd < MK; ++kd)
             if (DK || kd < static_cast<int>(nk)) {
                 ka[kd] = *reinterpret_cast<const bf16x8*>(k0 + kd * 32);
                 kc[kd] = *reinterpret_cast<const bf16x8*>(k1 + kd * 32);
             }
+    }
+    // kb: first key of the block, its K rows loaded; next: the block whose K rows are loaded meanwhile (UINT32_MAX:
+    // none); lo / hi: the visible range of this lane's column; inside: the whole block is visible to every column
+    // of the wavefront
+    __device__ __forceinline__ void block(const __bf16* kbase, const __bf16* vbase, uint32_t cap, uint32_t kb, uint32_t next, uint32_t nk,
+                                          uint32_t nv, uint32_t dim_p, const uint32_t (&lo)[CT], const uint32_t (&hi)[CT],
+                                          bool inside, float scale, const float (&bias)[CT], uint32_t lane) {
+        const uint32_t r = lane & 15, g = lane >> 4;
+        const __bf16* const v0 = vbase + static_cast<uint64_t>(r) * cap + kb + g * 8;
+        bf16x8 va[MV];
         if (VT) {
 #pragma unroll
             for (int vt = 0; vt < MV; ++vt) va[vt] = *reinterpret_cast<const bf16x8*>(v0 + static_cast<uint64_t>(vt * 16) * cap);
         }
-        bf16x8 ph[CT], pl[CT];
+        f32x4 s0[CT], s1[CT];
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct) {
-            f32x4 s0{0.f, 0.f, 0.f, 0.f}, s1{0.f, 0.f, 0.f, 0.f};
+            s0[ct] = s1[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int kd = 0; kd < MK; ++kd)
                 if (DK || kd < static_cast<int>(nk)) {
-                    s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ka[kd], q[ct][kd], s0, 0, 0, 0);
-                    s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kc[kd], q[ct][kd], s1, 0, 0, 0);
+                    s0[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ka[kd], q[ct][kd], s0[ct], 0, 0, 0);
+                    s1[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kc[kd], q[ct][kd], s1[ct], 0, 0, 0);
                 }
+        }
+        if (next != UINT32_MAX) load_k(kbase, next, nk, dim_p, lane);
+        bf16x8 ph[CT], pl[CT];
+#pragma unroll
+        for (int ct = 0; ct < CT; ++ct) {
 #pragma unroll
             for (int i = 0; i < 8; ++i) {
-                const float s = i < 4 ? s0[i & 3] : s1[i & 3];
+                const float s = i < 4 ? s0[ct][i & 3] : s1[ct][i & 3];
                 float p = sigmoid_fast(fmaf(s, scale, bias[ct]));
                 if (!inside) {
                     const uint32_t key = kb + g * 8 + i;
@@ -128,7 +139,8 @@ template <int DK, int VT, int CT> struct Tile<float, DK, VT, CT> {
             if ((DK || kd < static_cast<int>(2 * nk)) && live) q[ct][kd] = *reinterpret_cast<const f32x4*>(row + kd * 16 + g * 4);
         }
     }
-    __device__ __forceinline__ void block(const float* kbase, const float* vbase, uint32_t cap, uint32_t kb0, uint32_t nk,
+    __device__ __forceinline__ void load_k(const float*, uint32_t, uint32_t, uint32_t, uint32_t) {}   // read where they are used
+    __device__ __forceinline__ void block(const float* kbase, const float* vbase, uint32_t cap, uint32_t kb0, uint32_t, uint32_t nk,
                                           uint32_t nv, uint32_t dim_p, const uint32_t (&lo)[CT], const uint32_t (&hi)[CT],
                                           bool inside, float scale, const float (&bias)[CT], uint32_t lane) {
         const uint32_t r = lane & 15, g = lane >> 4;
@@ -229,8 +241,10 @@ __global__ __launch_bounds__(256) void sattn_rows_kernel(AArgs a) {
     }
     const T* const kb_ = static_cast<const T*>(a.kc) + static_cast<uint64_t>(kvh) * a.cap * a.dim_p;
     const T* const vb_ = static_cast<const T*>(a.vc) + static_cast<uint64_t>(kvh) * a.vdim_p * a.cap;
+    t.load_k(kb_, col.lo_min & ~31u, nk, a.dim_p, lane);
     for (uint32_t kb = col.lo_min & ~31u; kb <= col.hi_max; kb += 32)
-        t.block(kb_, vb_, a.cap, kb, nk, nv, a.dim_p, col.lo, col.hi, kb >= col.lo_max && kb + 31 <= col.hi_min, a.scale, col.bias, lane);
+        t.block(kb_, vb_, a.cap, kb, kb + 32 <= col.hi_max ? kb + 32 : UINT32_MAX, nk, nv, a.dim_p, col.lo, col.hi,
+                kb >= col.lo_max && kb + 31 <= col.hi_min, a.scale, col.bias, lane);
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct)
         if (col.live[ct]) {
@@ -279,6 +293,12 @@ __global__ __launch_bounds__(SPLIT_WAVES * 64) void sattn_split_kernel(AArgs a) 
     const uint32_t b0 = col.lo_min / 32, nb = col.hi_max / 32 + 1 - b0, per_split = (nb + a.splits - 1) / a.splits;
     const uint32_t first = b0 + split * per_split, last = min(b0 + nb, first + per_split);
     Tile<T, DK, VT, 1> t;
+    const T* const kb_ = static_cast<const T*>(a.kc) + static_cast<uint64_t>(kvh) * a.cap * a.dim_p;
+    const T* const vb_ = static_cast<const T*>(a.vc) + static_cast<uint64_t>(kvh) * a.vdim_p * a.cap;
+    // the first block's K rows are on their way while the queries are prepared, unless the block holds the new key
+    uint32_t b = first + wave;
+    const bool early = b < last && !(FUSED && b == b0 + nb - 1);
+    if (early) t.load_k(kb_, b * 32, nk, a.dim_p, lane);
     if (FUSED) {
         const float* const row = a.qkvg;
         const float* const kn = row + a.heads * a.dim + kvh * a.dim;
@@ -320,11 +340,11 @@ __global__ __launch_bounds__(SPLIT_WAVES * 64) void sattn_split_kernel(AArgs a) 
     }
 #pragma unroll
     for (int vt = 0; vt < MV; ++vt) t.o[0][vt] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const T* const kb_ = static_cast<const T*>(a.kc) + static_cast<uint64_t>(kvh) * a.cap * a.dim_p;
-    const T* const vb_ = static_cast<const T*>(a.vc) + static_cast<uint64_t>(kvh) * a.vdim_p * a.cap;
-    for (uint32_t b = first + wave; b < last; b += SPLIT_WAVES) {
+    if (b < last && !early) t.load_k(kb_, b * 32, nk, a.dim_p, lane);
+    for (; b < last; b += SPLIT_WAVES) {
         const uint32_t kb = b * 32;
-        t.block(kb_, vb_, a.cap, kb, nk, nv, a.dim_p, col.lo, col.hi, kb >= col.lo_max && kb + 31 <= col.hi_min, a.scale, col.bias, lane);
+        t.block(kb_, vb_, a.cap, kb, b + SPLIT_WAVES < last ? kb + 32 * SPLIT_WAVES : UINT32_MAX, nk, nv, a.dim_p, col.lo, col.hi,
+                kb >= col.lo_max && kb + 31 <= col.hi_min, a.scale, col.bias, lane);
     }
     // add the wavefronts up: the upper half hands its tile to the lower half, three times
 #pragma unroll
@@ -347,7 +367,7 @@ __global__ __launch_bounds__(SPLIT_WAVES * 64) void sattn_split_kernel(AArgs a) 
     for (int vt = 0; vt < MV; ++vt)
         if (VT || vt < static_cast<int>(nv)) {
             const uint32_t v = vt * 16 + (lane >> 4) * 4;
-            if (a.splits > 1)
+            if (a.part)
                 *reinterpret_cast<f32x4*>(a.part + ((static_cast<uint64_t>(split) * a.n + col.query[0]) * a.heads + col.head[0]) * a.vdim_p + v) = t.o[0][vt];
             else
                 finish4<T>(a, col.query[0], col.head[0], v, t.o[0][vt]);
@@ -459,12 +479,19 @@ uint32_t max_blocks(const AArgs& a) {
     const uint32_t end = a.start + a.n, reach = a.chunk ? std::min(a.chunk + 31, end) : end;
     return (reach + 31) / 32 + 1;
 }
-cera_hip_status run_split(cera_hip_ctx* ctx, AArgs& a, bool f32, bool fused) {
+// merge (nullable, fused only): where to leave the partial results for the consumer instead of merging them here
+cera_hip_status run_split(cera_hip_ctx* ctx, AArgs& a, bool f32, bool fused, SAttnPartials* merge) {
     const uint32_t tiles = (a.n * a.per + 15) / 16, wgs = tiles * a.kv_heads;
     const uint32_t nb = fused ? a.start / 32 + 1 - (a.chunk ? a.start - a.start % a.chunk : 0) / 32 : max_blocks(a);
     // two blocks per wavefront before a second workgroup takes a share; one round of the chip at most
     a.splits = std::max(1u, std::min({(nb + 2 * SPLIT_WAVES - 1) / (2 * SPLIT_WAVES), std::max(1u, 2 * ctx->n_cu / wgs), 64u}));
-    if (a.splits > 1) {
+    if (merge) {
+        *merge = SAttnPartials{};
+        const uint32_t fine = std::min((nb + SPLIT_WAVES - 1) / SPLIT_WAVES, SATTN_MERGE_SPLITS);
+        if (nb <= SATTN_MERGE_SPLITS * SPLIT_WAVES * 4) a.splits = fine;   // one block per wavefront, four at the most
+        else merge = nullptr;
+    }
+    if (a.splits > 1 || merge) {
         void* part;
         CERA_TRY(cera_scratch(ctx, 10, static_cast<uint64_t>(a.splits) * a.n * a.heads * a.vdim_p * sizeof(float), &part));
         a.part = static_cast<float*>(part);
@@ -483,7 +510,10 @@ cera_hip_status run_split(cera_hip_ctx* ctx, AArgs& a, bool f32, bool fused) {
         }
     });
     HIP_TRY(ctx, hipGetLastError());
-    if (a.splits > 1) {
+    if (merge) {
+        merge->part = a.part; merge->splits = a.splits; merge->heads = a.heads; merge->vdim = a.vdim; merge->vdim_p = a.vdim_p;
+        merge->gate = a.qkvg + a.heads * a.dim + a.kv_heads * (a.dim + a.vdim);
+    } else if (a.splits > 1) {
         const dim3 mg((a.n * a.heads * (a.vdim_p / 4) + 255) / 256);
         if (f32) hipLaunchKernelGGL(sattn_merge_kernel<float>, mg, dim3(256), 0, ctx->stream, a);
         else hipLaunchKernelGGL(sattn_merge_kernel<__bf16>, mg, dim3(256), 0, ctx->stream, a);
@@ -516,7 +546,7 @@ cera_hip_status cera_launch_sattn(cera_hip_ctx* ctx, const SAttnShape& s, const 
     CERA_TRY(fill(ctx, s, p, &a));
     const uint32_t cols = p.n * a.per;
     // too few columns to fill the chip with a wavefront each: share the keys out instead
-    if (static_cast<uint64_t>(cols) / 16 * s.kv_heads < 2 * ctx->n_cu) return run_split(ctx, a, f32, false);
+    if (static_cast<uint64_t>(cols) / 16 * s.kv_heads < 2 * ctx->n_cu) return run_split(ctx, a, f32, false, nullptr);
     const bool wide = static_cast<uint64_t>(cols) / 32 * s.kv_heads >= 4 * ctx->n_cu;
     by_size(a, f32, [&](auto dk, auto vt) {
         constexpr int DK = decltype(dk)::value, VT = decltype(vt)::value;
@@ -531,18 +561,19 @@ cera_hip_status cera_launch_sattn(cera_hip_ctx* ctx, const SAttnShape& s, const 
 }
 
 cera_hip_status cera_launch_sattn_step(cera_hip_ctx* ctx, const SAttnShape& s, const SAttnPass& p, const ConvRing& ring,
-                                       const ConvHist& hist, bool f32) {
+                                       const ConvHist& hist, SAttnPartials* merge, bool f32) {
+    if (merge) *merge = SAttnPartials{};
     AArgs a;
     CERA_TRY(fill(ctx, s, p, &a));
     if (p.n != 1) return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "sigmoid attention step: one token");
     if (a.per > 16) {   // more query heads per kv head than one tile of columns: separate append
         CERA_TRY(cera_launch_sattn_append(ctx, s, p, ConvRing{}, nullptr, 0, nullptr, nullptr, f32));
         if (ring.rows) CERA_TRY(cera_launch_conv_hist(ctx, ring, hist, p.start + 1));
-        return run_split(ctx, a, f32, false);
+        return run_split(ctx, a, f32, false, nullptr);
     }
     a.ring = ring;
     a.hist = hist;
-    return run_split(ctx, a, f32, true);
+    return run_split(ctx, a, f32, true, merge);
 }
 
 cera_hip_status cera_launch_conv_hist(cera_hip_ctx* ctx, const ConvRing& ring, const ConvHist& hist, uint32_t pos) {

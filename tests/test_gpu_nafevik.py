@@ -12,7 +12,7 @@ from cera_amd import _build, hip_api, llama_api
 
 pytestmark = pytest.mark.gpu
 
-TOL = {True: 3e-5, False: 3e-2}   # f32, bf16
+TOL = {True: 1e-5, False: 3e-2}   # f32, bf16
 DTYPES = pytest.mark.parametrize("f32", [True, False], ids=["f32", "bf16"])
 
 
