@@ -7,7 +7,7 @@
 //                    [--kv f32|f16] [--dtype bf16|f32]
 //   cera-hip trace   --model DIR --out DIR [--dtype bfloat16|float32] [--max-tokens N]
 //
-// --model of `run` is a GGUF file or a directory with config.json and model.safetensors (--dtype is
+// --model of `inspect` and `run` is a GGUF file or a directory with config.json and model.safetensors (--dtype is
 // for the latter).  `trace` replays given requests from standard input (trace.h).
 //
 // `run` is the workload `cera bench` times (cera-cli/src/main.rs:932-938 for the
@@ -26,6 +26,7 @@
 #include "cera_host.h"
 #include "gguf.h"
 #include "load_model.h"
+#include "safetensors.h"
 #include "trace.h"
 
 namespace {
@@ -108,7 +109,25 @@ int cmd_gen(const Args& a) {
     return 0;
 }
 
+// a model directory: its config.json as it is, and the tensors
+int inspect_dir(const std::string& dir) {
+    std::ifstream f(dir + "/config.json");
+    if (!f) { std::fprintf(stderr, "%s/config.json cannot be read\n", dir.c_str()); return 1; }
+    for (std::string line; std::getline(f, line);) std::printf("%s\n", line.c_str());
+    std::string err;
+    auto st = cera::SafeTensors::open(dir + "/model.safetensors", &err);
+    if (!st) { std::fprintf(stderr, "%s\n", err.c_str()); return 1; }
+    for (const auto& kv : st->tensors()) {
+        std::printf("%-32s %-5s [", kv.first.c_str(), kv.second.dtype.c_str());
+        for (size_t i = 0; i < kv.second.shape.size(); ++i)
+            std::printf("%s%llu", i ? ", " : "", static_cast<unsigned long long>(kv.second.shape[i]));
+        std::printf("]  %llu bytes\n", static_cast<unsigned long long>(kv.second.nbytes));
+    }
+    return 0;
+}
+
 int cmd_inspect(const Args& a) {
+    if (cera::is_model_dir(a.str("model", ""))) return inspect_dir(a.str("model", ""));
     std::string err;
     auto g = cera::GgufFile::open(a.str("model", ""), &err);
     if (!g) { std::fprintf(stderr, "%s\n", err.c_str()); return 1; }

@@ -374,15 +374,24 @@ __global__ __launch_bounds__(SPLIT_WAVES * 64) void sattn_split_kernel(AArgs a) 
         }
 }
 
+// One workgroup per (query, head): a thread holds four value columns of every `groups`-th partial result.
 template <typename T>
 __global__ __launch_bounds__(256) void sattn_merge_kernel(AArgs a) {
-    const uint32_t quads = a.heads * (a.vdim_p / 4), t = blockIdx.x * 256 + threadIdx.x;
-    if (t >= quads * a.n) return;
-    const uint32_t query = t / quads, head = t % quads / (a.vdim_p / 4), v = t % (a.vdim_p / 4) * 4;
-    const float* p = a.part + (static_cast<uint64_t>(query) * a.heads + head) * a.vdim_p + v;
+    __shared__ __align__(16) f32x4 red[256];
+    const uint32_t quads = a.vdim_p / 4, groups = 256 / quads, q = threadIdx.x % quads, grp = threadIdx.x / quads;
+    const uint32_t query = blockIdx.x / a.heads, head = blockIdx.x % a.heads;
+    const uint64_t slice = static_cast<uint64_t>(a.n) * a.heads * a.vdim_p;
+    const float* p = a.part + (static_cast<uint64_t>(query) * a.heads + head) * a.vdim_p + q * 4;
     f32x4 s{0.f, 0.f, 0.f, 0.f};
-    for (uint32_t z = 0; z < a.splits; ++z) s += *reinterpret_cast<const f32x4*>(p + static_cast<uint64_t>(z) * a.n * a.heads * a.vdim_p);
-    if (v < a.vdim) finish4<T>(a, query, head, v, s);
+    if (grp < groups) {
+#pragma unroll 4
+        for (uint32_t z = grp; z < a.splits; z += groups) s += *reinterpret_cast<const f32x4*>(p + z * slice);
+    }
+    red[threadIdx.x] = s;
+    __syncthreads();
+    if (grp != 0) return;
+    for (uint32_t i = 1; i < groups; ++i) s += red[i * quads + q];
+    if (q * 4 < a.vdim) finish4<T>(a, query, head, q * 4, s);
 }
 
 // ---- append ---------------------------------------------------------------------------------------
@@ -488,7 +497,7 @@ cera_hip_status run_split(cera_hip_ctx* ctx, AArgs& a, bool f32, bool fused, SAt
     if (merge) {
         *merge = SAttnPartials{};
         const uint32_t fine = std::min((nb + SPLIT_WAVES - 1) / SPLIT_WAVES, SATTN_MERGE_SPLITS);
-        if (nb <= SATTN_MERGE_SPLITS * SPLIT_WAVES * 4) a.splits = fine;   // one block per wavefront, four at the most
+        if (nb <= SATTN_MERGE_SPLITS * SPLIT_WAVES * 2) a.splits = fine;   // one block per wavefront, two at the most
         else merge = nullptr;
     }
     if (a.splits > 1 || merge) {
@@ -514,7 +523,7 @@ cera_hip_status run_split(cera_hip_ctx* ctx, AArgs& a, bool f32, bool fused, SAt
         merge->part = a.part; merge->splits = a.splits; merge->heads = a.heads; merge->vdim = a.vdim; merge->vdim_p = a.vdim_p;
         merge->gate = a.qkvg + a.heads * a.dim + a.kv_heads * (a.dim + a.vdim);
     } else if (a.splits > 1) {
-        const dim3 mg((a.n * a.heads * (a.vdim_p / 4) + 255) / 256);
+        const dim3 mg(a.n * a.heads);
         if (f32) hipLaunchKernelGGL(sattn_merge_kernel<float>, mg, dim3(256), 0, ctx->stream, a);
         else hipLaunchKernelGGL(sattn_merge_kernel<__bf16>, mg, dim3(256), 0, ctx->stream, a);
         HIP_TRY(ctx, hipGetLastError());

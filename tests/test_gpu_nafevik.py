@@ -289,6 +289,22 @@ def test_long_prompts_take_the_large_tiles(tmp_path, f32):
     m.close()
 
 
+@DTYPES
+def test_steps_behind_a_very_long_context(tmp_path, f32):
+    """Thousands of visible keys: decode steps and short portions split them over many workgroups."""
+    cfg = U.config([U.attention(4, 2, 64, 64, None, 64, 10000.0, U.YARN, ff=48), U.attention(2, 1, 24, 36, 4320, 16, 900.0)],
+                   width=48, vocab=30, taps=3, positions=4400)
+    w = R.random_model(cfg, 43)
+    m = _open(U.save(tmp_path / "m", cfg, w), f32, 4400)
+    toks = U.tokens(cfg, 4330, 3)
+    want = U.reference(cfg, w, toks)[4300:]
+    m.forward_prefill(toks[:4300], 0)
+    got = np.concatenate([m.forward(int(toks[4300]), 4300)[None], m.forward_prefill_logits_all(toks[4301:4303], 4301),
+                          m.forward_prefill_logits_all(toks[4303:4312], 4303)] + [m.forward(int(t), 4312 + i)[None] for i, t in enumerate(toks[4312:])])
+    assert U.rel(got, want) < TOL[f32]
+    m.close()
+
+
 def test_inputs_too_wide_for_the_gemv_take_the_gemm(hip):
     """A feed-forward wider than a workgroup's LDS: the decode step runs as a pass of one token."""
     cfg = U.config([U.attention(2, 1, 32, 32, 16, 32, 100.0, ff=16400)], width=64, vocab=24, taps=3)

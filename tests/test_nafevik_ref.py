@@ -87,6 +87,14 @@ def test_loader_refuses_what_it_cannot_run(tmp_path):
     assert "offsets outside the file" in _open_error(d)
 
 
+def test_inspect_lists_a_model_directory(tmp_path):
+    cfg = U.CONFIGS["plain"]
+    d = U.save(tmp_path / "m", cfg, R.random_model(cfg, 2))
+    r = subprocess.run([str(_build.CLI_BIN), "inspect", "--model", str(d)], capture_output=True, text=True, timeout=60)
+    assert r.returncode == 0 and '"architecture": "Nafevik"' in r.stdout
+    assert [line.split()[:2] for line in r.stdout.splitlines() if line.startswith("l1.mix.o")] == [["l1.mix.o", "BF16"]]
+
+
 def test_trace_runner_arguments():
     assert _build.TRACE_BIN.exists(), "cera-trace missing: run __graft_entry__.build()"
     run = lambda *a: subprocess.run([str(_build.TRACE_BIN), *a], capture_output=True, text=True, input="", timeout=60)  # noqa: E731
