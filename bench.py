@@ -268,8 +268,8 @@ def nafevik_model(ctx, hip_api, size, rng, f32=False):
              "mix.v": mat(G * D, W), "mix.g": mat(Hq, W), "mix.o": mat(W, Hq * D), "mlp.gate": mat(FF, W), "mlp.up": mat(FF, W), "mlp.down": mat(W, FF)}
     spec = {"type": "attention", "mlp": {"kind": "dense", "ff": FF},
             "mixer": {"heads": Hq, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": 2048},
-                      "rot": {"dims": D, "base": 50000.0, "scaling": {"factor": 8.0, "original": 1024, "fast": 32.0, "slow": 1.0}}}}
-    cfg = {"width": W, "vocab": DESIGN_VOCAB, "canon": {"taps": 4}, "norm": {"eps": 1e-6}, "residual_mult": 0.7, "max_positions": DESIGN_CTX,
+                      "rot": {"dims": D, "base": 100000.0, "scaling": {"factor": 4.0, "original": 2048, "fast": 24.0, "slow": 2.0}}}}
+    cfg = {"width": W, "vocab": DESIGN_VOCAB, "canon": {"taps": 4}, "norm": {"eps": 1e-5}, "residual_mult": 0.5, "max_positions": DESIGN_CTX,
            "layers": [spec] * DESIGN_LAYERS, "loop": {"start": 2, "stop": DESIGN_LAYERS, "times": 1}}
     weights = {f"l{i}.{k}": v for i in range(DESIGN_LAYERS) for k, v in layer.items()}
     weights.update({"embed": mat(DESIGN_VOCAB, W, 1.0), "pos": mat(DESIGN_CTX, W), "head": mat(DESIGN_VOCAB, W), "final.norm": 1 + vec(W),

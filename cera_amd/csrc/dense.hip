@@ -243,6 +243,11 @@ __global__ __launch_bounds__(256) void dense_reduce_kernel(GemmDArgs a, uint32_t
     const float* p = a.part + static_cast<uint64_t>(tok) * a.m;
     auto sum4 = [&](uint32_t row) {
         f32x4 v{0.f, 0.f, 0.f, 0.f};
+        if ((a.m & 3) == 0) {
+#pragma unroll 4
+            for (uint32_t z = 0; z < split; ++z) v += *reinterpret_cast<const f32x4*>(p + z * slice + row);
+            return v;
+        }
         for (uint32_t z = 0; z < split; ++z) {
             const float* s = p + z * slice + row;
 #pragma unroll
@@ -492,7 +497,7 @@ cera_hip_status cera_launch_dense_gemm(cera_hip_ctx* ctx, const DenseMat& w, con
     uint32_t bm = 64, bn = 32;
     auto count = [&](uint32_t tm, uint32_t tn) { return static_cast<uint64_t>((a.m + tm - 1) / tm) * ((n + tn - 1) / tn); };
     if (f32) { bm = bn = 64; }
-    else if (n > 64 && count(128, 128) >= ctx->n_cu) { shape = 0; bm = bn = 128; }
+    else if (n > 64 && (count(128, 128) >= ctx->n_cu || (a.kp >= 8192 && count(128, 128) * 4 >= ctx->n_cu))) { shape = 0; bm = bn = 128; }
     else if (n > 32) { shape = 1; bm = bn = 64; }
     a.tiles_m = (a.m + bm - 1) / bm;
     a.tiles_n = (n + bn - 1) / bn;
