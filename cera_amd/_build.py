@@ -29,7 +29,8 @@ HSACO = LIB_DIR / "cera_hip_gfx950.hsaco"
 
 HIP_SRCS = sorted((PKG / "csrc").glob("*.hip"))
 # what the layered float models need of csrc/
-LAYERED_SRCS = [PKG / "csrc" / f"{n}.hip" for n in ("ctx", "model_api", "layered", "dense", "sigmoid_attn", "conv_norm")]
+LAYERED_SRCS = [PKG / "csrc" / f"{n}.hip" for n in ("ctx", "model_api", "layered", "layered_seq", "dense", "sigmoid_attn", "softmax_attn",
+                                                      "latent", "conv_norm")]
 HOST_SRCS = sorted((PKG / "host").glob("*.cpp"))
 
 # -ffp-contract=off: the parity target never fuses a*b+c implicitly; FMAs in
@@ -133,7 +134,7 @@ def build_backend(verbose: bool = False) -> Path:
     b = PKG / "backend"
     # C++ classes are not exported by the host library: compile them in
     host = [str(PKG / "host" / f) for f in ("gguf.cpp", "json.cpp", "safetensors.cpp")]
-    models = [str(b / f) for f in ("hip_device_model.cpp", "hip_llama.cpp", "hip_layered.cpp", "load_dir.cpp", "load_model.cpp")]
+    models = [str(b / f) for f in ("hip_device_model.cpp", "hip_llama.cpp", "hip_layered.cpp", "nafevik.cpp", "fidinex.cpp", "load_dir.cpp", "load_model.cpp")]
     cmds = [
         [*common, "-shared", *models, str(b / "hip_llama_capi.cpp"), *host, "-o", str(LLAMA_LIB), *link],
         [*common, str(b / "cli.cpp"), str(b / "trace.cpp"), *models, *host, "-o", str(CLI_BIN), *link],
@@ -164,7 +165,7 @@ def build_trace(verbose: bool = False, objs=None, jobs: int = 8) -> Path:
         objs = compile_hip(LAYERED_SRCS, verbose, jobs)
     link_hip(objs, LAYERED_LIB, verbose)
     b, host = PKG / "backend", PKG / "host"
-    srcs = [b / "trace_run.cpp", b / "trace.cpp", b / "hip_device_model.cpp", b / "hip_layered.cpp", b / "load_dir.cpp",
+    srcs = [b / "trace_run.cpp", b / "trace.cpp", b / "hip_device_model.cpp", b / "hip_layered.cpp", b / "nafevik.cpp", b / "fidinex.cpp", b / "load_dir.cpp",
             host / "json.cpp", host / "safetensors.cpp"]
     _run(["g++", "-O2", "-std=c++17", "-fPIC", "-pthread", "-Wall", "-Wextra", "-fvisibility=hidden", f"-I{ROOT / 'include'}",
           f"-I{host}", f"-I{b}", *map(str, srcs), "-o", str(TRACE_BIN), f"-L{LIB_DIR}", "-lcera_hip_layered", "-lcera_host",

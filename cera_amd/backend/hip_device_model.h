@@ -27,13 +27,13 @@ public:
     uint64_t gpu_memory_bytes() const override;
     virtual KvCompression kv_compression() const { return KvCompression::None; }
     std::string device_name() const;
+    // floats of one cached K row / V row / the convolution state of a layer (0: none)
+    struct LayerState { size_t k = 0, v = 0, conv = 0; };
 
 protected:
     HipDeviceModel() = default;
     [[noreturn]] void device_panic(const char* what) const;
     void open_context(int device);
-    // floats of one cached K row / V row / the convolution state of layer `l` (0: none)
-    struct LayerState { size_t k = 0, v = 0, conv = 0; };
     virtual LayerState layer_state(size_t l) const = 0;
     virtual size_t state_layers() const { return config_.n_layers; }
 

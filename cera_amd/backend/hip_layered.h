@@ -1,10 +1,5 @@
 // HipLayeredModel: models described layer by layer in a config.json, with bfloat16 weights in a
-// model.safetensors beside it, over cera_hip_layered_create.
-//
-// Architectures: "Nafevik" -- embedding plus learned positions; parallel attention and gated
-// feed-forward behind one RMS norm, each reading its input through a short causal convolution; sigmoid
-// attention inside chunks, with YaRN rotation in adjacent pairs and a gate per head; a range of
-// layers run several times, each pass starting from a product over the residual and the embedding.
+// model.safetensors beside it, over cera_hip_layered_create.  One reader per architecture (layered_reader.h).
 #pragma once
 #include <memory>
 
@@ -12,12 +7,16 @@
 #include "load_model.h"
 
 namespace cera {
+namespace layered { struct Description; }
 
 class HipLayeredModel final : public HipDeviceModel {
 public:
-    // dir holds config.json (parsed: config) and model.safetensors.  Throws BackendError with the
+    using HipDeviceModel::LayerState;
+    // dir holds config.json (parsed: config) and model.safetensors.  Throw BackendError with the
     // reason on any failure.
-    static std::unique_ptr<Model> from_dir(const std::string& dir, const Json& config, const LoadOptions& opt);
+    static std::unique_ptr<Model> nafevik(const std::string& dir, const Json& config, const LoadOptions& opt);
+    static std::unique_ptr<Model> fidinex(const std::string& dir, const Json& config, const LoadOptions& opt);
+    static std::unique_ptr<Model> create(const ModelConfig& c, const layered::Description& d, const LoadOptions& opt);
 
 private:
     HipLayeredModel() = default;

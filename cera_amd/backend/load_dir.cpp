@@ -15,7 +15,8 @@ struct DirModel {
     std::unique_ptr<Model> (*load)(const std::string& dir, const Json& config, const LoadOptions& opt);
 };
 const DirModel MODELS[] = {
-    {"Nafevik", HipLayeredModel::from_dir},
+    {"Nafevik", HipLayeredModel::nafevik},
+    {"Fidinex", HipLayeredModel::fidinex},
 };
 
 }  // namespace

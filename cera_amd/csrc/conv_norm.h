@@ -8,6 +8,10 @@
 cera_hip_status cera_launch_embed_pos(cera_hip_ctx* ctx, const void* embed, const void* pos, const uint32_t* tokens, uint32_t token,
                                       uint32_t n, uint32_t start, uint32_t width, uint64_t ld, float* x, float* x0);
 
+// x_s[t] = embed[token[t]] for every one of `streams` streams, `stride` floats apart, and u[t] = u_scale * embed[token[t]]
+cera_hip_status cera_launch_embed_streams(cera_hip_ctx* ctx, const void* embed, const uint32_t* tokens, uint32_t token, uint32_t n, uint32_t width,
+                                          uint64_t ld, float* x, uint32_t streams, uint64_t stride, float u_scale, float* u);
+
 // h = rmsnorm(x) per row; out_a = h + conv(h; wa), out_b likewise (nullable), T [n][ld].  wa / wb:
 // [taps][ld] f32, tap taps-1 the current position; taps == 0: out_a = h.  Rows before the pass come from the ring.
 struct NormConv {

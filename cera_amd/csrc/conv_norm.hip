@@ -19,6 +19,17 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(const uint16_t* __restri
     x0[t * ld + c] = v;
 }
 
+__global__ __launch_bounds__(256) void embed_streams_kernel(const uint16_t* __restrict__ embed, const uint32_t* __restrict__ tokens, uint32_t token,
+                                                            uint32_t width, uint64_t ld, float* __restrict__ x, uint32_t streams, uint64_t stride,
+                                                            float u_scale, float* __restrict__ u) {
+    const uint32_t t = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
+    if (c >= ld) return;
+    const uint64_t tok = tokens ? tokens[t] : token;
+    const float v = c < width ? bf16_at(embed, tok * width + c) : 0.0f;
+    for (uint32_t s = 0; s < streams; ++s) x[s * stride + t * ld + c] = v;
+    u[t * ld + c] = u_scale * v;
+}
+
 // A workgroup takes `rows` consecutive rows: first 1 / rms of those rows and of the taps - 1 before them
 // (recomputed, so that workgroups need nothing from each other), one row per wavefront; then the channels,
 // four per thread, walking down the rows.  TAPS > 0: the window of rows and the taps' weights stay in
@@ -116,6 +127,14 @@ cera_hip_status cera_launch_embed_pos(cera_hip_ctx* ctx, const void* embed, cons
                                       uint32_t n, uint32_t start, uint32_t width, uint64_t ld, float* x, float* x0) {
     hipLaunchKernelGGL(embed_pos_kernel, dim3(static_cast<uint32_t>((ld + 255) / 256), n), dim3(256), 0, ctx->stream,
                        static_cast<const uint16_t*>(embed), static_cast<const uint16_t*>(pos), tokens, token, start, width, ld, x, x0);
+    HIP_TRY(ctx, hipGetLastError());
+    return CERA_HIP_OK;
+}
+
+cera_hip_status cera_launch_embed_streams(cera_hip_ctx* ctx, const void* embed, const uint32_t* tokens, uint32_t token, uint32_t n, uint32_t width,
+                                          uint64_t ld, float* x, uint32_t streams, uint64_t stride, float u_scale, float* u) {
+    hipLaunchKernelGGL(embed_streams_kernel, dim3(static_cast<uint32_t>((ld + 255) / 256), n), dim3(256), 0, ctx->stream,
+                       static_cast<const uint16_t*>(embed), tokens, token, width, ld, x, streams, stride, u_scale, u);
     HIP_TRY(ctx, hipGetLastError());
     return CERA_HIP_OK;
 }

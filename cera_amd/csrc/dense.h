@@ -17,7 +17,19 @@ struct DenseMat {
 enum DenseEpilogue {
     DENSE_STORE = 0,    // out[row] = y (+ bias[row])                        f32
     DENSE_ADD = 1,      // out[row] += mult * y                              f32
-    DENSE_SWIGLU = 2    // rows come in groups of 16 gate rows then 16 up rows: out[i] = silu(gate_i) * up_i   element type
+    DENSE_SWIGLU = 2,   // rows come in groups of 16 gate rows then 16 up rows: out[i] = silu(gate_i) * up_i   element type
+    DENSE_CAST = 3,     // out[row] = y                                       element type
+    DENSE_RELU2 = 4,    // out[row] = max(y, 0)^2                             element type
+    DENSE_STREAMS = 5   // adds y to several residual streams at once (DenseStreams)          f32
+};
+// Residual streams x_0 .. x_{count-1}: x_t <- sum_s mix[s][t] x_s + out[t] y, all from the old ones, and the next
+// reader's input u = sum_t next[t] x_t on the way.  DenseOut::out is x_0, the others follow `stride` floats apart.
+constexpr uint32_t DENSE_MAX_STREAMS = 8;
+struct DenseStreams {
+    uint32_t count = 0;
+    uint64_t stride = 0;
+    float out[DENSE_MAX_STREAMS] = {}, next[DENSE_MAX_STREAMS] = {};
+    float mix[DENSE_MAX_STREAMS][DENSE_MAX_STREAMS] = {};   // [from][to]
 };
 struct DenseOut {
     int epi = DENSE_STORE;
@@ -26,16 +38,24 @@ struct DenseOut {
     const float* bias = nullptr;  // DENSE_STORE, nullable
     float mult = 1.0f;            // DENSE_ADD
     uint32_t rows = 0;            // output elements per token
+    const DenseStreams* streams = nullptr;   // DENSE_STREAMS, host
+    float* u = nullptr;                      // DENSE_STREAMS: the next reader's input, rows as x's
+};
+// Several products of the same shape in one launch, as the heads of a layer have them: number g reads rows
+// [g * w.rows / count, ...) of the matrix and its own columns of x, and writes its own columns of out.
+struct DenseGroups {
+    uint32_t count = 1;
+    uint64_t x_stride = 0, out_stride = 0;   // elements between the groups' x and out
 };
 
 // many tokens: x [n][ldx] of bf16 (f32 == false) or float, ldx >= w.kp
 cera_hip_status cera_launch_dense_gemm(cera_hip_ctx* ctx, const DenseMat& w, const void* x, uint64_t ldx, uint32_t n,
-                                       const DenseOut& o, bool f32);
+                                       const DenseOut& o, bool f32, const DenseGroups& groups = {});
 
 // One token.  Where its activations come from:
 struct DenseIn {
     // RAW: element-type vector [kp].  NORM: x f32 [kp], normalised over its first n_mean entries.
-    // MERGE: as RAW, but the first heads * vdim elements are the sum of attention's partial results, gated.
+    // MERGE: as RAW, but the first heads * vdim elements are the sum of attention's partial results.
     // CONCAT: x | x2, f32 [kp / 2] each.  Pad columns of x, x2, scale, add and plain are zero.
     enum Kind { RAW = 0, NORM = 1, CONCAT = 2, MERGE = 3 } kind = RAW;
     const void* x = nullptr;

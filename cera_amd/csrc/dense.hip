@@ -13,6 +13,7 @@
 
 #include "bf16.hip.h"
 #include "dense.h"
+#include "partials.hip.h"
 
 namespace {
 
@@ -29,13 +30,82 @@ struct GemmDArgs {
     float mult;
     uint32_t out_rows;
     float* part;           // split K: [split][n][m] f32
+    uint64_t gw, gx, go;   // groups (blockIdx.z): elements between their matrices, inputs and outputs
+    bool vec;              // four outputs of a token in a row may be stored as one vector
+    float* u;
+    DenseStreams st;
 };
 
+// four consecutive channels of every stream (n < 4: the first n of them)
+template <int S> __device__ __forceinline__ void dense_streams4(const DenseStreams& st, float* x, float* u, bool vec, int n, const float (&y)[4]) {
+    float o[S][4];
+#pragma unroll
+    for (int s = 0; s < S; ++s)
+        if (s < static_cast<int>(st.count)) {
+            float* const p = x + s * st.stride;
+            if (vec) {
+                const float4 v = *reinterpret_cast<const float4*>(p);
+                o[s][0] = v.x; o[s][1] = v.y; o[s][2] = v.z; o[s][3] = v.w;
+            } else {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) o[s][i] = i < n ? p[i] : 0.0f;
+            }
+        }
+    float sum[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int t = 0; t < S; ++t)
+        if (t < static_cast<int>(st.count)) {
+            float v[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                v[i] = st.out[t] * y[i];
+#pragma unroll
+                for (int s = 0; s < S; ++s)
+                    if (s < static_cast<int>(st.count)) v[i] = fmaf(st.mix[s][t], o[s][i], v[i]);
+                sum[i] = fmaf(st.next[t], v[i], sum[i]);
+            }
+            float* const p = x + t * st.stride;
+            if (vec) *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+            else
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                    if (i < n) p[i] = v[i];
+        }
+    if (vec) *reinterpret_cast<float4*>(u) = make_float4(sum[0], sum[1], sum[2], sum[3]);
+    else
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+            if (i < n) u[i] = sum[i];
+}
+// one channel of every stream
+__device__ __forceinline__ void dense_streams1(const DenseStreams& st, float* x, float* u, float y) {
+    float o[DENSE_MAX_STREAMS], sum = 0.0f;
+#pragma unroll
+    for (int s = 0; s < static_cast<int>(DENSE_MAX_STREAMS); ++s)
+        if (s < static_cast<int>(st.count)) o[s] = x[s * st.stride];
+#pragma unroll
+    for (int t = 0; t < static_cast<int>(DENSE_MAX_STREAMS); ++t)
+        if (t < static_cast<int>(st.count)) {
+            float v = st.out[t] * y;
+#pragma unroll
+            for (int s = 0; s < static_cast<int>(DENSE_MAX_STREAMS); ++s)
+                if (s < static_cast<int>(st.count)) v = fmaf(st.mix[s][t], o[s], v);
+            x[t * st.stride] = v;
+            sum = fmaf(st.next[t], v, sum);
+        }
+    *u = sum;
+}
+__device__ __forceinline__ float dense_relu2(float y) {
+    const float r = fmaxf(y, 0.0f);
+    return r * r;
+}
+
 // ---- epilogues on four consecutive rows m .. m+3 of one token -----------------------------------
-__device__ __forceinline__ void dense_store4(const GemmDArgs& a, uint32_t row, uint32_t tok, f32x4 v) {
+template <typename T> __device__ __forceinline__ void dense_store4(const GemmDArgs& a, uint32_t row, uint32_t tok, f32x4 v) {
+    const uint64_t at = blockIdx.z * a.go + static_cast<uint64_t>(tok) * a.ldo + row;
     if (a.epi == DENSE_STORE) {
-        float* o = static_cast<float*>(a.out) + static_cast<uint64_t>(tok) * a.ldo + row;
-        if (row + 4 <= a.m && (a.ldo & 3) == 0) {
+        float* o = static_cast<float*>(a.out) + at;
+        if (row + 4 <= a.m && a.vec) {
             if (a.bias) {
                 const float4 b = *reinterpret_cast<const float4*>(a.bias + row);
                 v.x += b.x; v.y += b.y; v.z += b.z; v.w += b.w;
@@ -46,9 +116,25 @@ __device__ __forceinline__ void dense_store4(const GemmDArgs& a, uint32_t row, u
             for (int i = 0; i < 4; ++i)
                 if (row + i < a.m) o[i] = a.bias ? v[i] + a.bias[row + i] : v[i];
         }
+    } else if (a.epi == DENSE_CAST || a.epi == DENSE_RELU2) {
+        T* o = static_cast<T*>(a.out) + at;
+        if (a.epi == DENSE_RELU2) { v.x = dense_relu2(v.x); v.y = dense_relu2(v.y); v.z = dense_relu2(v.z); v.w = dense_relu2(v.w); }
+        if (row + 4 <= a.m && a.vec) {
+            ElemOps<T>::store4(o, v.x, v.y, v.z, v.w);
+        } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (row + i < a.m) o[i] = ElemOps<T>::from(v[i]);
+        }
+    } else if (a.epi == DENSE_STREAMS) {
+        const float y[4] = {v.x, v.y, v.z, v.w};
+        float* const x = static_cast<float*>(a.out) + at;
+        const int n = static_cast<int>(min(4u, a.m - row));
+        if (a.st.count <= 4) dense_streams4<4>(a.st, x, a.u + at, n == 4 && a.vec, n, y);
+        else dense_streams4<DENSE_MAX_STREAMS>(a.st, x, a.u + at, n == 4 && a.vec, n, y);
     } else {
-        float* o = static_cast<float*>(a.out) + static_cast<uint64_t>(tok) * a.ldo + row;
-        if (row + 4 <= a.m && (a.ldo & 3) == 0) {
+        float* o = static_cast<float*>(a.out) + at;
+        if (row + 4 <= a.m && a.vec) {
             float4 r = *reinterpret_cast<const float4*>(o);
             r.x = fmaf(a.mult, v.x, r.x); r.y = fmaf(a.mult, v.y, r.y);
             r.z = fmaf(a.mult, v.z, r.z); r.w = fmaf(a.mult, v.w, r.w);
@@ -106,7 +192,7 @@ __device__ __forceinline__ void dense_epilogue(const GemmDArgs& a, uint32_t m0, 
 #pragma unroll
             for (int mi = 0; mi < MI; ++mi) {
                 const uint32_t row = m0 + 16 * mi + g4;
-                if (row < a.m) dense_store4(a, row, tok, acc[mi][ni]);
+                if (row < a.m) dense_store4<T>(a, row, tok, acc[mi][ni]);
             }
         }
     }
@@ -132,14 +218,15 @@ __global__ __launch_bounds__(256) void dense_gemm_bf16_kernel(GemmDArgs a) {
     if (!dense_tile(a, tm, tn)) return;
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const uint32_t k0 = blockIdx.y * a.k_chunk, k1 = min(a.kp, k0 + a.k_chunk);
-    const __bf16* const x = static_cast<const __bf16*>(a.x);
+    const __bf16* const w = a.w + blockIdx.z * a.gw;
+    const __bf16* const x = static_cast<const __bf16*>(a.x) + blockIdx.z * a.gx;
     // this lane's source address per 1 KB piece; rows past the matrix / batch re-read the last one
     const uint32_t sub = lane >> 3, slot = lane & 7, chunk = (slot ^ sub) * 8;
     const __bf16* src[SEGS / 4];
 #pragma unroll
     for (int s = 0; s < SEGS / 4; ++s) {
         const uint32_t r = (wave * (SEGS / 4) + s) * 8 + sub;
-        src[s] = r < BM ? a.w + static_cast<uint64_t>(min(tm * BM + r, a.m - 1)) * a.kp + chunk
+        src[s] = r < BM ? w + static_cast<uint64_t>(min(tm * BM + r, a.m - 1)) * a.kp + chunk
                         : x + static_cast<uint64_t>(min(tn * BN + (r - BM), a.n - 1)) * a.ldx + chunk;
     }
     auto stage = [&](uint32_t k, int buf) {
@@ -192,9 +279,10 @@ __global__ __launch_bounds__(256) void dense_gemm_f32_kernel(GemmDArgs a) {
     if (!dense_tile(a, tm, tn)) return;
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const uint32_t k0 = blockIdx.y * a.k_chunk, k1 = min(a.kp, k0 + a.k_chunk);
-    const float* const x = static_cast<const float*>(a.x);
+    const __bf16* const w0 = a.w + blockIdx.z * a.gw;
+    const float* const x = static_cast<const float*>(a.x) + blockIdx.z * a.gx;
     const uint32_t r = threadIdx.x >> 2, c = (threadIdx.x & 3) * 8;   // eight k of one row per thread
-    const __bf16* const ws = a.w + static_cast<uint64_t>(min(tm * BM + r, a.m - 1)) * a.kp + c;
+    const __bf16* const ws = w0 + static_cast<uint64_t>(min(tm * BM + r, a.m - 1)) * a.kp + c;
     const float* const xs = x + static_cast<uint64_t>(min(tn * BN + r, a.n - 1)) * a.ldx + c;
     f32x4 acc[2][2];
 #pragma unroll
@@ -260,7 +348,7 @@ __global__ __launch_bounds__(256) void dense_reduce_kernel(GemmDArgs a, uint32_t
         const uint32_t row = (q >> 4) * 32 + (q & 15);
         dense_swiglu4<T>(a, q, tok, sum4(row), sum4(row + 16));
     } else {
-        dense_store4(a, q, tok, sum4(q));
+        dense_store4<T>(a, q, tok, sum4(q));
     }
 }
 
@@ -271,6 +359,7 @@ struct GemvDArgs {
     uint32_t rows_a, rows_b, kp, stage_len;   // stage_len: LDS elements, kp rounded up to a whole step of the wavefront
     uint32_t blocks_a, groups_a, groups_b, blocks_b;   // groups of R rows
     DenseOut oa, ob;
+    DenseStreams st;
 };
 
 constexpr int GEMV_WAVES = 8;
@@ -292,7 +381,6 @@ __device__ __forceinline__ void gemv_stage(const GemvDArgs& a, bool second, bool
         const T* x = static_cast<const T*>(in.x);
         const SAttnPartials& m = in.merge;
         const uint32_t cols = m.heads * m.vdim, cols_p = (cols + DENSE_PAD - 1) / DENSE_PAD * DENSE_PAD;
-        const uint64_t slice = static_cast<uint64_t>(m.heads) * m.vdim_p;
         constexpr uint32_t V = 16 / sizeof(T);
 #pragma unroll 4
         for (uint32_t i = cols_p + threadIdx.x * V; i < a.stage_len; i += GEMV_WAVES * 64 * V)
@@ -301,21 +389,12 @@ __device__ __forceinline__ void gemv_stage(const GemvDArgs& a, bool second, bool
         for (uint32_t i = threadIdx.x * 4; i < cols_p; i += GEMV_WAVES * 256) {
             if (i + 4 <= cols && m.vdim % 4 == 0) {
                 const uint32_t h = i / m.vdim;
-                const float* p = m.part + h * m.vdim_p + (i - h * m.vdim);
-                f32x4 s = *reinterpret_cast<const f32x4*>(p);
-#pragma unroll 4
-                for (uint32_t z = 1; z < m.splits; ++z) s += *reinterpret_cast<const f32x4*>(p + z * slice);
-                const float g = sigmoid_f32(m.gate[h]);
-                ElemOps<T>::store4(xs + i, s.x * g, s.y * g, s.z * g, s.w * g);
+                const f32x4 s = partials_sum4(m, h, i - h * m.vdim);
+                ElemOps<T>::store4(xs + i, s.x, s.y, s.z, s.w);
             } else {
 #pragma unroll
                 for (uint32_t e = i; e < i + 4; ++e) {
-                    float s = 0.0f;
-                    if (e < cols) {
-                        const uint32_t h = e / m.vdim;
-                        for (uint32_t z = 0; z < m.splits; ++z) s += m.part[z * slice + h * m.vdim_p + (e - h * m.vdim)];
-                        s *= sigmoid_f32(m.gate[h]);
-                    }
+                    const float s = e < cols ? partials_sum(m, e / m.vdim, e % m.vdim) : 0.0f;
                     xs[e] = ElemOps<T>::from(s);
                 }
             }
@@ -409,7 +488,7 @@ template <typename T, int R> struct GemvWalk {
         return true;
     }
     // multiplies a step of group g at k; at the group's last step reduces and stores, and moves on
-    __device__ __forceinline__ void use(const Buf& b, uint32_t& g, uint32_t& k, const T* xs, const DenseOut& o) {
+    __device__ __forceinline__ void use(const Buf& b, uint32_t& g, uint32_t& k, const T* xs, const DenseOut& o, const DenseStreams& st) {
 #pragma unroll
         for (int u = 0; u < U; ++u) {
             const typename ElemOps<T>::X8 xv = ElemOps<T>::ld8(xs + k + (u * 64 + lane) * 8);
@@ -437,7 +516,9 @@ template <typename T, int R> struct GemvWalk {
             if (lane < static_cast<uint32_t>(R) && i < rows) {
                 float* out = static_cast<float*>(o.out) + i;
                 if (o.epi == DENSE_ADD) *out = fmaf(o.mult, y, *out);
-                else *out = o.bias ? y + o.bias[i] : y;
+                else if (o.epi == DENSE_STORE) *out = o.bias ? y + o.bias[i] : y;
+                else if (o.epi == DENSE_STREAMS) dense_streams1(st, out, o.u + i, y);
+                else static_cast<T*>(o.out)[i] = ElemOps<T>::from(o.epi == DENSE_RELU2 ? dense_relu2(y) : y);
             }
         }
 #pragma unroll
@@ -467,10 +548,10 @@ __global__ __launch_bounds__(GEMV_WAVES * 64) void dense_gemv_kernel(GemvDArgs a
     gemv_stage<T, KIND>(a, second, KIND == DenseIn::NORM && a.in.h_out && blockIdx.x == 0, xs, red);
     while (more0) {
         const bool more1 = walk.load(w1);
-        walk.use(w0, g, k, xs, o);
+        walk.use(w0, g, k, xs, o, a.st);
         if (!more1) break;
         more0 = walk.load(w0);
-        walk.use(w1, g, k, xs, o);
+        walk.use(w1, g, k, xs, o, a.st);
     }
 }
 
@@ -478,6 +559,7 @@ constexpr uint64_t GEMV_LDS_MAX = 60 * 1024;
 
 }  // namespace
 
+static bool streams_ok(const DenseOut& o) { return o.streams && o.u && o.streams->count >= 1 && o.streams->count <= DENSE_MAX_STREAMS && o.streams->stride % 4 == 0; }
 static uint64_t gemv_stage_len(uint64_t kp, int r) {
     const uint64_t step = 64ull * 8 * (8 / r);
     return (kp + step - 1) / step * step;
@@ -485,17 +567,22 @@ static uint64_t gemv_stage_len(uint64_t kp, int r) {
 bool cera_dense_gemv_fits(uint64_t kp, bool f32) { return gemv_stage_len(kp, 1) * (f32 ? 4 : 2) <= GEMV_LDS_MAX; }
 
 cera_hip_status cera_launch_dense_gemm(cera_hip_ctx* ctx, const DenseMat& w, const void* x, uint64_t ldx, uint32_t n,
-                                       const DenseOut& o, bool f32) {
-    if (n == 0 || w.rows == 0 || w.kp == 0 || w.kp % DENSE_PAD || ldx < w.kp || ldx % 8)
+                                       const DenseOut& o, bool f32, const DenseGroups& groups) {
+    if (n == 0 || w.rows == 0 || groups.count == 0 || w.rows % groups.count || w.kp == 0 || w.kp % DENSE_PAD || ldx < w.kp || ldx % 8)
         return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemm: bad shape");
     if (o.epi == DENSE_SWIGLU && w.rows % 32) return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemm: gate | up rows come in groups of 32");
+    if (o.epi == DENSE_STREAMS && !streams_ok(o)) return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemm: streams");
     GemmDArgs a{};
-    a.w = static_cast<const __bf16*>(w.w); a.x = x; a.ldx = ldx; a.m = w.rows; a.n = n; a.kp = w.kp;
+    a.w = static_cast<const __bf16*>(w.w); a.x = x; a.ldx = ldx; a.m = w.rows / groups.count; a.n = n; a.kp = w.kp;
+    a.gw = static_cast<uint64_t>(a.m) * w.kp; a.gx = groups.x_stride; a.go = groups.out_stride;
+    a.vec = (o.ld & 3) == 0 && (groups.out_stride & 3) == 0;
+    a.u = o.u;
+    if (o.streams) a.st = *o.streams;
     a.epi = o.epi; a.out = o.out; a.ldo = o.ld; a.bias = o.bias; a.mult = o.mult; a.out_rows = o.rows;
     // tile: large where it fills the chip, else smaller, else K is split
     int shape = 2;
     uint32_t bm = 64, bn = 32;
-    auto count = [&](uint32_t tm, uint32_t tn) { return static_cast<uint64_t>((a.m + tm - 1) / tm) * ((n + tn - 1) / tn); };
+    auto count = [&](uint32_t tm, uint32_t tn) { return static_cast<uint64_t>((a.m + tm - 1) / tm) * ((n + tn - 1) / tn) * groups.count; };
     if (f32) { bm = bn = 64; }
     else if (n > 64 && (count(128, 128) >= ctx->n_cu || (a.kp >= 8192 && count(128, 128) * 4 >= ctx->n_cu))) { shape = 0; bm = bn = 128; }
     else if (n > 32) { shape = 1; bm = bn = 64; }
@@ -505,7 +592,7 @@ cera_hip_status cera_launch_dense_gemm(cera_hip_ctx* ctx, const DenseMat& w, con
     const uint32_t steps = a.kp / DENSE_PAD;
     uint32_t split = 1;
     const uint32_t want_wgs = 2 * ctx->n_cu;
-    if (wgs < want_wgs) split = static_cast<uint32_t>(std::min<uint64_t>({(want_wgs + wgs - 1) / wgs, steps / 4, 16}));
+    if (wgs < want_wgs && groups.count == 1) split = static_cast<uint32_t>(std::min<uint64_t>({(want_wgs + wgs - 1) / wgs, steps / 4, 16}));
     if (split < 1) split = 1;
     const uint32_t per = (steps + split - 1) / split;
     split = (steps + per - 1) / per;
@@ -515,7 +602,7 @@ cera_hip_status cera_launch_dense_gemm(cera_hip_ctx* ctx, const DenseMat& w, con
         CERA_TRY(cera_scratch(ctx, 9, static_cast<uint64_t>(split) * n * a.m * sizeof(float), &part));
         a.part = static_cast<float*>(part);
     }
-    const dim3 grid((a.tiles_m + 7) / 8 * 8 * a.tiles_n, split);
+    const dim3 grid((a.tiles_m + 7) / 8 * 8 * a.tiles_n, split, groups.count);
     if (f32) hipLaunchKernelGGL(dense_gemm_f32_kernel, grid, dim3(256), 0, ctx->stream, a);
     else if (shape == 0) hipLaunchKernelGGL((dense_gemm_bf16_kernel<128, 128, 2, 2>), grid, dim3(256), 0, ctx->stream, a);
     else if (shape == 1) hipLaunchKernelGGL((dense_gemm_bf16_kernel<64, 64, 2, 2>), grid, dim3(256), 0, ctx->stream, a);
@@ -536,7 +623,9 @@ cera_hip_status cera_launch_dense_gemv(cera_hip_ctx* ctx, const DenseIn& in, con
     *launched = false;
     if (wa.rows == 0 || wa.kp == 0 || wa.kp % DENSE_PAD || (wb && wb->kp != wa.kp))
         return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemv: bad shape");
+    if (oa.epi == DENSE_STREAMS && !streams_ok(oa)) return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemv: streams");
     GemvDArgs a{};
+    if (oa.streams) a.st = *oa.streams;
     a.in = in;
     a.wa = static_cast<const __bf16*>(wa.w); a.rows_a = wa.rows; a.kp = wa.kp; a.oa = oa;
     if (!cera_dense_gemv_fits(wa.kp, f32)) return CERA_HIP_OK;

@@ -1,0 +1,196 @@
+// Kernels of latent.h.
+#include <algorithm>
+
+#include "bf16.hip.h"
+#include "latent.h"
+#include "partials.hip.h"
+
+namespace {
+
+struct LArgs {
+    LatentShape l;
+    const float* x;
+    uint64_t ld;
+    uint32_t n, start, kp, rank_p, dim_p, row, rot_p;
+    void *cache, *q, *qn;
+    const __bf16* w;          // step: per-head matrices
+    uint32_t slices, rows;    // step: workgroups and rows per head
+    SAttnPartials parts;
+    void* out;
+};
+
+// entry c of a rotated part at `pos`
+__device__ __forceinline__ float rotated(const LatentShape& l, const float* x, uint32_t c, uint32_t pos) {
+    if (c >= l.rot_dims) return x[c];
+    const float* const cs = l.rot_table + static_cast<uint64_t>(pos) * l.rot_dims + (c & ~1u);
+    const float u = x[c & ~1u], v = x[c | 1u];
+    return c & 1 ? v * cs[0] + u * cs[1] : u * cs[0] - v * cs[1];
+}
+// by one wavefront: the cache row of a token
+template <typename T> __device__ __forceinline__ void latent_append(const LArgs& a, const float* down, uint32_t pos, uint32_t lane) {
+    const LatentShape& l = a.l;
+    T* const dst = static_cast<T*>(a.cache) + static_cast<uint64_t>(pos) * a.row;
+    float ss = 0.0f;
+    for (uint32_t c = lane; c < l.rank; c += 64) ss = fmaf(down[c], down[c], ss);
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(l.rank) + l.eps);
+    for (uint32_t c = lane; c < a.rank_p; c += 64) dst[c] = ElemOps<T>::from(c < l.rank ? down[c] * inv * l.c_norm[c] : 0.0f);
+    for (uint32_t c = lane; c < a.row - a.rank_p; c += 64)
+        dst[a.rank_p + c] = ElemOps<T>::from(c < l.rot_dim ? rotated(l, down + l.rank, c, pos) : 0.0f);
+}
+
+// a wavefront per query head, and one for the cache row
+template <typename T> __global__ __launch_bounds__(256) void latent_prep_kernel(LArgs a) {
+    const LatentShape& l = a.l;
+    const uint32_t lane = threadIdx.x & 63, item = blockIdx.x * 4 + (threadIdx.x >> 6), tok = blockIdx.y, pos = a.start + tok;
+    if (item > l.heads) return;
+    const float* const row = a.x + tok * a.ld;
+    if (item == l.heads) {
+        latent_append<T>(a, row + l.heads * (l.dim + l.rot_dim), pos, lane);
+        return;
+    }
+    const float* const x = row + item * (l.dim + l.rot_dim);
+    T* const q = static_cast<T*>(a.q) + (static_cast<uint64_t>(tok) * l.heads + item) * a.kp;
+    uint32_t at = l.dim;
+    if (a.qn) {
+        T* const qn = static_cast<T*>(a.qn) + (static_cast<uint64_t>(tok) * l.heads + item) * a.dim_p;
+        for (uint32_t c = lane; c < a.dim_p; c += 64) qn[c] = ElemOps<T>::from(c < l.dim ? x[c] : 0.0f);
+        at = a.rank_p;
+    } else {
+        for (uint32_t c = lane; c < l.dim; c += 64) q[c] = ElemOps<T>::from(x[c]);
+    }
+    for (uint32_t c = lane; at + c < a.kp; c += 64) q[at + c] = ElemOps<T>::from(c < l.rot_dim ? rotated(l, x + l.dim, c, pos) : 0.0f);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_spread_kernel(const T* __restrict__ cache, uint32_t cache_row, uint32_t rank_p, uint32_t rot_dim, uint32_t dim,
+                                                            uint32_t vdim, uint32_t v_off, uint32_t row, uint32_t total, uint32_t cap, T* __restrict__ rows) {
+    const uint32_t pos = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    T* const dst = rows + (static_cast<uint64_t>(blockIdx.y) * cap + pos) * row;
+    const T* const kr = cache + static_cast<uint64_t>(pos) * cache_row + rank_p;
+    const bool live = pos < total;
+    for (uint32_t c = lane; c < row; c += 64) {
+        if (live && (c < dim || (c >= v_off && c < v_off + vdim))) continue;   // the products' columns
+        dst[c] = live && c >= dim && c < dim + rot_dim ? kr[c - dim] : ElemOps<T>::from(0.0f);
+    }
+}
+
+// y[r] = w[r] . xs for rows r0 + 4 j + (lane / 16) of a matrix with k columns (a multiple of 64): sixteen lanes per row
+template <typename T> __device__ __forceinline__ float head_row_dot(const __bf16* w, uint64_t row, uint32_t k, const T* xs, uint32_t l16) {
+    const __bf16* const p = w + row * k;
+    float acc = 0.0f;
+#pragma unroll 4
+    for (uint32_t c = l16 * 8; c < k; c += 128) acc = ElemOps<T>::dot8(*reinterpret_cast<const uint4*>(p + c), ElemOps<T>::ld8(xs + c), acc);
+    return wave_row_sum(acc);
+}
+
+// workgroups (head, slice of the rank); the last one appends
+template <typename T> __global__ __launch_bounds__(256) void latent_step_kernel(LArgs a) {
+    extern __shared__ __align__(16) unsigned char smem[];
+    T* const xs = reinterpret_cast<T*>(smem);
+    const LatentShape& l = a.l;
+    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    if (blockIdx.x == l.heads * a.slices) {
+        if (wave == 0) latent_append<T>(a, a.x + l.heads * (l.dim + l.rot_dim), a.start, lane);
+        return;
+    }
+    const uint32_t head = blockIdx.x / a.slices, slice = blockIdx.x % a.slices;
+    const float* const x = a.x + head * (l.dim + l.rot_dim);
+    T* const q = static_cast<T*>(a.q) + static_cast<uint64_t>(head) * a.kp;
+    for (uint32_t c = threadIdx.x; c < a.dim_p; c += 256) xs[c] = ElemOps<T>::from(c < l.dim ? x[c] : 0.0f);
+    if (slice == 0)
+        for (uint32_t c = threadIdx.x; a.rank_p + c < a.kp; c += 256)
+            q[a.rank_p + c] = ElemOps<T>::from(c < l.rot_dim ? rotated(l, x + l.dim, c, a.start) : 0.0f);
+    __syncthreads();
+    const uint32_t r0 = slice * a.rows, r1 = min(r0 + a.rows, a.rank_p);
+    for (uint32_t r = r0 + wave * 4 + (lane >> 4); r < r1; r += 16) {   // row counts are multiples of 4: the lanes of a row stay together
+        const float y = head_row_dot<T>(a.w, static_cast<uint64_t>(head) * a.rank_p + r, a.dim_p, xs, lane & 15);
+        if ((lane & 15) == 0) q[r] = ElemOps<T>::from(y);
+    }
+}
+
+// workgroups (head, slice of its values)
+template <typename T> __global__ __launch_bounds__(256) void latent_values_kernel(LArgs a) {
+    extern __shared__ __align__(16) unsigned char smem[];
+    T* const xs = reinterpret_cast<T*>(smem);
+    const LatentShape& l = a.l;
+    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, head = blockIdx.x / a.slices, slice = blockIdx.x % a.slices;
+    for (uint32_t c = threadIdx.x * 4; c < a.rank_p; c += 1024) {
+        const f32x4 s = partials_sum4(a.parts, head, c);
+        ElemOps<T>::store4(xs + c, s.x, s.y, s.z, s.w);
+    }
+    __syncthreads();
+    const uint32_t r0 = slice * a.rows, r1 = min(r0 + a.rows, l.vdim);
+    for (uint32_t rb = r0 + wave * 4; rb < r1; rb += 16) {
+        const uint32_t r = rb + (lane >> 4);
+        const float y = head_row_dot<T>(a.w, static_cast<uint64_t>(head) * l.vdim + min(r, l.vdim - 1), a.rank_p, xs, lane & 15);
+        if ((lane & 15) == 0 && r < r1) static_cast<T*>(a.out)[head * l.vdim + r] = ElemOps<T>::from(y);
+    }
+}
+
+LArgs fill(const LatentShape& l, const FAttnShape& s) {
+    LArgs a{};
+    a.l = l;
+    a.rank_p = l.rank_p(); a.dim_p = l.dim_p(); a.row = s.row; a.kp = s.kp;
+    return a;
+}
+// rows per workgroup so that the heads' products spread over about two workgroups per CU
+void slice_rows(cera_hip_ctx* ctx, LArgs& a, uint32_t heads, uint32_t rows) {
+    const uint32_t want = std::max(1u, 2 * ctx->n_cu / heads);
+    a.rows = std::max(16u, fattn_pad((rows + want - 1) / want, 16));
+    a.slices = (rows + a.rows - 1) / a.rows;
+}
+
+}  // namespace
+
+cera_hip_status cera_launch_latent_prep(cera_hip_ctx* ctx, const LatentShape& l, const FAttnShape& absorbed, const float* x, uint64_t ld, uint32_t n,
+                                        uint32_t start, void* cache, void* q, uint32_t kp, void* qn, bool f32) {
+    LArgs a = fill(l, absorbed);
+    a.x = x; a.ld = ld; a.n = n; a.start = start; a.cache = cache; a.q = q; a.qn = qn; a.kp = kp;
+    const dim3 grid((l.heads + 1 + 3) / 4, n);
+    if (f32) hipLaunchKernelGGL(latent_prep_kernel<float>, grid, dim3(256), 0, ctx->stream, a);
+    else hipLaunchKernelGGL(latent_prep_kernel<__bf16>, grid, dim3(256), 0, ctx->stream, a);
+    HIP_TRY(ctx, hipGetLastError());
+    return CERA_HIP_OK;
+}
+
+cera_hip_status cera_launch_latent_spread(cera_hip_ctx* ctx, const LatentShape& l, const FAttnShape& absorbed, const FAttnShape& expanded,
+                                          const void* cache, uint32_t total, void* rows, uint32_t cap, bool f32) {
+    const uint32_t to = fattn_pad(total, FATTN_CAP_STEP);
+    if (to > cap) return cera_fail(ctx, CERA_HIP_ERR_POSITION, "latent attention: positions beyond the expanded rows");
+    const dim3 grid(to / 4, l.heads);
+    auto go = [&](auto tag) {
+        using T = decltype(tag);
+        hipLaunchKernelGGL(latent_spread_kernel<T>, grid, dim3(256), 0, ctx->stream, static_cast<const T*>(cache), absorbed.row, l.rank_p(), l.rot_dim, l.dim,
+                           l.vdim, expanded.v_off, expanded.row, total, cap, static_cast<T*>(rows));
+    };
+    if (f32) go(float{});
+    else go(static_cast<__bf16>(0.0f));
+    HIP_TRY(ctx, hipGetLastError());
+    return CERA_HIP_OK;
+}
+
+cera_hip_status cera_launch_latent_step(cera_hip_ctx* ctx, const LatentShape& l, const FAttnShape& absorbed, const DenseMat& wk, const float* x,
+                                        uint32_t pos, void* cache, void* q, bool f32) {
+    LArgs a = fill(l, absorbed);
+    a.x = x; a.start = pos; a.cache = cache; a.q = q; a.w = static_cast<const __bf16*>(wk.w);
+    if (wk.rows != l.heads * a.rank_p || wk.kp != a.dim_p) return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "latent step: key matrix shape");
+    slice_rows(ctx, a, l.heads, a.rank_p);
+    const dim3 grid(l.heads * a.slices + 1);
+    if (f32) hipLaunchKernelGGL(latent_step_kernel<float>, grid, dim3(256), a.dim_p * 4, ctx->stream, a);
+    else hipLaunchKernelGGL(latent_step_kernel<__bf16>, grid, dim3(256), a.dim_p * 2, ctx->stream, a);
+    HIP_TRY(ctx, hipGetLastError());
+    return CERA_HIP_OK;
+}
+
+cera_hip_status cera_launch_latent_values(cera_hip_ctx* ctx, const LatentShape& l, const DenseMat& wv, const SAttnPartials& parts, void* out, bool f32) {
+    LArgs a{};
+    a.l = l; a.rank_p = l.rank_p(); a.parts = parts; a.out = out; a.w = static_cast<const __bf16*>(wv.w);
+    if (wv.rows != l.heads * l.vdim || wv.kp != a.rank_p || !parts.part || parts.vdim_p != a.rank_p || parts.heads != l.heads)
+        return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "latent values: matrix or partial results do not fit");
+    slice_rows(ctx, a, l.heads, l.vdim);
+    const dim3 grid(l.heads * a.slices);
+    if (f32) hipLaunchKernelGGL(latent_values_kernel<float>, grid, dim3(256), a.rank_p * 4, ctx->stream, a);
+    else hipLaunchKernelGGL(latent_values_kernel<__bf16>, grid, dim3(256), a.rank_p * 2, ctx->stream, a);
+    HIP_TRY(ctx, hipGetLastError());
+    return CERA_HIP_OK;
+}

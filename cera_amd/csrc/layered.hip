@@ -1,5 +1,6 @@
-// The layered float model family (cera_hip_layered_create): weights in HBM, the per-layer state (KV
-// cache and convolution ring of every pass over a layer), the decode step and the batched pass.
+// The layered float model family (cera_hip_layered_create), parallel blocks: weights in HBM, the per-layer state (KV
+// cache and convolution ring of every pass over a layer), the decode step and the batched pass; and what parallel
+// and sequential blocks share.
 //
 // Decode, per layer, three launches: [norm, both input convolutions, Q|K|V|gate and gate|up
 // with SwiGLU] - [rotation, append, attention, head gates; the convolutions' history for the next
@@ -9,74 +10,17 @@
 #include <algorithm>
 #include <cmath>
 #include <cstring>
-#include <map>
 #include <new>
-#include <tuple>
 
-#include "conv_norm.h"
-#include "copy_budget.h"
-#include "dense.h"
-#include "model.h"
-#include "sigmoid_attn.h"
+#include "layered.h"
 
 namespace {
 
 constexpr uint32_t RING_DEPTH = 64;   // rows a convolution ring keeps: how far a sequence can be cut back
 
-struct LayerW {
-    SAttnShape shape;
-    DenseMat qkvg, gate_up, down;      // down: O | down side by side
-    uint32_t ff = 0;
-    uint64_t att_p = 0;                // columns of the attention output in down's input
-    float *norm = nullptr, *conv_a = nullptr, *conv_b = nullptr;    // [ld], [taps][ld]
-    float *scale_a = nullptr, *scale_b = nullptr;                   // norm * (1 + last tap)
-};
-// One pass over a layer, with its own cache and state
-struct Run {
-    uint32_t layer = 0;
-    int step = -1;                     // number of the pass that begins here, or -1
-    void *kc = nullptr, *vc = nullptr;
-    ConvRing ring;
-    ConvHist hist;
-};
-
 }  // namespace
 
-struct CeraLayered {
-    cera_hip_layered_config cfg{};
-    bool f32 = false;
-    uint32_t esz = 2;                  // bytes of an activation / cache element
-    uint64_t ld = 0;                   // floats of a residual row: width padded
-    uint32_t cap = 0;                  // cache positions
-    uint32_t steps = 0;                // rows of loop_step
-    std::vector<LayerW> layers;
-    std::vector<Run> runs;
-    void *embed = nullptr, *pos = nullptr;
-    DenseMat head, loop_in;
-    float *loop_step = nullptr, *final_norm = nullptr;
-    bool step_fits = true;             // every decode product's input fits the GEMV's LDS
-    // one token
-    float *x = nullptr, *xb = nullptr, *x0 = nullptr, *qkvg = nullptr;
-    void *cat = nullptr, *q = nullptr;
-    // state of the sequence
-    uint32_t hist_pos = UINT32_MAX;    // position the convolution history sums are for
-    uint32_t ring_lo = 0;              // oldest position the rings still hold
-    // batched pass, token-major, `cap_n` rows
-    uint32_t cap_n = 0;
-    float *bx = nullptr, *bx0 = nullptr, *bqkvg = nullptr, *binv = nullptr;
-    void *ba = nullptr, *bb = nullptr, *bq = nullptr, *bcat = nullptr, *bcat2 = nullptr;
-    uint32_t* btok = nullptr;
-    float* blogits = nullptr;
-    uint32_t logits_cap = 0;
-    uint64_t b_bytes = 0;
-    std::vector<void*> b_owned;
-};
-
-namespace {
-
-using L = CeraLayered;
-
-cera_hip_status dalloc(cera_hip_model* m, uint64_t bytes, void** out, bool zero) {
+cera_hip_status layered_alloc(cera_hip_model* m, uint64_t bytes, void** out, bool zero) {
     *out = nullptr;
     HIP_TRY(m->ctx, hipMalloc(out, bytes ? bytes : 256));
     m->owned.push_back(*out);
@@ -84,35 +28,81 @@ cera_hip_status dalloc(cera_hip_model* m, uint64_t bytes, void** out, bool zero)
     if (zero) HIP_TRY(m->ctx, hipMemsetAsync(*out, 0, bytes, m->ctx->stream));
     return CERA_HIP_OK;
 }
-template <class T> cera_hip_status dalloc_t(cera_hip_model* m, uint64_t n, T** out, bool zero = true) {
-    return dalloc(m, n * sizeof(T), reinterpret_cast<void**>(out), zero);
-}
-// a host vector of n floats into ld floats (pad zero)
-cera_hip_status put_vec(cera_hip_model* m, const float* src, uint64_t n, uint64_t ld, float** out) {
+cera_hip_status layered_put_vec(cera_hip_model* m, const float* src, uint64_t n, uint64_t ld, float** out) {
     std::vector<float> v(ld, 0.0f);
     std::copy(src, src + n, v.begin());
-    CERA_TRY(dalloc_t(m, ld, out, false));
+    CERA_TRY(layered_alloc_t(m, ld, out, false));
     return cera_hip_upload(m->ctx, *out, v.data(), ld * 4);
 }
+void Packer::row(uint64_t dst, uint64_t col, const cera_hip_tensor& t, uint64_t src, uint64_t c0, uint64_t n) {
+    std::memcpy(host.data() + dst * kp + col, static_cast<const uint16_t*>(t.data) + src * t.k + c0, (n ? n : t.k) * 2);
+}
+void Packer::rows(uint64_t dst, uint64_t col, const cera_hip_tensor& t) {
+    for (uint64_t r = 0; r < t.m; ++r) row(dst + r, col, t, r);
+}
+cera_hip_status Packer::put(cera_hip_model* m, DenseMat* out) {
+    out->kp = static_cast<uint32_t>(kp);
+    out->rows = static_cast<uint32_t>(host.size() / kp);
+    CERA_TRY(layered_alloc(m, host.size() * 2, &out->w, false));
+    return cera_hip_upload(m->ctx, out->w, host.data(), host.size() * 2);
+}
+float layered_get(const CeraLayered& g, const void* rows, uint64_t i) {
+    if (g.f32) return static_cast<const float*>(rows)[i];
+    const uint32_t b = static_cast<uint32_t>(static_cast<const uint16_t*>(rows)[i]) << 16;
+    float f;
+    std::memcpy(&f, &b, 4);
+    return f;
+}
+void layered_set(const CeraLayered& g, void* rows, uint64_t i, float f) {
+    if (g.f32) { static_cast<float*>(rows)[i] = f; return; }
+    uint32_t b;
+    std::memcpy(&b, &f, 4);
+    static_cast<uint16_t*>(rows)[i] = static_cast<uint16_t>((b + 0x7FFFu + ((b >> 16) & 1)) >> 16);   // nearest even
+}
+void layered_batch_free(cera_hip_model* m) {
+    CeraLayered& g = *m->layered;
+    for (void* p : g.b_owned) (void)hipFree(p);
+    g.b_owned.clear();
+    m->bytes -= std::min(m->bytes, g.b_bytes);
+    g.b_bytes = 0;
+    g.cap_n = g.logits_cap = 0;
+    g.blogits = nullptr;
+}
+cera_hip_status layered_batch_alloc(cera_hip_model* m, uint64_t bytes, void** out) {
+    CeraLayered& g = *m->layered;
+    *out = nullptr;
+    HIP_TRY(m->ctx, hipMalloc(out, bytes));
+    g.b_owned.push_back(*out);
+    g.b_bytes += bytes;
+    m->bytes += bytes;
+    // pad columns are read by the products, against zero weights: they have to be finite
+    HIP_TRY(m->ctx, hipMemsetAsync(*out, 0, bytes, m->ctx->stream));
+    return CERA_HIP_OK;
+}
+cera_hip_status layered_batch_logits(cera_hip_model* m, uint32_t n) {
+    CeraLayered& g = *m->layered;
+    if (g.logits_cap >= n) return CERA_HIP_OK;   // grows with the pass buffers only: an older, smaller one is freed with them
+    CERA_TRY(layered_batch_alloc(m, static_cast<uint64_t>(g.cap_n) * g.cfg.vocab * 4, reinterpret_cast<void**>(&g.blogits)));
+    g.logits_cap = g.cap_n;
+    return CERA_HIP_OK;
+}
+cera_hip_status layered_portions(cera_hip_model* m, LayeredPass pass, const uint32_t* tokens, uint32_t n, uint32_t start, float* last_logits, float* all) {
+    if (n == 1) {
+        CERA_TRY(m->ops->decode(m, tokens[0], start, true));
+        m->seq_len = start + 1;
+        return cera_hip_download(m->ctx, all ? all : last_logits, m->logits, static_cast<uint64_t>(m->cfg.vocab) * 4);
+    }
+    for (uint32_t off = 0; off < n; off += CERA_PREFILL_CHUNK) {
+        const uint32_t len = std::min(CERA_PREFILL_CHUNK, n - off);
+        CERA_TRY(pass(m, tokens + off, len, start + off, !all && off + len == n, all ? all + static_cast<uint64_t>(off) * m->cfg.vocab : nullptr));
+        m->seq_len = start + off + len;
+    }
+    return all ? CERA_HIP_OK : cera_hip_download(m->ctx, last_logits, m->logits, static_cast<uint64_t>(m->cfg.vocab) * 4);
+}
 
-// ---- weights: bf16 rows of several matrices packed into one padded matrix -------------------------
-struct Packer {
-    std::vector<uint16_t> host;
-    uint64_t kp = 0;
-    Packer(uint64_t rows, uint64_t kp_) : host(rows * kp_, 0), kp(kp_) {}
-    void row(uint64_t dst, uint64_t col, const cera_hip_tensor& t, uint64_t src, uint64_t c0 = 0, uint64_t n = 0) {
-        std::memcpy(host.data() + dst * kp + col, static_cast<const uint16_t*>(t.data) + src * t.k + c0, (n ? n : t.k) * 2);
-    }
-    void rows(uint64_t dst, uint64_t col, const cera_hip_tensor& t) {
-        for (uint64_t r = 0; r < t.m; ++r) row(dst + r, col, t, r);
-    }
-    cera_hip_status put(cera_hip_model* m, DenseMat* out) {
-        out->kp = static_cast<uint32_t>(kp);
-        out->rows = static_cast<uint32_t>(host.size() / kp);
-        CERA_TRY(dalloc(m, host.size() * 2, &out->w, false));
-        return cera_hip_upload(m->ctx, out->w, host.data(), host.size() * 2);
-    }
-};
+namespace {
+
+using L = CeraLayered;
 
 // Per-pair (cos, sin) of every position.  Frequencies base^(-2 i / dims); with yarn the low ones are
 // divided by the factor, the high ones kept, blended linearly between the dimensions that turn `fast`
@@ -141,6 +131,21 @@ std::vector<float> rotation_table(const cera_hip_attn_spec& s, uint32_t position
         }
     return t;
 }
+
+}  // namespace
+
+cera_hip_status layered_rotation(cera_hip_model* m, const cera_hip_attn_spec& s, RotationTables* tables, const float** out) {
+    if (!s.rot_dims) return CERA_HIP_OK;
+    float*& t = (*tables)[std::make_tuple(s.rot_dims, s.rot_base, s.yarn, s.yarn_factor, s.yarn_original, s.yarn_fast, s.yarn_slow)];
+    if (!t) {
+        const std::vector<float> host = rotation_table(s, m->layered->cap);
+        CERA_TRY(layered_put_vec(m, host.data(), host.size(), host.size(), &t));
+    }
+    *out = t;
+    return CERA_HIP_OK;
+}
+
+namespace {
 
 // ---- the decode step ------------------------------------------------------------------------------
 cera_hip_status batch_pass(cera_hip_model* m, const uint32_t* tokens, uint32_t n, uint32_t start, bool last, float* all);
@@ -215,32 +220,12 @@ cera_hip_status decode(cera_hip_model* m, uint32_t token, uint32_t pos, bool wan
 }
 
 // ---- the batched pass -----------------------------------------------------------------------------
-void free_batch(cera_hip_model* m) {
-    L& g = *m->layered;
-    for (void* p : g.b_owned) (void)hipFree(p);
-    g.b_owned.clear();
-    m->bytes -= std::min(m->bytes, g.b_bytes);
-    g.b_bytes = 0;
-    g.cap_n = g.logits_cap = 0;
-    g.blogits = nullptr;
-}
-cera_hip_status balloc(cera_hip_model* m, uint64_t bytes, void** out) {
-    L& g = *m->layered;
-    *out = nullptr;
-    HIP_TRY(m->ctx, hipMalloc(out, bytes));
-    g.b_owned.push_back(*out);
-    g.b_bytes += bytes;
-    m->bytes += bytes;
-    // pad columns are read by the products, against zero weights: they have to be finite
-    HIP_TRY(m->ctx, hipMemsetAsync(*out, 0, bytes, m->ctx->stream));
-    return CERA_HIP_OK;
-}
 cera_hip_status ensure_batch(cera_hip_model* m, uint32_t n, bool logits) {
     L& g = *m->layered;
     const uint32_t limit = std::min<uint32_t>(CERA_PREFILL_CHUNK, g.cfg.max_seq_len);
     if (g.cap_n < n) {
         HIP_TRY(m->ctx, hipStreamSynchronize(m->ctx->stream));
-        free_batch(m);
+        layered_batch_free(m);
         const uint64_t N = std::min<uint64_t>(limit, (n + 255) / 256 * 256);
         uint64_t qkvg = 0, cat = 0, q = 0;
         for (const LayerW& W : g.layers) {
@@ -249,26 +234,23 @@ cera_hip_status ensure_batch(cera_hip_model* m, uint32_t n, bool logits) {
             q = std::max<uint64_t>(q, static_cast<uint64_t>(W.shape.heads) * sattn_pad32(W.shape.dim));
         }
         auto all = [&]() -> cera_hip_status {
-            auto fl = [&](uint64_t n_el, float** p) { return balloc(m, n_el * 4, reinterpret_cast<void**>(p)); };
+            auto fl = [&](uint64_t n_el, float** p) { return layered_batch_alloc(m, n_el * 4, reinterpret_cast<void**>(p)); };
             CERA_TRY(fl(N * g.ld, &g.bx));
             CERA_TRY(fl(N * g.ld, &g.bx0));
             CERA_TRY(fl(N * qkvg, &g.bqkvg));
             CERA_TRY(fl(N, &g.binv));
-            CERA_TRY(balloc(m, N * g.ld * g.esz, &g.ba));
-            CERA_TRY(balloc(m, N * g.ld * g.esz, &g.bb));
-            CERA_TRY(balloc(m, N * q * g.esz, &g.bq));
-            CERA_TRY(balloc(m, N * cat * g.esz, &g.bcat));
-            if (g.loop_in.w) CERA_TRY(balloc(m, N * 2 * g.ld * g.esz, &g.bcat2));
-            return balloc(m, N * 4, reinterpret_cast<void**>(&g.btok));
+            CERA_TRY(layered_batch_alloc(m, N * g.ld * g.esz, &g.ba));
+            CERA_TRY(layered_batch_alloc(m, N * g.ld * g.esz, &g.bb));
+            CERA_TRY(layered_batch_alloc(m, N * q * g.esz, &g.bq));
+            CERA_TRY(layered_batch_alloc(m, N * cat * g.esz, &g.bcat));
+            if (g.loop_in.w) CERA_TRY(layered_batch_alloc(m, N * 2 * g.ld * g.esz, &g.bcat2));
+            return layered_batch_alloc(m, N * 4, reinterpret_cast<void**>(&g.btok));
         };
         const cera_hip_status st = all();
-        if (st != CERA_HIP_OK) { free_batch(m); return st; }
+        if (st != CERA_HIP_OK) { layered_batch_free(m); return st; }
         g.cap_n = static_cast<uint32_t>(N);
     }
-    if (logits && g.logits_cap < n) {   // grows with the pass buffers only: an older, smaller one is freed with them
-        CERA_TRY(balloc(m, static_cast<uint64_t>(g.cap_n) * g.cfg.vocab * 4, reinterpret_cast<void**>(&g.blogits)));
-        g.logits_cap = g.cap_n;
-    }
+    if (logits) CERA_TRY(layered_batch_logits(m, n));
     return CERA_HIP_OK;
 }
 
@@ -326,26 +308,10 @@ cera_hip_status batch_pass(cera_hip_model* m, const uint32_t* tokens, uint32_t n
 }
 
 cera_hip_status prefill(cera_hip_model* m, const uint32_t* tokens, uint32_t n, uint32_t start, float* last_logits) {
-    if (n == 1) {
-        CERA_TRY(decode(m, tokens[0], start, true));
-        m->seq_len = start + 1;
-    } else {
-        for (uint32_t off = 0; off < n; off += CERA_PREFILL_CHUNK) {
-            const uint32_t len = std::min(CERA_PREFILL_CHUNK, n - off);
-            CERA_TRY(batch_pass(m, tokens + off, len, start + off, off + len == n, nullptr));
-            m->seq_len = start + off + len;
-        }
-    }
-    return cera_hip_download(m->ctx, last_logits, m->logits, static_cast<uint64_t>(m->cfg.vocab) * 4);
+    return layered_portions(m, batch_pass, tokens, n, start, last_logits, nullptr);
 }
 cera_hip_status prefill_all(cera_hip_model* m, const uint32_t* tokens, uint32_t n, uint32_t start, float* logits) {
-    if (n == 1) return prefill(m, tokens, 1, start, logits);
-    for (uint32_t off = 0; off < n; off += CERA_PREFILL_CHUNK) {
-        const uint32_t len = std::min(CERA_PREFILL_CHUNK, n - off);
-        CERA_TRY(batch_pass(m, tokens + off, len, start + off, false, logits + static_cast<uint64_t>(off) * m->cfg.vocab));
-        m->seq_len = start + off + len;
-    }
-    return CERA_HIP_OK;
+    return layered_portions(m, batch_pass, tokens, n, start, nullptr, logits);
 }
 
 // ---- state ----------------------------------------------------------------------------------------
@@ -368,19 +334,8 @@ cera_hip_status move_kv(cera_hip_model* m, uint32_t run, float* k, float* v, uin
     const SAttnShape& s = g.layers[R.layer].shape;
     const uint64_t dp = sattn_pad32(s.dim), vp = sattn_pad32(s.vdim);
     std::vector<char> rows;
-    auto get = [&](uint64_t i) {
-        if (g.f32) return reinterpret_cast<const float*>(rows.data())[i];
-        const uint32_t b = static_cast<uint32_t>(reinterpret_cast<const uint16_t*>(rows.data())[i]) << 16;
-        float f;
-        std::memcpy(&f, &b, 4);
-        return f;
-    };
-    auto set = [&](uint64_t i, float f) {
-        if (g.f32) { reinterpret_cast<float*>(rows.data())[i] = f; return; }
-        uint32_t b;
-        std::memcpy(&b, &f, 4);
-        reinterpret_cast<uint16_t*>(rows.data())[i] = static_cast<uint16_t>((b + 0x7FFFu + ((b >> 16) & 1)) >> 16);   // nearest even
-    };
+    auto get = [&](uint64_t i) { return layered_get(g, rows.data(), i); };
+    auto set = [&](uint64_t i, float f) { layered_set(g, rows.data(), i, f); };
     for (uint32_t h = 0; h < s.kv_heads && n; ++h) {
         char* const kd = static_cast<char*>(R.kc) + static_cast<uint64_t>(h) * g.cap * dp * g.esz;
         rows.assign(static_cast<uint64_t>(n) * dp * g.esz, 0);
@@ -430,7 +385,11 @@ cera_hip_status write_conv(cera_hip_model* m, uint32_t run, const float* rows, u
     return CERA_HIP_OK;
 }
 
-void destroy(cera_hip_model* m) {
+const CeraModelOps OPS = {decode, prefill, prefill_all, truncate, read_kv, write_kv, read_conv, write_conv, layered_destroy};
+
+}  // namespace
+
+void layered_destroy(cera_hip_model* m) {
     cera_hip_ctx* ctx = m->ctx;
     std::lock_guard<std::recursive_mutex> lk(ctx->op_mu);
     (void)hipStreamSynchronize(ctx->stream);
@@ -442,22 +401,26 @@ void destroy(cera_hip_model* m) {
         if (p) (void)hipFree(p);
     delete m;
 }
+cera_hip_status layered_bad(cera_hip_ctx* ctx, const std::string& what) { return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "layered_create: " + what); }
+cera_hip_status layered_mat(cera_hip_ctx* ctx, const cera_hip_tensor& t, uint64_t m, uint64_t k, const char* name) {
+    if (t.ggml_type != CERA_HIP_BF16)
+        return cera_fail(ctx, CERA_HIP_ERR_UNSUPPORTED_DTYPE, std::string(name) + ": the layered family takes bf16 matrices");
+    if (!t.data || t.m != m || t.k != k || t.nbytes != m * k * 2)
+        return layered_bad(ctx, std::string(name) + ": expected [" + std::to_string(m) + " x " + std::to_string(k) + "], got [" + std::to_string(t.m) +
+                                    " x " + std::to_string(t.k) + "]");
+    return CERA_HIP_OK;
+}
 
-const CeraModelOps OPS = {decode, prefill, prefill_all, truncate, read_kv, write_kv, read_conv, write_conv, destroy};
+namespace {
 
 cera_hip_status check(cera_hip_ctx* ctx, const cera_hip_layered_config& c, const cera_hip_layered_layer* layers) {
-    auto bad = [&](const std::string& what) { return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "layered_create: " + what); };
+    auto bad = [&](const std::string& what) { return layered_bad(ctx, what); };
+    if (c.block == CERA_HIP_BLOCK_SEQUENTIAL) return layered_seq_check(ctx, c, layers);
+    if (c.block != CERA_HIP_BLOCK_PARALLEL) return bad("unknown block form");
     if (!c.n_layers || !c.width || !c.vocab || !c.max_seq_len || !c.conv_taps) return bad("zero dimension in config");
     if (c.conv_taps > CONV_MAX_TAPS) return bad("conv_taps above " + std::to_string(CONV_MAX_TAPS));
     if (!c.final_norm) return cera_fail(ctx, CERA_HIP_ERR_ARGUMENT, "layered_create: final_norm missing");
-    auto mat = [&](const cera_hip_tensor& t, uint64_t m, uint64_t k, const char* name) -> cera_hip_status {
-        if (t.ggml_type != CERA_HIP_BF16)
-            return cera_fail(ctx, CERA_HIP_ERR_UNSUPPORTED_DTYPE, std::string(name) + ": the layered family takes bf16 matrices");
-        if (!t.data || t.m != m || t.k != k || t.nbytes != m * k * 2)
-            return bad(std::string(name) + ": expected [" + std::to_string(m) + " x " + std::to_string(k) + "], got [" + std::to_string(t.m) +
-                       " x " + std::to_string(t.k) + "]");
-        return CERA_HIP_OK;
-    };
+    auto mat = [&](const cera_hip_tensor& t, uint64_t rows, uint64_t k, const char* name) { return layered_mat(ctx, t, rows, k, name); };
     CERA_TRY(mat(c.embed, c.vocab, c.width, "embed"));
     CERA_TRY(mat(c.head, c.vocab, c.width, "head"));
     if (c.pos.m < c.max_seq_len) return bad("pos has fewer rows than max_seq_len");
@@ -470,6 +433,7 @@ cera_hip_status check(cera_hip_ctx* ctx, const cera_hip_layered_config& c, const
     for (uint32_t i = 0; i < c.n_layers; ++i) {
         const cera_hip_layered_layer& Y = layers[i];
         const cera_hip_attn_spec& a = Y.attn;
+        if (a.kind != CERA_HIP_MIXER_SIGMOID) return bad("layer " + std::to_string(i) + ": parallel blocks take the sigmoid mixer");
         if (!a.heads || !a.kv_heads || a.heads % a.kv_heads || !a.dim || !a.vdim || a.dim > 256 || a.vdim > 256)
             return bad("layer " + std::to_string(i) + ": heads must be a multiple of kv_heads, head sizes at most 256");
         if (a.rot_dims % 2 || a.rot_dims > a.dim) return bad("layer " + std::to_string(i) + ": rot_dims must be even and at most dim");
@@ -499,17 +463,20 @@ cera_hip_status build(cera_hip_model* m, const cera_hip_layered_config& c, const
     const uint64_t ld = g.ld;
     // tables of bf16 rows, as they are
     auto table = [&](const cera_hip_tensor& t, void** out) -> cera_hip_status {
-        CERA_TRY(dalloc(m, t.nbytes, out, false));
+        CERA_TRY(layered_alloc(m, t.nbytes, out, false));
         return cera_hip_upload(ctx, *out, t.data, t.nbytes);
     };
     CERA_TRY(table(c.embed, &g.embed));
-    CERA_TRY(table(c.pos, &g.pos));
     {
         Packer p(c.vocab, ld);
         p.rows(0, 0, c.head);
         CERA_TRY(p.put(m, &g.head));
     }
-    CERA_TRY(put_vec(m, c.final_norm, c.width, ld, &g.final_norm));
+    CERA_TRY(layered_put_vec(m, c.final_norm, c.width, ld, &g.final_norm));
+    CERA_TRY(layered_alloc_t(m, dense_pad(c.vocab), &m->logits));
+    CERA_TRY(layered_alloc_t(m, 4, &m->scalars));
+    if (c.block == CERA_HIP_BLOCK_SEQUENTIAL) return layered_seq_build(m, c, layers);
+    CERA_TRY(table(c.pos, &g.pos));
     if (c.loop_times) {
         Packer p(c.width, 2 * ld);
         for (uint32_t r = 0; r < c.width; ++r) {
@@ -519,9 +486,9 @@ cera_hip_status build(cera_hip_model* m, const cera_hip_layered_config& c, const
         CERA_TRY(p.put(m, &g.loop_in));
         std::vector<float> st(c.loop_times * ld, 0.0f);
         for (uint32_t t = 0; t < c.loop_times; ++t) std::copy(c.loop_step + static_cast<uint64_t>(t) * c.width, c.loop_step + static_cast<uint64_t>(t + 1) * c.width, st.begin() + t * ld);
-        CERA_TRY(put_vec(m, st.data(), st.size(), st.size(), &g.loop_step));
+        CERA_TRY(layered_put_vec(m, st.data(), st.size(), st.size(), &g.loop_step));
     }
-    std::map<std::tuple<uint32_t, double, uint32_t, double, double, double, double>, float*> tables;   // rotations shared between layers
+    RotationTables tables;   // shared between layers
     uint64_t max_qkvg = 0, max_cat = 0, max_q = 0;
     g.layers.resize(c.n_layers);
     for (uint32_t i = 0; i < c.n_layers; ++i) {
@@ -530,16 +497,9 @@ cera_hip_status build(cera_hip_model* m, const cera_hip_layered_config& c, const
         LayerW& W = g.layers[i];
         SAttnShape& s = W.shape;
         s.heads = a.heads; s.kv_heads = a.kv_heads; s.dim = a.dim; s.vdim = a.vdim; s.chunk = a.chunk; s.scale = a.scale; s.rot_dims = a.rot_dims;
-        if (a.rot_dims) {
-            float*& t = tables[std::make_tuple(a.rot_dims, a.rot_base, a.yarn, a.yarn_factor, a.yarn_original, a.yarn_fast, a.yarn_slow)];
-            if (!t) {
-                const std::vector<float> host = rotation_table(a, g.cap);
-                CERA_TRY(put_vec(m, host.data(), host.size(), host.size(), &t));
-            }
-            s.rot_table = t;
-        }
+        CERA_TRY(layered_rotation(m, a, &tables, &s.rot_table));
         float* bias;
-        CERA_TRY(put_vec(m, Y.score_bias, a.heads, a.heads, &bias));
+        CERA_TRY(layered_put_vec(m, Y.score_bias, a.heads, a.heads, &bias));
         s.bias = bias;
         {
             Packer p(Y.q.m + Y.k.m + Y.v.m + Y.head_gate.m, ld);
@@ -564,15 +524,15 @@ cera_hip_status build(cera_hip_model* m, const cera_hip_layered_config& c, const
             pd.rows(0, W.att_p, Y.ffn_down);
         }
         CERA_TRY(pd.put(m, &W.down));
-        CERA_TRY(put_vec(m, Y.norm, c.width, ld, &W.norm));
+        CERA_TRY(layered_put_vec(m, Y.norm, c.width, ld, &W.norm));
         auto conv = [&](const float* src, float** taps_out, float** scale_out) -> cera_hip_status {
             std::vector<float> t(c.conv_taps * ld, 0.0f), sc(ld, 0.0f);
             for (uint32_t ch = 0; ch < c.width; ++ch) {
                 for (uint32_t j = 0; j < c.conv_taps; ++j) t[j * ld + ch] = src[static_cast<uint64_t>(ch) * c.conv_taps + j];
                 sc[ch] = Y.norm[ch] * (1.0f + src[static_cast<uint64_t>(ch) * c.conv_taps + c.conv_taps - 1]);
             }
-            CERA_TRY(put_vec(m, t.data(), t.size(), t.size(), taps_out));
-            return put_vec(m, sc.data(), ld, ld, scale_out);
+            CERA_TRY(layered_put_vec(m, t.data(), t.size(), t.size(), taps_out));
+            return layered_put_vec(m, sc.data(), ld, ld, scale_out);
         };
         CERA_TRY(conv(Y.conv_attn, &W.conv_a, &W.scale_a));
         if (Y.ff) CERA_TRY(conv(Y.conv_ffn, &W.conv_b, &W.scale_b));
@@ -594,24 +554,22 @@ cera_hip_status build(cera_hip_model* m, const cera_hip_layered_config& c, const
     for (Run& R : g.runs) {
         const LayerW& W = g.layers[R.layer];
         const SAttnShape& s = W.shape;
-        CERA_TRY(dalloc(m, static_cast<uint64_t>(s.kv_heads) * g.cap * sattn_pad32(s.dim) * g.esz, &R.kc, true));
-        CERA_TRY(dalloc(m, static_cast<uint64_t>(s.kv_heads) * g.cap * sattn_pad32(s.vdim) * g.esz, &R.vc, true));
+        CERA_TRY(layered_alloc(m, static_cast<uint64_t>(s.kv_heads) * g.cap * sattn_pad32(s.dim) * g.esz, &R.kc, true));
+        CERA_TRY(layered_alloc(m, static_cast<uint64_t>(s.kv_heads) * g.cap * sattn_pad32(s.vdim) * g.esz, &R.vc, true));
         if (c.conv_taps > 1) {
             R.ring.depth = RING_DEPTH; R.ring.ld = ld; R.ring.width = static_cast<uint32_t>(ld);
-            CERA_TRY(dalloc_t(m, RING_DEPTH * ld, &R.ring.rows));
+            CERA_TRY(layered_alloc_t(m, RING_DEPTH * ld, &R.ring.rows));
             R.hist.wa = W.conv_a; R.hist.wb = W.conv_b; R.hist.taps = c.conv_taps;
-            CERA_TRY(dalloc_t(m, ld, &R.hist.a));
-            CERA_TRY(dalloc_t(m, ld, &R.hist.b));
+            CERA_TRY(layered_alloc_t(m, ld, &R.hist.a));
+            CERA_TRY(layered_alloc_t(m, ld, &R.hist.b));
         }
     }
-    CERA_TRY(dalloc_t(m, ld, &g.x));
-    CERA_TRY(dalloc_t(m, ld, &g.xb));
-    CERA_TRY(dalloc_t(m, ld, &g.x0));
-    CERA_TRY(dalloc_t(m, max_qkvg, &g.qkvg));
-    CERA_TRY(dalloc(m, max_q * g.esz, &g.q, true));
-    CERA_TRY(dalloc(m, max_cat * g.esz, &g.cat, true));
-    CERA_TRY(dalloc_t(m, dense_pad(c.vocab), &m->logits));
-    CERA_TRY(dalloc_t(m, 4, &m->scalars));
+    CERA_TRY(layered_alloc_t(m, ld, &g.x));
+    CERA_TRY(layered_alloc_t(m, ld, &g.xb));
+    CERA_TRY(layered_alloc_t(m, ld, &g.x0));
+    CERA_TRY(layered_alloc_t(m, max_qkvg, &g.qkvg));
+    CERA_TRY(layered_alloc(m, max_q * g.esz, &g.q, true));
+    CERA_TRY(layered_alloc(m, max_cat * g.esz, &g.cat, true));
     m->hidden = g.x;
     const uint64_t widest = std::max<uint64_t>(max_cat, (c.loop_times ? 2 : 1) * ld);
     g.step_fits = cera_dense_gemv_fits(widest, g.f32);
@@ -629,7 +587,7 @@ extern "C" cera_hip_status cera_hip_layered_create(cera_hip_ctx* ctx, const cera
     cera_hip_model* m = new (std::nothrow) cera_hip_model();
     if (!m) return cera_fail(ctx, CERA_HIP_ERR_OOM, "host allocation failed");
     m->ctx = ctx;
-    m->ops = &OPS;
+    m->ops = cfg->block == CERA_HIP_BLOCK_SEQUENTIAL ? layered_seq_ops() : &OPS;
     m->layered = new (std::nothrow) CeraLayered();
     cera_hip_status st = m->layered ? CERA_HIP_OK : cera_fail(ctx, CERA_HIP_ERR_OOM, "host allocation failed");
     if (st == CERA_HIP_OK) {
@@ -638,7 +596,7 @@ extern "C" cera_hip_status cera_hip_layered_create(cera_hip_ctx* ctx, const cera
     }
     if (st != CERA_HIP_OK) {
         const std::string keep = ctx->err;
-        destroy(m);
+        layered_destroy(m);
         ctx->err = keep;
         return st;
     }
@@ -646,7 +604,7 @@ extern "C" cera_hip_status cera_hip_layered_create(cera_hip_ctx* ctx, const cera
     cera_hip_layered_config& c = m->layered->cfg;
     c.embed.data = c.pos.data = c.head.data = c.loop_in.data = nullptr;
     c.loop_step = c.final_norm = nullptr;
-    m->cfg.n_layers = static_cast<uint32_t>(m->layered->runs.size());
+    m->cfg.n_layers = static_cast<uint32_t>(m->layered->runs.size() + m->layered->seq.size());
     m->cfg.hidden = cfg->width;
     m->cfg.vocab = cfg->vocab;
     m->cfg.max_seq_len = cfg->max_seq_len;

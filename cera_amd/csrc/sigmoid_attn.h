@@ -61,7 +61,9 @@ struct ConvHist {
 constexpr uint32_t SATTN_MERGE_SPLITS = 8;
 struct SAttnPartials {
     const float* part = nullptr;   // [splits][heads][vdim_p]
-    const float* gate = nullptr;   // [heads], before the sigmoid
+    const float* gate = nullptr;   // sigmoid weights: [heads], before the sigmoid
+    // softmax weights: maximum (in powers of two) and sum of every part, [splits][heads][2], and the heads' sinks
+    const float *ml = nullptr, *sink = nullptr;
     uint32_t splits = 0, heads = 0, vdim = 0, vdim_p = 0;
 };
 cera_hip_status cera_launch_sattn_step(cera_hip_ctx* ctx, const SAttnShape& s, const SAttnPass& p, const ConvRing& ring,

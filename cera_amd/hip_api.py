@@ -70,22 +70,24 @@ class Config(C.Structure):
 
 class AttnSpec(C.Structure):
     """cera_hip_attn_spec."""
-    _fields_ = [("heads", C.c_uint32), ("kv_heads", C.c_uint32), ("dim", C.c_uint32), ("vdim", C.c_uint32),
-                ("scale", C.c_float), ("chunk", C.c_uint32), ("rot_dims", C.c_uint32), ("yarn", C.c_uint32),
-                ("rot_base", C.c_double), ("yarn_factor", C.c_double), ("yarn_original", C.c_double),
-                ("yarn_fast", C.c_double), ("yarn_slow", C.c_double)]
+    SIGMOID, SOFTMAX, LATENT = range(3)
+    _fields_ = [(n, C.c_uint32) for n in ("kind", "heads", "kv_heads", "dim", "vdim")] + [("scale", C.c_float)] + \
+               [(n, C.c_uint32) for n in ("chunk", "rot_dims", "yarn", "rot_dim", "kv_rank", "v_mix")] + \
+               [(n, C.c_double) for n in ("rot_base", "yarn_factor", "yarn_original", "yarn_fast", "yarn_slow", "q_temp_coef", "q_temp_every")]
 
 
 class LayeredLayer(C.Structure):
     """cera_hip_layered_layer."""
-    _fields_ = [("attn", AttnSpec), ("ff", C.c_uint32), ("_reserved", C.c_uint32), ("norm", C.c_void_p),
-                ("conv_attn", C.c_void_p), ("conv_ffn", C.c_void_p), ("score_bias", C.c_void_p)] + \
-               [(n, Tensor) for n in ("q", "k", "v", "head_gate", "o", "ffn_gate", "ffn_up", "ffn_down")]
+    _fields_ = [("attn", AttnSpec), ("ff", C.c_uint32), ("v_mix_lambda", C.c_float)] + \
+               [(n, C.c_void_p) for n in ("norm", "norm_ffn", "conv_attn", "conv_ffn", "streams_attn", "streams_ffn", "score_bias", "sink",
+                                          "q_norm", "k_norm", "latent_norm")] + \
+               [(n, Tensor) for n in ("q", "k", "v", "head_gate", "o", "kv_down", "k_up", "v_up", "ffn_gate", "ffn_up", "ffn_down")]
 
 
 class LayeredConfig(C.Structure):
     """cera_hip_layered_config."""
-    _fields_ = [(n, C.c_uint32) for n in ("n_layers", "width", "vocab", "max_seq_len", "conv_taps", "loop_start",
+    PARALLEL, SEQUENTIAL = range(2)
+    _fields_ = [(n, C.c_uint32) for n in ("n_layers", "width", "vocab", "max_seq_len", "block", "streams", "conv_taps", "loop_start",
                                           "loop_stop", "loop_times")] + \
                [("eps", C.c_float), ("residual_mult", C.c_float), ("f32", C.c_uint32), ("_reserved", C.c_uint32)] + \
                [(n, Tensor) for n in ("embed", "pos", "head", "loop_in")] + \
@@ -732,30 +734,39 @@ class Model:
 
 
 class LayeredModel(Model):
-    """cera_hip_layered_create over arrays: ``cfg`` as a Nafevik config.json, ``weights`` by tensor name --
-    uint16 bf16 bits [out, in] for matrices, float32 for vectors."""
+    """cera_hip_layered_create over arrays: ``cfg`` as the config.json of a Nafevik (the default) or a Fidinex
+    (``"architecture"``), ``weights`` by tensor name -- uint16 bf16 bits [out, in] for matrices, float32 for vectors."""
 
     def __init__(self, ctx: Context, cfg: dict, weights: dict, max_seq_len: int, f32: bool = False):
         self.ctx, self.cfg = ctx, dict(cfg)
-        keep = []
+        self._keep, self._weights = [], weights
+        c = LayeredConfig(len(cfg["layers"]), cfg["width"], cfg["vocab"], max_seq_len)
+        c.eps, c.f32, c.final_norm = cfg["norm"]["eps"], int(f32), self._vec("final.norm")
+        c.embed = self._mat("embed")
+        layers = (LayeredLayer * c.n_layers)()
+        (self._fidinex if cfg.get("architecture") == "Fidinex" else self._nafevik)(c, layers)
+        h = C.c_void_p()
+        ctx.check(ctx.lib.cera_hip_layered_create(ctx.h, C.byref(c), layers, C.byref(h)))
+        self.h, self.vocab, self.hidden = h, c.vocab, c.width
+        del self._keep, self._weights
 
-        def mat(name):
-            a = weights[name]
-            assert a.dtype == np.uint16 and a.flags["C_CONTIGUOUS"], name
-            return Tensor(BF16, 0, a.shape[0], a.shape[1], a.ctypes.data, a.nbytes)
+    def _mat(self, name):
+        a = self._weights[name]
+        assert a.dtype == np.uint16 and a.flags["C_CONTIGUOUS"], name
+        return Tensor(BF16, 0, a.shape[0], a.shape[1], a.ctypes.data, a.nbytes)
 
-        def vec(name):
-            a = np.ascontiguousarray(weights[name], np.float32)
-            keep.append(a)
-            return a.ctypes.data
+    def _vec(self, *names):
+        a = np.concatenate([np.asarray(self._weights[n], np.float32).ravel() for n in names])
+        self._keep.append(a)
+        return a.ctypes.data
 
-        c = LayeredConfig(len(cfg["layers"]), cfg["width"], cfg["vocab"], max_seq_len, cfg["canon"]["taps"])
-        c.eps, c.residual_mult, c.f32 = cfg["norm"]["eps"], cfg["residual_mult"], int(f32)
-        c.embed, c.pos, c.head, c.final_norm = mat("embed"), mat("pos"), mat("head"), vec("final.norm")
+    def _nafevik(self, c, layers):
+        cfg, mat, vec = self.cfg, self._mat, self._vec
+        c.conv_taps, c.residual_mult = cfg["canon"]["taps"], cfg["residual_mult"]
+        c.pos, c.head = mat("pos"), mat("head")
         if cfg.get("loop"):
             c.loop_start, c.loop_stop, c.loop_times = (cfg["loop"][k] for k in ("start", "stop", "times"))
             c.loop_in, c.loop_step = mat("loop.in"), vec("loop.step")
-        layers = (LayeredLayer * c.n_layers)()
         for i, spec in enumerate(cfg["layers"]):
             Y, p, m = layers[i], f"l{i}.", spec["mixer"]
             a = Y.attn
@@ -773,6 +784,30 @@ class LayeredModel(Model):
             if spec.get("mlp"):
                 Y.ff, Y.conv_ffn = spec["mlp"]["ff"], vec(p + "canon2")
                 Y.ffn_gate, Y.ffn_up, Y.ffn_down = (mat(p + "mlp." + n) for n in ("gate", "up", "down"))
-        h = C.c_void_p()
-        ctx.check(ctx.lib.cera_hip_layered_create(ctx.h, C.byref(c), layers, C.byref(h)))
-        self.h, self.vocab, self.hidden = h, c.vocab, c.width
+
+    def _fidinex(self, c, layers):
+        cfg, mat, vec = self.cfg, self._mat, self._vec
+        c.block, c.streams, c.head = LayeredConfig.SEQUENTIAL, cfg["streams"], c.embed
+        for i, spec in enumerate(cfg["layers"]):
+            Y, p, m = layers[i], f"l{i}.", spec["mixer"]
+            a = Y.attn
+            a.heads, a.dim, a.vdim, a.scale = m["heads"], m["dim"], m["vdim"], m["scale"]
+            Y.norm, Y.sink = vec(p + "norm1"), vec(p + "mix.sink")
+            Y.streams_attn = vec(p + "hc1.in", p + "hc1.out", p + "hc1.mix")
+            Y.q, Y.o = mat(p + "mix.q"), mat(p + "mix.o")
+            if spec["type"] == "latent_attention":
+                a.kind, a.rot_dim, a.kv_rank, a.rot_dims, a.rot_base = AttnSpec.LATENT, m["rot_dim"], m["kv_rank"], m["rot"]["dims"], m["rot"]["base"]
+                Y.latent_norm = vec(p + "mix.dkv.norm")
+                Y.kv_down, Y.k_up, Y.v_up = (mat(p + "mix." + n) for n in ("dkv", "uk", "uv"))
+            else:
+                a.kind, a.kv_heads, a.v_mix = AttnSpec.SOFTMAX, m["kv_heads"], int(bool(m.get("v_mix")))
+                if m.get("q_temp"):
+                    a.q_temp_coef, a.q_temp_every = m["q_temp"]["coef"], m["q_temp"]["every"]
+                if a.v_mix:
+                    Y.v_mix_lambda = float(np.asarray(self._weights[p + "mix.vmix"], np.float32).reshape(()))
+                Y.q_norm, Y.k_norm = vec(p + "mix.q.norm"), vec(p + "mix.k.norm")
+                Y.k, Y.v = mat(p + "mix.k"), mat(p + "mix.v")
+            if spec.get("mlp"):
+                Y.ff, Y.norm_ffn = spec["mlp"]["ff"], vec(p + "norm2")
+                Y.streams_ffn = vec(p + "hc2.in", p + "hc2.out", p + "hc2.mix")
+                Y.ffn_up, Y.ffn_down = mat(p + "mlp.up"), mat(p + "mlp.down")

@@ -470,42 +470,69 @@ CERA_HIP_API cera_hip_status cera_hip_model_create(cera_hip_ctx*, const cera_hip
                                                    const float* output_norm, const cera_hip_layer* layers,
                                                    cera_hip_model** out);
 /* ---- layered float models -------------------------------------------------
- * A decoder described layer by layer: bfloat16 weights, RMS norms, one norm per layer read by an
- * attention mixer and a feed-forward side by side (x += residual_mult * (mixer + feed-forward)),
- * each reading its input through a short causal convolution; attention with unnormalised sigmoid
- * weights inside chunks of positions and a gate per head; learned position vectors; a range of layers
- * that runs several times over.  Every size and constant is a field.  The Nafevik architecture is
- * one such model (its config.json reader is HipLayeredModel, cera_amd/backend/hip_layered.h).
+ * A decoder described layer by layer: bfloat16 weights, RMS norms.  Two forms of a layer:
+ *   CERA_HIP_BLOCK_PARALLEL    one norm per layer read by an attention mixer and a gated feed-forward side by side
+ *       (x += residual_mult * (mixer + feed-forward)), each reading its input through a short causal convolution;
+ *       learned position vectors; a range of layers that runs several times over;
+ *   CERA_HIP_BLOCK_SEQUENTIAL  mixer and feed-forward one after the other, each behind its own norm, over `streams`
+ *       residual streams: a sublayer reads u = sum_s in[s] x_s and its output y goes to all of them at once,
+ *       x_t <- sum_s mix[s][t] x_s + out[t] y; the sum of the streams leaves the last layer.
+ * Mixers:
+ *   CERA_HIP_MIXER_SIGMOID  unnormalised sigmoid weights inside chunks of positions, a gate per head (parallel blocks);
+ *   CERA_HIP_MIXER_SOFTMAX  softmax with a sink per head, norms on query and key heads, a factor on the queries that
+ *       grows with the position, values mixed with those of the first mixing layer (sequential blocks);
+ *   CERA_HIP_MIXER_LATENT   softmax with a sink per head over a cache of one normalised latent and one rotated key part
+ *       per token, keys and values being products of the latent (sequential blocks).
+ * Every size and constant is a field.  The Nafevik and the Fidinex architecture are such models (their config.json
+ * readers are cera_amd/backend/nafevik.cpp and fidinex.cpp).
  * All the model-level calls below take the handle; those that only a llama has (configure_kv,
  * shift_kv, set_reference_order, drop_decode_copies) fail with CERA_HIP_ERR_ARGUMENT. */
+#define CERA_HIP_BLOCK_PARALLEL 0u
+#define CERA_HIP_BLOCK_SEQUENTIAL 1u
+#define CERA_HIP_MIXER_SIGMOID 0u
+#define CERA_HIP_MIXER_SOFTMAX 1u
+#define CERA_HIP_MIXER_LATENT 2u
+#define CERA_HIP_MAX_STREAMS 8u
 typedef struct {
-    uint32_t heads, kv_heads, dim, vdim; /* dim: query / key size, vdim: value size; each at most 256 */
-    float scale;                         /* score = q . k * scale + score_bias[head] */
-    uint32_t chunk;                      /* positions per attention chunk; 0: the whole sequence */
-    uint32_t rot_dims;                   /* leading dimensions rotated in adjacent pairs; 0: none */
+    uint32_t kind;                       /* CERA_HIP_MIXER_* */
+    uint32_t heads, kv_heads, dim, vdim; /* dim: query / key size (latent: the unrotated part), vdim: value size */
+    float scale;                         /* score = q . k * scale (+ score_bias[head]) */
+    uint32_t chunk;                      /* sigmoid: positions per attention chunk; 0: the whole sequence */
+    uint32_t rot_dims;                   /* leading dimensions rotated in adjacent pairs (latent: of the rotated part); 0: none */
     uint32_t yarn;                       /* 1: the frequencies are blended as below */
+    uint32_t rot_dim, kv_rank;           /* latent: rotated dimensions per head, latent size */
+    uint32_t v_mix;                      /* softmax: the values take part in the mixing between layers */
     double rot_base;
     double yarn_factor, yarn_original, yarn_fast, yarn_slow;
+    double q_temp_coef, q_temp_every;    /* softmax: q *= 1 + coef * ln(floor((position + 1) / every) + 1); every 0: no */
 } cera_hip_attn_spec;
 /* Matrices are bf16 tensors (ggml_type CERA_HIP_BF16), [m = outputs][k = inputs]; vectors f32. */
 typedef struct {
     cera_hip_attn_spec attn;
     uint32_t ff;                       /* feed-forward width; 0: the layer has none */
-    uint32_t _reserved;
+    float v_mix_lambda;                /* softmax: v <- (1 - lambda) v + lambda v_first */
     const float* norm;                 /* [width] */
-    const float *conv_attn, *conv_ffn; /* [width][conv_taps]; the second null without a feed-forward */
-    const float* score_bias;           /* [heads] */
-    cera_hip_tensor q, k, v, head_gate, o;
-    cera_hip_tensor ffn_gate, ffn_up, ffn_down;
+    const float* norm_ffn;             /* sequential: [width] */
+    const float *conv_attn, *conv_ffn; /* parallel: [width][conv_taps]; the second null without a feed-forward */
+    const float *streams_attn, *streams_ffn; /* sequential: in [streams] | out [streams] | mix [streams][streams] (from, to) */
+    const float* score_bias;           /* sigmoid: [heads] */
+    const float* sink;                 /* softmax, latent: [heads] */
+    const float *q_norm, *k_norm;      /* softmax: [dim] */
+    const float* latent_norm;          /* latent: [kv_rank] */
+    cera_hip_tensor q, k, v, head_gate, o; /* latent: q, o only */
+    cera_hip_tensor kv_down, k_up, v_up;   /* latent: [kv_rank + rot_dim][width], [heads * dim][kv_rank], [heads * vdim][kv_rank] */
+    cera_hip_tensor ffn_gate, ffn_up, ffn_down; /* parallel: down (silu(gate h) * up h); sequential: down max(up h, 0)^2 */
 } cera_hip_layered_layer;
 typedef struct {
     uint32_t n_layers, width, vocab, max_seq_len;
-    uint32_t conv_taps;
-    uint32_t loop_start, loop_stop, loop_times; /* layers [start, stop) run `times` times in a row; times 0: no loop */
-    float eps, residual_mult;
+    uint32_t block;                      /* CERA_HIP_BLOCK_* */
+    uint32_t streams;                    /* sequential: residual streams, at most CERA_HIP_MAX_STREAMS */
+    uint32_t conv_taps;                  /* parallel */
+    uint32_t loop_start, loop_stop, loop_times; /* parallel: layers [start, stop) run `times` times in a row; times 0: no loop */
+    float eps, residual_mult;            /* residual_mult: parallel */
     uint32_t f32;                        /* 0: matrix products and activations in bf16; 1: everything in f32 */
     uint32_t _reserved;
-    cera_hip_tensor embed, pos, head;    /* [vocab][width], [positions][width], [vocab][width] */
+    cera_hip_tensor embed, pos, head;    /* [vocab][width], [positions][width] (parallel), [vocab][width] */
     cera_hip_tensor loop_in;             /* [width][2 width]: reads the residual, then the embedding output */
     const float* loop_step;              /* [loop_times][width], added after loop_in in each pass */
     const float* final_norm;             /* [width] */
@@ -588,6 +615,7 @@ CERA_HIP_API cera_hip_status cera_hip_shift_kv(cera_hip_model*, uint32_t n_keep,
  * cera/src/kv_cache.rs:1382-1396): K and V cache rows [0, seq_len) to host in the reference's
  * time-major [pos][kv_dim] f32 order.  Also the parity tests' view of the cache. */
 CERA_HIP_API cera_hip_status cera_hip_read_kv(cera_hip_model*, uint32_t layer, float* k_out, float* v_out);
+/* (A latent layer's rows are its latents in k_out and the shared rotated key parts in v_out.) */
 /* Model::restore_state, one layer (cera/src/model/mod.rs:526-533): the inverse of
  * cera_hip_read_kv for rows [0, n_pos).  After the last layer call cera_hip_set_seq_len(n_pos),
  * which "sets internal seq_len" as the trait method does. */

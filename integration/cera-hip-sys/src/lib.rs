@@ -89,10 +89,11 @@ pub struct cera_hip_tensor {
     pub nbytes: u64,
 }
 
-/// One layer's attention in a layered float model (sizes, score scale, chunked mask, rotation).
+/// One layer's attention in a layered float model (kind, sizes, score scale, chunked mask, rotation, query temperature).
 #[repr(C)]
 #[derive(Clone, Copy, Debug)]
 pub struct cera_hip_attn_spec {
+    pub kind: u32,
     pub heads: u32,
     pub kv_heads: u32,
     pub dim: u32,
@@ -101,11 +102,16 @@ pub struct cera_hip_attn_spec {
     pub chunk: u32,
     pub rot_dims: u32,
     pub yarn: u32,
+    pub rot_dim: u32,
+    pub kv_rank: u32,
+    pub v_mix: u32,
     pub rot_base: f64,
     pub yarn_factor: f64,
     pub yarn_original: f64,
     pub yarn_fast: f64,
     pub yarn_slow: f64,
+    pub q_temp_coef: f64,
+    pub q_temp_every: f64,
 }
 
 /// Weights of one layer of a layered float model: bf16 matrices, `f32` vectors (host).
@@ -114,16 +120,26 @@ pub struct cera_hip_attn_spec {
 pub struct cera_hip_layered_layer {
     pub attn: cera_hip_attn_spec,
     pub ff: u32,
-    pub _reserved: u32,
+    pub v_mix_lambda: f32,
     pub norm: *const f32,
+    pub norm_ffn: *const f32,
     pub conv_attn: *const f32,
     pub conv_ffn: *const f32,
+    pub streams_attn: *const f32,
+    pub streams_ffn: *const f32,
     pub score_bias: *const f32,
+    pub sink: *const f32,
+    pub q_norm: *const f32,
+    pub k_norm: *const f32,
+    pub latent_norm: *const f32,
     pub q: cera_hip_tensor,
     pub k: cera_hip_tensor,
     pub v: cera_hip_tensor,
     pub head_gate: cera_hip_tensor,
     pub o: cera_hip_tensor,
+    pub kv_down: cera_hip_tensor,
+    pub k_up: cera_hip_tensor,
+    pub v_up: cera_hip_tensor,
     pub ffn_gate: cera_hip_tensor,
     pub ffn_up: cera_hip_tensor,
     pub ffn_down: cera_hip_tensor,
@@ -137,6 +153,8 @@ pub struct cera_hip_layered_config {
     pub width: u32,
     pub vocab: u32,
     pub max_seq_len: u32,
+    pub block: u32,
+    pub streams: u32,
     pub conv_taps: u32,
     pub loop_start: u32,
     pub loop_stop: u32,
