@@ -255,15 +255,21 @@ DESIGN_SIZES = {
 DESIGN_LAYERS, DESIGN_VOCAB, DESIGN_CTX = 8, 32000, 4096
 
 
-def nafevik_model(ctx, hip_api, size, rng, f32=False):
-    """A random-init Nafevik of DESIGN_LAYERS layers, the last six of them a loop run once (chunks of 2048,
-    four taps): (model, weight bytes a decode step reads).  The layers share host arrays, not HBM."""
-    W, FF, Hq, G, D = (size[k] for k in ("width", "ff", "heads", "kv_heads", "dim"))
+def _random(rng):
+    """Makers of bf16 matrices (bits) and of f32 vectors."""
     def mat(m, k, sigma=0.02):
         w = rng.standard_normal((m, k), dtype=np.float32) * np.float32(sigma)
         return (w.view(np.uint32) >> 16).astype(np.uint16)
     def vec(*shape):
         return (0.1 * rng.standard_normal(shape)).astype(np.float32)
+    return mat, vec
+
+
+def nafevik_model(ctx, hip_api, size, rng, f32=False):
+    """A random-init Nafevik of DESIGN_LAYERS layers, the last six of them a loop run once (chunks of 2048,
+    four taps): (model, weight bytes a decode step reads).  The layers share host arrays, not HBM."""
+    W, FF, Hq, G, D = (size[k] for k in ("width", "ff", "heads", "kv_heads", "dim"))
+    mat, vec = _random(rng)
     layer = {"norm1": 1 + vec(W), "canon1": vec(W, 4), "canon2": vec(W, 4), "mix.pb": vec(Hq) - 4, "mix.q": mat(Hq * D, W), "mix.k": mat(G * D, W),
              "mix.v": mat(G * D, W), "mix.g": mat(Hq, W), "mix.o": mat(W, Hq * D), "mlp.gate": mat(FF, W), "mlp.up": mat(FF, W), "mlp.down": mat(W, FF)}
     spec = {"type": "attention", "mlp": {"kind": "dense", "ff": FF},
@@ -275,6 +281,34 @@ def nafevik_model(ctx, hip_api, size, rng, f32=False):
     weights.update({"embed": mat(DESIGN_VOCAB, W, 1.0), "pos": mat(DESIGN_CTX, W), "head": mat(DESIGN_VOCAB, W), "final.norm": 1 + vec(W),
                     "loop.in": mat(W, 2 * W), "loop.step": vec(1, W)})
     nbytes = DESIGN_LAYERS * sum(v.nbytes for v in layer.values() if v.dtype == np.uint16) + weights["head"].nbytes + weights["loop.in"].nbytes
+    return hip_api.LayeredModel(ctx, cfg, weights, DESIGN_CTX, f32), nbytes
+
+
+FIDINEX_STREAMS, FIDINEX_RANK, FIDINEX_ROT = 4, 512, 64
+
+
+def fidinex_model(ctx, hip_api, size, rng, f32=False):
+    """A random-init Fidinex of DESIGN_LAYERS layers: every fourth one latent attention (rank 512, 64 rotated entries), the
+    others grouped heads whose values mix; four streams.  (model, weight bytes a decode step reads)."""
+    W, FF, Hq, G, D = (size[k] for k in ("width", "ff", "heads", "kv_heads", "dim"))
+    mat, vec = _random(rng)
+    S, rank, rot = FIDINEX_STREAMS, FIDINEX_RANK, FIDINEX_ROT
+    hc = {f"hc{q}.{k}": v for q in (1, 2) for k, v in (("in", 1 / S + vec(S)), ("out", 0.7 + vec(S)), ("mix", 0.8 * np.eye(S, dtype=np.float32) + vec(S, S)))}
+    common = {"norm1": 1 + vec(W), "norm2": 1 + vec(W), "mix.sink": 1 + vec(Hq), "mix.o": mat(W, Hq * D), "mlp.up": mat(FF, W), "mlp.down": mat(W, FF), **hc}
+    att = {"mix.q": mat(Hq * D, W), "mix.k": mat(G * D, W), "mix.v": mat(G * D, W), "mix.q.norm": 1 + vec(D), "mix.k.norm": 1 + vec(D),
+           "mix.vmix": np.float32(0.4), **common}
+    lat = {"mix.q": mat(Hq * (D + rot), W), "mix.dkv": mat(rank + rot, W), "mix.dkv.norm": 1 + vec(rank), "mix.uk": mat(Hq * D, rank, 0.05),
+           "mix.uv": mat(Hq * D, rank, 0.05), **common}
+    mlp = {"kind": "dense", "ff": FF}
+    specs = {True: {"type": "latent_attention", "mlp": mlp, "mixer": {"heads": Hq, "dim": D, "rot_dim": rot, "vdim": D, "kv_rank": rank,
+                                                                     "rot": {"dims": rot, "base": 50000.0}, "scale": (D + rot) ** -0.5}},
+             False: {"type": "attention", "mlp": mlp, "mixer": {"heads": Hq, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "v_mix": True,
+                                                                "q_temp": {"coef": 0.1, "every": 1024}}}}
+    kinds = [i % 4 == 0 for i in range(DESIGN_LAYERS)]
+    cfg = {"architecture": "Fidinex", "width": W, "vocab": DESIGN_VOCAB, "streams": S, "norm": {"eps": 1e-6}, "layers": [specs[k] for k in kinds]}
+    weights = {f"l{i}.{k}": v for i, latent in enumerate(kinds) for k, v in (lat if latent else att).items()}
+    weights.update({"embed": mat(DESIGN_VOCAB, W, 1.0), "final.norm": 1 + vec(W)})
+    nbytes = sum(v.nbytes for v in weights.values() if v.dtype == np.uint16)   # the embedding is the head
     return hip_api.LayeredModel(ctx, cfg, weights, DESIGN_CTX, f32), nbytes
 
 
@@ -293,13 +327,13 @@ def llama_model(ctx, hip_api, H, size, quant, seed, n_thr):
 
 
 def measure_design(ctx, hip_api, H, args, n_thr):
-    """Prefill and decode rates of a Nafevik and of the llama of equal layer sizes, in turn, random weights."""
+    """Prefill and decode rates of a model design, of a Nafevik and of the llama of equal layer sizes, in turn, random weights."""
     rng = np.random.default_rng(args.seed)
     out = []
     for name in args.design_sizes.split(","):
         size = DESIGN_SIZES[name]
-        flops = 2 * DESIGN_LAYERS * (size["width"] * (2 * size["heads"] + 2 * size["kv_heads"]) * size["dim"] + 3 * size["width"] * size["ff"])
-        models = [("nafevik_bf16", *nafevik_model(ctx, hip_api, size, rng))]
+        models = [("fidinex_bf16", *fidinex_model(ctx, hip_api, size, rng))] if args.design == "fidinex" else []
+        models.append(("nafevik_bf16", *nafevik_model(ctx, hip_api, size, rng)))
         for quant in args.design_llama.split(",") if args.design_llama else []:
             models.append((f"llama_{quant}", *llama_model(ctx, hip_api, H, size, quant, args.seed, n_thr)))
         best = {m[0]: {} for m in models}
@@ -331,7 +365,9 @@ def measure_design(ctx, hip_api, H, args, n_thr):
             r["weight_bytes_per_step"] = nbytes
             r["decode_weight_GB/s"] = round(best[label]["decode_at_512_tok_s"] * nbytes / 1e9, 1)
             r["decode_frac_of_hbm_peak"] = round(r["decode_weight_GB/s"] / HBM_PEAK_GBS, 4)
-            r["prefill_2048_TFLOP/s"] = round(best[label]["prefill_2048_tok_s"] * flops / 1e12, 1)
+            if label.endswith("bf16"):   # two operations per weight the layers read, the head left out
+                flops = nbytes - 2 * DESIGN_VOCAB * size["width"]
+                r["prefill_2048_TFLOP/s"] = round(best[label]["prefill_2048_tok_s"] * flops / 1e12, 1)
             out.append({"size": name, "model": label, **r})
             m.close()
     return {"design": args.design, "layers": DESIGN_LAYERS, "vocab": DESIGN_VOCAB, "sizes": DESIGN_SIZES, "data": "synthetic, random-init weights",
@@ -371,9 +407,9 @@ def main() -> int:
                     help="run only a 1 GiB copy kernel, a few launches of each per-layer GEMV kernel, decode attention at "
                          "131072 and 8192 keys and the two prefill GEMMs at 2048 tokens, for a hardware-counter pass under "
                          "rocprofv3 --pmc; prints no JSON")
-    ap.add_argument("--design", choices=["nafevik"],
+    ap.add_argument("--design", choices=["nafevik", "fidinex"],
                     help="instead of the workload above: prefill and decode rates of this model design with random weights at a few "
-                         "layer sizes, beside the llama of equal size; prints one JSON line")
+                         "layer sizes, beside the llama of equal size (and the Nafevik, when it is another); prints one JSON line")
     ap.add_argument("--design-sizes", default=",".join(DESIGN_SIZES), help="of " + ", ".join(DESIGN_SIZES))
     ap.add_argument("--design-llama", default="q4_k_m,q8_0", help="type mixes of the llama beside it (empty: none)")
     ap.add_argument("--design-reps", type=int, default=3)

@@ -28,6 +28,12 @@ template <> struct ElemOps<__bf16> {
     __device__ static __forceinline__ void store4(__bf16* p, float a, float b, float c, float d) {
         *reinterpret_cast<bf16x4*>(p) = bf16x4{static_cast<__bf16>(a), static_cast<__bf16>(b), static_cast<__bf16>(c), static_cast<__bf16>(d)};
     }
+    __device__ static __forceinline__ void store8(__bf16* p, const float (&v)[8]) {
+        bf16x8 o;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) o[i] = static_cast<__bf16>(v[i]);
+        *reinterpret_cast<bf16x8*>(p) = o;
+    }
     // acc += 8 weights (two bf16 per dword) . 8 activations
     typedef uint4 X8;
     __device__ static __forceinline__ X8 ld8(const __bf16* p) { return *reinterpret_cast<const uint4*>(p); }
@@ -43,6 +49,10 @@ template <> struct ElemOps<float> {
     __device__ static __forceinline__ void store4(float* p, float a, float b, float c, float d) {
         *reinterpret_cast<float4*>(p) = make_float4(a, b, c, d);
     }
+    __device__ static __forceinline__ void store8(float* p, const float (&v)[8]) {
+        store4(p, v[0], v[1], v[2], v[3]);
+        store4(p + 4, v[4], v[5], v[6], v[7]);
+    }
     struct X8 { float4 a, b; };
     __device__ static __forceinline__ X8 ld8(const float* p) {
         return X8{reinterpret_cast<const float4*>(p)[0], reinterpret_cast<const float4*>(p)[1]};
@@ -54,3 +64,14 @@ template <> struct ElemOps<float> {
         acc = fmaf(bf16_lo(w.w), x.b.z, acc); return fmaf(bf16_hi(w.w), x.b.w, acc);
     }
 };
+
+// x[c .. c + 8) of a vector of n floats, zeros behind its end; whole: 16-byte aligned and in whole eights
+__device__ __forceinline__ void load8(const float* x, uint32_t c, uint32_t n, bool whole, float (&v)[8]) {
+    if (whole && c < n) {
+        const float4 a = *reinterpret_cast<const float4*>(x + c), b = *reinterpret_cast<const float4*>(x + c + 4);
+        v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+    } else {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] = c + i < n ? x[c + i] : 0.0f;
+    }
+}

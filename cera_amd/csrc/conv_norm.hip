@@ -22,12 +22,13 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(const uint16_t* __restri
 __global__ __launch_bounds__(256) void embed_streams_kernel(const uint16_t* __restrict__ embed, const uint32_t* __restrict__ tokens, uint32_t token,
                                                             uint32_t width, uint64_t ld, float* __restrict__ x, uint32_t streams, uint64_t stride,
                                                             float u_scale, float* __restrict__ u) {
-    const uint32_t t = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
+    const uint32_t t = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * 4;   // ld is a multiple of 4
     if (c >= ld) return;
-    const uint64_t tok = tokens ? tokens[t] : token;
-    const float v = c < width ? bf16_at(embed, tok * width + c) : 0.0f;
-    for (uint32_t s = 0; s < streams; ++s) x[s * stride + t * ld + c] = v;
-    u[t * ld + c] = u_scale * v;
+    const uint16_t* const row = embed + static_cast<uint64_t>(tokens ? tokens[t] : token) * width;
+    const float4 v = make_float4(c < width ? bf16_at(row, c) : 0.0f, c + 1 < width ? bf16_at(row, c + 1) : 0.0f,
+                                 c + 2 < width ? bf16_at(row, c + 2) : 0.0f, c + 3 < width ? bf16_at(row, c + 3) : 0.0f);
+    for (uint32_t s = 0; s < streams; ++s) *reinterpret_cast<float4*>(x + s * stride + t * ld + c) = v;
+    *reinterpret_cast<float4*>(u + t * ld + c) = make_float4(u_scale * v.x, u_scale * v.y, u_scale * v.z, u_scale * v.w);
 }
 
 // A workgroup takes `rows` consecutive rows: first 1 / rms of those rows and of the taps - 1 before them
@@ -133,7 +134,8 @@ cera_hip_status cera_launch_embed_pos(cera_hip_ctx* ctx, const void* embed, cons
 
 cera_hip_status cera_launch_embed_streams(cera_hip_ctx* ctx, const void* embed, const uint32_t* tokens, uint32_t token, uint32_t n, uint32_t width,
                                           uint64_t ld, float* x, uint32_t streams, uint64_t stride, float u_scale, float* u) {
-    hipLaunchKernelGGL(embed_streams_kernel, dim3(static_cast<uint32_t>((ld + 255) / 256), n), dim3(256), 0, ctx->stream,
+    if (ld % 4 || stride % 4) return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "embed_streams: rows in whole vectors");
+    hipLaunchKernelGGL(embed_streams_kernel, dim3(static_cast<uint32_t>((ld + 1023) / 1024), n), dim3(256), 0, ctx->stream,
                        static_cast<const uint16_t*>(embed), tokens, token, width, ld, x, streams, stride, u_scale, u);
     HIP_TRY(ctx, hipGetLastError());
     return CERA_HIP_OK;

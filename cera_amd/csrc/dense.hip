@@ -30,18 +30,20 @@ struct GemmDArgs {
     float mult;
     uint32_t out_rows;
     float* part;           // split K: [split][n][m] f32
-    uint64_t gw, gx, go;   // groups (blockIdx.z): elements between their matrices, inputs and outputs
+    uint32_t groups;
+    uint64_t gw, gx, go;   // between the groups: elements of their matrices and inputs, bytes of their outputs
     bool vec;              // four outputs of a token in a row may be stored as one vector
     float* u;
     DenseStreams st;
 };
 
-// four consecutive channels of every stream (n < 4: the first n of them)
-template <int S> __device__ __forceinline__ void dense_streams4(const DenseStreams& st, float* x, float* u, bool vec, int n, const float (&y)[4]) {
+// four consecutive channels of every stream (n < 4: the first n of them).  S: the number of streams, 0: any, at run time
+template <int SN> __device__ __forceinline__ void dense_streams4(const DenseStreams& st, float* x, float* u, bool vec, int n, const float (&y)[4]) {
+    constexpr int S = SN ? SN : static_cast<int>(DENSE_MAX_STREAMS);
     float o[S][4];
 #pragma unroll
     for (int s = 0; s < S; ++s)
-        if (s < static_cast<int>(st.count)) {
+        if (SN || s < static_cast<int>(st.count)) {
             float* const p = x + s * st.stride;
             if (vec) {
                 const float4 v = *reinterpret_cast<const float4*>(p);
@@ -54,14 +56,14 @@ template <int S> __device__ __forceinline__ void dense_streams4(const DenseStrea
     float sum[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int t = 0; t < S; ++t)
-        if (t < static_cast<int>(st.count)) {
+        if (SN || t < static_cast<int>(st.count)) {
             float v[4];
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 v[i] = st.out[t] * y[i];
 #pragma unroll
                 for (int s = 0; s < S; ++s)
-                    if (s < static_cast<int>(st.count)) v[i] = fmaf(st.mix[s][t], o[s][i], v[i]);
+                    if (SN || s < static_cast<int>(st.count)) v[i] = fmaf(st.mix[s][t], o[s][i], v[i]);
                 sum[i] = fmaf(st.next[t], v[i], sum[i]);
             }
             float* const p = x + t * st.stride;
@@ -78,18 +80,19 @@ template <int S> __device__ __forceinline__ void dense_streams4(const DenseStrea
             if (i < n) u[i] = sum[i];
 }
 // one channel of every stream
-__device__ __forceinline__ void dense_streams1(const DenseStreams& st, float* x, float* u, float y) {
-    float o[DENSE_MAX_STREAMS], sum = 0.0f;
+template <int SN> __device__ __forceinline__ void dense_streams1(const DenseStreams& st, float* x, float* u, float y) {
+    constexpr int S = SN ? SN : static_cast<int>(DENSE_MAX_STREAMS);
+    float o[S], sum = 0.0f;
 #pragma unroll
-    for (int s = 0; s < static_cast<int>(DENSE_MAX_STREAMS); ++s)
-        if (s < static_cast<int>(st.count)) o[s] = x[s * st.stride];
+    for (int s = 0; s < S; ++s)
+        if (SN || s < static_cast<int>(st.count)) o[s] = x[s * st.stride];
 #pragma unroll
-    for (int t = 0; t < static_cast<int>(DENSE_MAX_STREAMS); ++t)
-        if (t < static_cast<int>(st.count)) {
+    for (int t = 0; t < S; ++t)
+        if (SN || t < static_cast<int>(st.count)) {
             float v = st.out[t] * y;
 #pragma unroll
-            for (int s = 0; s < static_cast<int>(DENSE_MAX_STREAMS); ++s)
-                if (s < static_cast<int>(st.count)) v = fmaf(st.mix[s][t], o[s], v);
+            for (int s = 0; s < S; ++s)
+                if (SN || s < static_cast<int>(st.count)) v = fmaf(st.mix[s][t], o[s], v);
             x[t * st.stride] = v;
             sum = fmaf(st.next[t], v, sum);
         }
@@ -101,9 +104,10 @@ __device__ __forceinline__ float dense_relu2(float y) {
 }
 
 // ---- epilogues on four consecutive rows m .. m+3 of one token -----------------------------------
-template <typename T> __device__ __forceinline__ void dense_store4(const GemmDArgs& a, uint32_t row, uint32_t tok, f32x4 v) {
-    const uint64_t at = blockIdx.z * a.go + static_cast<uint64_t>(tok) * a.ldo + row;
-    if (a.epi == DENSE_STORE) {
+// EPI: a DenseEpilogue; SN: of DENSE_STREAMS
+template <typename T, int EPI, int SN> __device__ __forceinline__ void dense_store4(const GemmDArgs& a, uint32_t row, uint32_t tok, f32x4 v) {
+    const uint64_t at = static_cast<uint64_t>(tok) * a.ldo + row;
+    if constexpr (EPI == DENSE_STORE) {
         float* o = static_cast<float*>(a.out) + at;
         if (row + 4 <= a.m && a.vec) {
             if (a.bias) {
@@ -116,9 +120,9 @@ template <typename T> __device__ __forceinline__ void dense_store4(const GemmDAr
             for (int i = 0; i < 4; ++i)
                 if (row + i < a.m) o[i] = a.bias ? v[i] + a.bias[row + i] : v[i];
         }
-    } else if (a.epi == DENSE_CAST || a.epi == DENSE_RELU2) {
+    } else if constexpr (EPI == DENSE_CAST || EPI == DENSE_RELU2) {
         T* o = static_cast<T*>(a.out) + at;
-        if (a.epi == DENSE_RELU2) { v.x = dense_relu2(v.x); v.y = dense_relu2(v.y); v.z = dense_relu2(v.z); v.w = dense_relu2(v.w); }
+        if (EPI == DENSE_RELU2) { v.x = dense_relu2(v.x); v.y = dense_relu2(v.y); v.z = dense_relu2(v.z); v.w = dense_relu2(v.w); }
         if (row + 4 <= a.m && a.vec) {
             ElemOps<T>::store4(o, v.x, v.y, v.z, v.w);
         } else {
@@ -126,12 +130,11 @@ template <typename T> __device__ __forceinline__ void dense_store4(const GemmDAr
             for (int i = 0; i < 4; ++i)
                 if (row + i < a.m) o[i] = ElemOps<T>::from(v[i]);
         }
-    } else if (a.epi == DENSE_STREAMS) {
+    } else if constexpr (EPI == DENSE_STREAMS) {
         const float y[4] = {v.x, v.y, v.z, v.w};
         float* const x = static_cast<float*>(a.out) + at;
         const int n = static_cast<int>(min(4u, a.m - row));
-        if (a.st.count <= 4) dense_streams4<4>(a.st, x, a.u + at, n == 4 && a.vec, n, y);
-        else dense_streams4<DENSE_MAX_STREAMS>(a.st, x, a.u + at, n == 4 && a.vec, n, y);
+        dense_streams4<SN>(a.st, x, a.u + at, n == 4 && a.vec, n, y);
     } else {
         float* o = static_cast<float*>(a.out) + at;
         if (row + 4 <= a.m && a.vec) {
@@ -162,7 +165,7 @@ __device__ __forceinline__ void dense_swiglu4(const GemmDArgs& a, uint32_t i0, u
     }
 }
 // one wavefront's tile: acc[mi][ni], rows m0 + 16 mi + 4 (lane / 16) + i, token n0 + 16 ni + lane % 16
-template <typename T, int MI, int NI>
+template <typename T, int EPI, int SN, int MI, int NI>
 __device__ __forceinline__ void dense_epilogue(const GemmDArgs& a, uint32_t m0, uint32_t n0, uint32_t lane, uint32_t z,
                                                f32x4 (&acc)[MI][NI]) {
     const uint32_t g4 = (lane >> 4) * 4;
@@ -181,7 +184,7 @@ __device__ __forceinline__ void dense_epilogue(const GemmDArgs& a, uint32_t m0, 
                     for (int i = 0; i < 4; ++i)
                         if (row + i < a.m) p[row + i] = acc[mi][ni][i];
             }
-        } else if (a.epi == DENSE_SWIGLU) {
+        } else if constexpr (EPI == DENSE_SWIGLU) {
             static_assert(MI % 2 == 0, "a wavefront holds gate rows with their up rows");
 #pragma unroll
             for (int mi = 0; mi < MI; mi += 2) {
@@ -192,34 +195,36 @@ __device__ __forceinline__ void dense_epilogue(const GemmDArgs& a, uint32_t m0, 
 #pragma unroll
             for (int mi = 0; mi < MI; ++mi) {
                 const uint32_t row = m0 + 16 * mi + g4;
-                if (row < a.m) dense_store4<T>(a, row, tok, acc[mi][ni]);
+                if (row < a.m) dense_store4<T, EPI, SN>(a, row, tok, acc[mi][ni]);
             }
         }
     }
 }
 
-// Workgroups go to the eight XCDs round robin in launch order; the token tiles of one weight tile
+// Workgroups go to the eight XCDs round robin in launch order; the token tiles of one weight tile (of one group)
 // take indices 8 apart, so one XCD's L2 reads that weight tile for all of them.
-__device__ __forceinline__ bool dense_tile(const GemmDArgs& a, uint32_t& tm, uint32_t& tn) {
+__device__ __forceinline__ bool dense_tile(const GemmDArgs& a, uint32_t& tm, uint32_t& tn, uint32_t& group) {
     const uint32_t b = blockIdx.x, xcd = b & 7, t = b >> 3;
     tn = t % a.tiles_n;
-    tm = (t / a.tiles_n) * 8 + xcd;
-    return tm < a.tiles_m;
+    const uint32_t i = (t / a.tiles_n) * 8 + xcd;
+    group = a.groups > 1 ? i / a.tiles_m : 0;
+    tm = i - group * a.tiles_m;
+    return i < a.tiles_m * a.groups;
 }
 
 // BM x BN tile, four wavefronts as WM x WN
-template <int BM, int BN, int WM, int WN>
+template <int EPI, int SN, int BM, int BN, int WM, int WN>
 __global__ __launch_bounds__(256) void dense_gemm_bf16_kernel(GemmDArgs a) {
     constexpr int BK = 64, TM = BM / WM, TN = BN / WN, MI = TM / 16, NI = TN / 16;
     constexpr int SEGS = (BM + BN) / 8;   // 1 KB pieces: eight rows of one K step
     static_assert(WM * WN == 4 && SEGS % 4 == 0 && MI >= 1 && NI >= 1, "tile shape");
     __shared__ __align__(1024) __bf16 lds[2][(BM + BN) * BK];
-    uint32_t tm, tn;
-    if (!dense_tile(a, tm, tn)) return;
+    uint32_t tm, tn, group;
+    if (!dense_tile(a, tm, tn, group)) return;
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const uint32_t k0 = blockIdx.y * a.k_chunk, k1 = min(a.kp, k0 + a.k_chunk);
-    const __bf16* const w = a.w + blockIdx.z * a.gw;
-    const __bf16* const x = static_cast<const __bf16*>(a.x) + blockIdx.z * a.gx;
+    const __bf16* const w = a.w + group * a.gw;
+    const __bf16* const x = static_cast<const __bf16*>(a.x) + group * a.gx;
     // this lane's source address per 1 KB piece; rows past the matrix / batch re-read the last one
     const uint32_t sub = lane >> 3, slot = lane & 7, chunk = (slot ^ sub) * 8;
     const __bf16* src[SEGS / 4];
@@ -267,20 +272,21 @@ __global__ __launch_bounds__(256) void dense_gemm_bf16_kernel(GemmDArgs a) {
                     acc[mi][ni] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[mi], fb[ni], acc[mi][ni], 0, 0, 0);
         }
     }
-    dense_epilogue<__bf16, MI, NI>(a, tm * BM + wm * TM, tn * BN + wn * TN, lane, blockIdx.y, acc);
+    a.out = static_cast<char*>(a.out) + group * a.go;
+    dense_epilogue<__bf16, EPI, SN, MI, NI>(a, tm * BM + wm * TM, tn * BN + wn * TN, lane, blockIdx.y, acc);
 }
 
 // 64 x 64 tile in true f32: weights widened on their way into LDS, K in steps of 32.  A lane's four
 // consecutive k of a 16-wide block feed four MFMA steps (the same k order in both operands).
-__global__ __launch_bounds__(256) void dense_gemm_f32_kernel(GemmDArgs a) {
+template <int EPI, int SN> __global__ __launch_bounds__(256) void dense_gemm_f32_kernel(GemmDArgs a) {
     constexpr int BM = 64, BN = 64, BK = 32, LD = BK + 4;
     __shared__ __align__(16) float lw[BM * LD], lx[BN * LD];
-    uint32_t tm, tn;
-    if (!dense_tile(a, tm, tn)) return;
+    uint32_t tm, tn, group;
+    if (!dense_tile(a, tm, tn, group)) return;
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const uint32_t k0 = blockIdx.y * a.k_chunk, k1 = min(a.kp, k0 + a.k_chunk);
-    const __bf16* const w0 = a.w + blockIdx.z * a.gw;
-    const float* const x = static_cast<const float*>(a.x) + blockIdx.z * a.gx;
+    const __bf16* const w0 = a.w + group * a.gw;
+    const float* const x = static_cast<const float*>(a.x) + group * a.gx;
     const uint32_t r = threadIdx.x >> 2, c = (threadIdx.x & 3) * 8;   // eight k of one row per thread
     const __bf16* const ws = w0 + static_cast<uint64_t>(min(tm * BM + r, a.m - 1)) * a.kp + c;
     const float* const xs = x + static_cast<uint64_t>(min(tn * BN + r, a.n - 1)) * a.ldx + c;
@@ -316,14 +322,15 @@ __global__ __launch_bounds__(256) void dense_gemm_f32_kernel(GemmDArgs a) {
                         acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(fa[i][s], fb[j][s], acc[i][j], 0, 0, 0);
         }
     }
-    dense_epilogue<float, 2, 2>(a, tm * BM + wm * 32, tn * BN + wn * 32, lane, blockIdx.y, acc);
+    a.out = static_cast<char*>(a.out) + group * a.go;
+    dense_epilogue<float, EPI, SN, 2, 2>(a, tm * BM + wm * 32, tn * BN + wn * 32, lane, blockIdx.y, acc);
 }
 
 // split K: adds the partial sums in split order, then the epilogue.  One thread per four rows of a token
 // (SWIGLU: per four outputs).
-template <typename T>
+template <typename T, int EPI, int SN>
 __global__ __launch_bounds__(256) void dense_reduce_kernel(GemmDArgs a, uint32_t split) {
-    const uint32_t quads = a.epi == DENSE_SWIGLU ? (a.m / 2 + 3) / 4 : (a.m + 3) / 4;
+    const uint32_t quads = EPI == DENSE_SWIGLU ? (a.m / 2 + 3) / 4 : (a.m + 3) / 4;
     const uint64_t t = static_cast<uint64_t>(blockIdx.x) * 256 + threadIdx.x;
     if (t >= static_cast<uint64_t>(quads) * a.n) return;
     const uint32_t tok = static_cast<uint32_t>(t / quads), q = static_cast<uint32_t>(t % quads) * 4;
@@ -344,11 +351,11 @@ __global__ __launch_bounds__(256) void dense_reduce_kernel(GemmDArgs a, uint32_t
         }
         return v;
     };
-    if (a.epi == DENSE_SWIGLU) {
+    if constexpr (EPI == DENSE_SWIGLU) {
         const uint32_t row = (q >> 4) * 32 + (q & 15);
         dense_swiglu4<T>(a, q, tok, sum4(row), sum4(row + 16));
     } else {
-        dense_store4<T>(a, q, tok, sum4(q));
+        dense_store4<T, EPI, SN>(a, q, tok, sum4(q));
     }
 }
 
@@ -369,7 +376,7 @@ template <int R> constexpr uint32_t GEMV_STEP = 64 * 8 * GEMV_U<R>;
 
 // Fills the workgroup's activation vector xs[0, stage_len).
 template <typename T, int KIND>
-__device__ __forceinline__ void gemv_stage(const GemvDArgs& a, bool second, bool store_h, T* xs, float* red) {
+__device__ __forceinline__ void gemv_stage(const GemvDArgs& a, bool second, bool store_h, T* xs, float* red, float* wz) {
     const DenseIn& in = a.in;
     if (KIND == DenseIn::RAW) {
         const T* x = static_cast<const T*>(in.x);
@@ -381,20 +388,22 @@ __device__ __forceinline__ void gemv_stage(const GemvDArgs& a, bool second, bool
         const T* x = static_cast<const T*>(in.x);
         const SAttnPartials& m = in.merge;
         const uint32_t cols = m.heads * m.vdim, cols_p = (cols + DENSE_PAD - 1) / DENSE_PAD * DENSE_PAD;
+        partials_weights(m, 0, m.heads, threadIdx.x, GEMV_WAVES * 64, wz);
         constexpr uint32_t V = 16 / sizeof(T);
 #pragma unroll 4
         for (uint32_t i = cols_p + threadIdx.x * V; i < a.stage_len; i += GEMV_WAVES * 64 * V)
             *reinterpret_cast<uint4*>(xs + i) = i < a.kp ? *reinterpret_cast<const uint4*>(x + i) : make_uint4(0, 0, 0, 0);
+        lds_barrier();
 #pragma unroll 2
         for (uint32_t i = threadIdx.x * 4; i < cols_p; i += GEMV_WAVES * 256) {
             if (i + 4 <= cols && m.vdim % 4 == 0) {
                 const uint32_t h = i / m.vdim;
-                const f32x4 s = partials_sum4(m, h, i - h * m.vdim);
+                const f32x4 s = partials_sum4(m, wz + h * m.splits, h, i - h * m.vdim);
                 ElemOps<T>::store4(xs + i, s.x, s.y, s.z, s.w);
             } else {
 #pragma unroll
                 for (uint32_t e = i; e < i + 4; ++e) {
-                    const float s = e < cols ? partials_sum(m, e / m.vdim, e % m.vdim) : 0.0f;
+                    const float s = e < cols ? partials_sum(m, wz + e / m.vdim * m.splits, e / m.vdim, e % m.vdim) : 0.0f;
                     xs[e] = ElemOps<T>::from(s);
                 }
             }
@@ -443,7 +452,8 @@ __device__ __forceinline__ void gemv_stage(const GemvDArgs& a, bool second, bool
 // One wavefront's walk over its groups of R rows (g, g + GEMV_WAVES, ... below g1) of one matrix, a step of
 // U * 64 16-byte chunks at a time; SWIGLU: a group is R / 2 gate rows and their up rows.  Two step buffers
 // alternate, the next step's loads -- of the next group too -- going out before the current one is multiplied.
-template <typename T, int R> struct GemvWalk {
+// SN: streams of the epilogue (0: any number, -1: it is another one)
+template <typename T, int R, int SN> struct GemvWalk {
     static constexpr int U = GEMV_U<R>, H = R > 1 ? R / 2 : 1;
     typedef uint4 Buf[U][R];
     const __bf16* w;
@@ -515,9 +525,9 @@ template <typename T, int R> struct GemvWalk {
                 if (lane == static_cast<uint32_t>(r)) y = acc[r];
             if (lane < static_cast<uint32_t>(R) && i < rows) {
                 float* out = static_cast<float*>(o.out) + i;
-                if (o.epi == DENSE_ADD) *out = fmaf(o.mult, y, *out);
+                if constexpr (SN >= 0) dense_streams1<SN>(st, out, o.u + i, y);
+                else if (o.epi == DENSE_ADD) *out = fmaf(o.mult, y, *out);
                 else if (o.epi == DENSE_STORE) *out = o.bias ? y + o.bias[i] : y;
-                else if (o.epi == DENSE_STREAMS) dense_streams1(st, out, o.u + i, y);
                 else static_cast<T*>(o.out)[i] = ElemOps<T>::from(o.epi == DENSE_RELU2 ? dense_relu2(y) : y);
             }
         }
@@ -527,10 +537,10 @@ template <typename T, int R> struct GemvWalk {
     }
 };
 
-template <typename T, int KIND, int R>
+template <typename T, int KIND, int R, int SN>
 __global__ __launch_bounds__(GEMV_WAVES * 64) void dense_gemv_kernel(GemvDArgs a) {
     extern __shared__ __align__(16) unsigned char smem[];
-    __shared__ float red[GEMV_WAVES];
+    __shared__ float red[GEMV_WAVES], wz[KIND == DenseIn::MERGE ? PARTIALS_MAX : 1];
     T* const xs = reinterpret_cast<T*>(smem);
     const bool second = blockIdx.x >= a.blocks_a;
     const uint32_t groups = second ? a.groups_b : a.groups_a, blocks = second ? a.blocks_b : a.blocks_a;
@@ -539,13 +549,13 @@ __global__ __launch_bounds__(GEMV_WAVES * 64) void dense_gemv_kernel(GemvDArgs a
     const uint32_t each = groups / blocks, more = groups % blocks;
     const uint32_t g0 = b * each + min(b, more), g1 = g0 + each + (b < more ? 1 : 0);
     const DenseOut& o = second ? a.ob : a.oa;
-    GemvWalk<T, R> walk;
-    typename GemvWalk<T, R>::Buf w0, w1;
+    GemvWalk<T, R, SN> walk;
+    typename GemvWalk<T, R, SN>::Buf w0, w1;
     uint32_t g = g0 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), k = 0;
     walk.begin(second ? a.wb : a.wa, second ? a.rows_b : a.rows_a, a.kp, a.stage_len, o.epi == DENSE_SWIGLU, g, g1);
     // the first weights are on their way while the activation vector is prepared
     bool more0 = walk.load(w0);
-    gemv_stage<T, KIND>(a, second, KIND == DenseIn::NORM && a.in.h_out && blockIdx.x == 0, xs, red);
+    gemv_stage<T, KIND>(a, second, KIND == DenseIn::NORM && a.in.h_out && blockIdx.x == 0, xs, red, wz);
     while (more0) {
         const bool more1 = walk.load(w1);
         walk.use(w0, g, k, xs, o, a.st);
@@ -571,10 +581,11 @@ cera_hip_status cera_launch_dense_gemm(cera_hip_ctx* ctx, const DenseMat& w, con
     if (n == 0 || w.rows == 0 || groups.count == 0 || w.rows % groups.count || w.kp == 0 || w.kp % DENSE_PAD || ldx < w.kp || ldx % 8)
         return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemm: bad shape");
     if (o.epi == DENSE_SWIGLU && w.rows % 32) return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemm: gate | up rows come in groups of 32");
-    if (o.epi == DENSE_STREAMS && !streams_ok(o)) return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemm: streams");
+    if (o.epi == DENSE_STREAMS && (!streams_ok(o) || groups.count != 1)) return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemm: streams");
     GemmDArgs a{};
     a.w = static_cast<const __bf16*>(w.w); a.x = x; a.ldx = ldx; a.m = w.rows / groups.count; a.n = n; a.kp = w.kp;
-    a.gw = static_cast<uint64_t>(a.m) * w.kp; a.gx = groups.x_stride; a.go = groups.out_stride;
+    a.gw = static_cast<uint64_t>(a.m) * w.kp; a.groups = groups.count; a.gx = groups.x_stride;
+    a.go = groups.out_stride * (f32 || (o.epi != DENSE_CAST && o.epi != DENSE_RELU2 && o.epi != DENSE_SWIGLU) ? 4 : 2);
     a.vec = (o.ld & 3) == 0 && (groups.out_stride & 3) == 0;
     a.u = o.u;
     if (o.streams) a.st = *o.streams;
@@ -597,24 +608,39 @@ cera_hip_status cera_launch_dense_gemm(cera_hip_ctx* ctx, const DenseMat& w, con
     const uint32_t per = (steps + split - 1) / split;
     split = (steps + per - 1) / per;
     a.k_chunk = per * DENSE_PAD;
-    if (split > 1) {
+    // any number of streams but four: through the reduction, whose threads hold little else
+    const bool apart = o.epi == DENSE_STREAMS && o.streams->count != 4;
+    if (split > 1 || apart) {
         void* part;
         CERA_TRY(cera_scratch(ctx, 9, static_cast<uint64_t>(split) * n * a.m * sizeof(float), &part));
         a.part = static_cast<float*>(part);
     }
-    const dim3 grid((a.tiles_m + 7) / 8 * 8 * a.tiles_n, split, groups.count);
-    if (f32) hipLaunchKernelGGL(dense_gemm_f32_kernel, grid, dim3(256), 0, ctx->stream, a);
-    else if (shape == 0) hipLaunchKernelGGL((dense_gemm_bf16_kernel<128, 128, 2, 2>), grid, dim3(256), 0, ctx->stream, a);
-    else if (shape == 1) hipLaunchKernelGGL((dense_gemm_bf16_kernel<64, 64, 2, 2>), grid, dim3(256), 0, ctx->stream, a);
-    else hipLaunchKernelGGL((dense_gemm_bf16_kernel<64, 32, 2, 2>), grid, dim3(256), 0, ctx->stream, a);
-    HIP_TRY(ctx, hipGetLastError());
-    if (split > 1) {
-        const uint64_t quads = (a.epi == DENSE_SWIGLU ? (a.m / 2 + 3) / 4 : (a.m + 3) / 4) * static_cast<uint64_t>(n);
-        const dim3 rg(static_cast<uint32_t>((quads + 255) / 256));
-        if (f32) hipLaunchKernelGGL(dense_reduce_kernel<float>, rg, dim3(256), 0, ctx->stream, a, split);
-        else hipLaunchKernelGGL(dense_reduce_kernel<__bf16>, rg, dim3(256), 0, ctx->stream, a, split);
-        HIP_TRY(ctx, hipGetLastError());
+    const dim3 grid((a.tiles_m * groups.count + 7) / 8 * 8 * a.tiles_n, split);
+    const uint64_t quads = (a.epi == DENSE_SWIGLU ? (a.m / 2 + 3) / 4 : (a.m + 3) / 4) * static_cast<uint64_t>(n);
+    const dim3 rg(static_cast<uint32_t>((quads + 255) / 256)), block(256);
+    auto go = [&](auto epi, auto streams) {
+        constexpr int E = decltype(epi)::value, SN = decltype(streams)::value;
+        constexpr int EG = E == DENSE_STREAMS && SN == 0 ? DENSE_STORE : E;   // leaves partial sums, whatever it is
+        if (f32) hipLaunchKernelGGL((dense_gemm_f32_kernel<EG, SN>), grid, block, 0, ctx->stream, a);
+        else if (shape == 0) hipLaunchKernelGGL((dense_gemm_bf16_kernel<EG, SN, 128, 128, 2, 2>), grid, block, 0, ctx->stream, a);
+        else if (shape == 1) hipLaunchKernelGGL((dense_gemm_bf16_kernel<EG, SN, 64, 64, 2, 2>), grid, block, 0, ctx->stream, a);
+        else hipLaunchKernelGGL((dense_gemm_bf16_kernel<EG, SN, 64, 32, 2, 2>), grid, block, 0, ctx->stream, a);
+        if (!a.part) return;
+        if (f32) hipLaunchKernelGGL((dense_reduce_kernel<float, E, SN>), rg, block, 0, ctx->stream, a, split);
+        else hipLaunchKernelGGL((dense_reduce_kernel<__bf16, E, SN>), rg, block, 0, ctx->stream, a, split);
+    };
+    const std::integral_constant<int, 0> any{};
+    switch (a.epi) {
+        case DENSE_STORE: go(std::integral_constant<int, DENSE_STORE>{}, any); break;
+        case DENSE_ADD: go(std::integral_constant<int, DENSE_ADD>{}, any); break;
+        case DENSE_SWIGLU: go(std::integral_constant<int, DENSE_SWIGLU>{}, any); break;
+        case DENSE_CAST: go(std::integral_constant<int, DENSE_CAST>{}, any); break;
+        case DENSE_RELU2: go(std::integral_constant<int, DENSE_RELU2>{}, any); break;
+        default:
+            if (a.st.count == 4) go(std::integral_constant<int, DENSE_STREAMS>{}, std::integral_constant<int, 4>{});
+            else go(std::integral_constant<int, DENSE_STREAMS>{}, any);
     }
+    HIP_TRY(ctx, hipGetLastError());
     return CERA_HIP_OK;
 }
 
@@ -623,7 +649,10 @@ cera_hip_status cera_launch_dense_gemv(cera_hip_ctx* ctx, const DenseIn& in, con
     *launched = false;
     if (wa.rows == 0 || wa.kp == 0 || wa.kp % DENSE_PAD || (wb && wb->kp != wa.kp))
         return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemv: bad shape");
-    if (oa.epi == DENSE_STREAMS && !streams_ok(oa)) return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemv: streams");
+    if (oa.epi == DENSE_STREAMS && (!streams_ok(oa) || wb || (in.kind != DenseIn::RAW && in.kind != DenseIn::MERGE)))
+        return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemv: streams take one matrix and a finished or partial input");
+    if (in.kind == DenseIn::MERGE && (!in.merge.part || in.merge.heads * in.merge.splits > PARTIALS_MAX))
+        return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "dense_gemv: partial results of too many heads and key ranges");
     GemvDArgs a{};
     if (oa.streams) a.st = *oa.streams;
     a.in = in;
@@ -651,10 +680,18 @@ cera_hip_status cera_launch_dense_gemv(cera_hip_ctx* ctx, const DenseIn& in, con
     auto go = [&](auto tag, auto rows) {
         using T = decltype(tag);
         constexpr int R = decltype(rows)::value;
-        if (in.kind == DenseIn::RAW) hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::RAW, R>), grid, block, lds, ctx->stream, a);
-        else if (in.kind == DenseIn::MERGE) hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::MERGE, R>), grid, block, lds, ctx->stream, a);
-        else if (in.kind == DenseIn::NORM) hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::NORM, R>), grid, block, lds, ctx->stream, a);
-        else hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::CONCAT, R>), grid, block, lds, ctx->stream, a);
+        auto kind = [&](auto streams) {
+            constexpr int SN = decltype(streams)::value;
+            if (in.kind == DenseIn::RAW) hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::RAW, R, SN>), grid, block, lds, ctx->stream, a);
+            else if (in.kind == DenseIn::MERGE) hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::MERGE, R, SN>), grid, block, lds, ctx->stream, a);
+            else if constexpr (SN < 0) {
+                if (in.kind == DenseIn::NORM) hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::NORM, R, SN>), grid, block, lds, ctx->stream, a);
+                else hipLaunchKernelGGL((dense_gemv_kernel<T, DenseIn::CONCAT, R, SN>), grid, block, lds, ctx->stream, a);
+            }
+        };
+        if (oa.epi != DENSE_STREAMS) kind(std::integral_constant<int, -1>{});
+        else if (a.st.count == 4) kind(std::integral_constant<int, 4>{});
+        else kind(std::integral_constant<int, 0>{});
     };
     auto by_rows = [&](auto tag) {
         if (r == 4) go(tag, std::integral_constant<int, 4>{});

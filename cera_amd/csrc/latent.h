@@ -43,5 +43,8 @@ cera_hip_status cera_launch_latent_spread(cera_hip_ctx* ctx, const LatentShape& 
 // One token, absorbed: the preparation above and q' = W_uk^T q in one launch.  wk [heads][rank_p][dim_p].
 cera_hip_status cera_launch_latent_step(cera_hip_ctx* ctx, const LatentShape& l, const FAttnShape& absorbed, const DenseMat& wk, const float* x,
                                         uint32_t pos, void* cache, void* q, bool f32);
-// One token: adds attention's partial results up and applies W_uv; wv [heads * vdim][rank_p], out T, head h at h * vdim.
-cera_hip_status cera_launch_latent_values(cera_hip_ctx* ctx, const LatentShape& l, const DenseMat& wv, const SAttnPartials& parts, void* out, bool f32);
+// One token: adds attention's partial results up (at most LATENT_PARTS; parts.part null: `merged` [heads][rank_p] T holds
+// the sum) and applies W_uv; wv [heads * vdim][rank_p], out T, head h at h * vdim.
+constexpr uint32_t LATENT_PARTS = 32;
+cera_hip_status cera_launch_latent_values(cera_hip_ctx* ctx, const LatentShape& l, const DenseMat& wv, const SAttnPartials& parts, const void* merged,
+                                          void* out, bool f32);

@@ -13,6 +13,7 @@ struct LArgs {
     uint64_t ld;
     uint32_t n, start, kp, rank_p, dim_p, row, rot_p;
     void *cache, *q, *qn;
+    bool whole;               // query heads start 16-byte aligned and their unrotated part is in whole eights
     const __bf16* w;          // step: per-head matrices
     uint32_t slices, rows;    // step: workgroups and rows per head
     SAttnPartials parts;
@@ -38,27 +39,29 @@ template <typename T> __device__ __forceinline__ void latent_append(const LArgs&
         dst[a.rank_p + c] = ElemOps<T>::from(c < l.rot_dim ? rotated(l, down + l.rank, c, pos) : 0.0f);
 }
 
-// a wavefront per query head, and one for the cache row
+// sixteen lanes per query head, eight entries each at a time, and a wavefront for the cache row
 template <typename T> __global__ __launch_bounds__(256) void latent_prep_kernel(LArgs a) {
     const LatentShape& l = a.l;
-    const uint32_t lane = threadIdx.x & 63, item = blockIdx.x * 4 + (threadIdx.x >> 6), tok = blockIdx.y, pos = a.start + tok;
-    if (item > l.heads) return;
+    const uint32_t lane = threadIdx.x & 63, l8 = (lane & 15) * 8, item = blockIdx.x * 16 + (threadIdx.x >> 4), tok = blockIdx.y, pos = a.start + tok;
     const float* const row = a.x + tok * a.ld;
-    if (item == l.heads) {
-        latent_append<T>(a, row + l.heads * (l.dim + l.rot_dim), pos, lane);
+    if (blockIdx.x == gridDim.x - 1) {
+        if (threadIdx.x < 64) latent_append<T>(a, row + l.heads * (l.dim + l.rot_dim), pos, lane);
         return;
     }
+    if (item >= l.heads) return;
     const float* const x = row + item * (l.dim + l.rot_dim);
     T* const q = static_cast<T*>(a.q) + (static_cast<uint64_t>(tok) * l.heads + item) * a.kp;
-    uint32_t at = l.dim;
-    if (a.qn) {
-        T* const qn = static_cast<T*>(a.qn) + (static_cast<uint64_t>(tok) * l.heads + item) * a.dim_p;
-        for (uint32_t c = lane; c < a.dim_p; c += 64) qn[c] = ElemOps<T>::from(c < l.dim ? x[c] : 0.0f);
-        at = a.rank_p;
-    } else {
-        for (uint32_t c = lane; c < l.dim; c += 64) q[c] = ElemOps<T>::from(x[c]);
+    float v[8];
+    // unrotated entries: whole eights, but in front of the rotated ones the last few one by one
+    T* const un = a.qn ? static_cast<T*>(a.qn) + (static_cast<uint64_t>(tok) * l.heads + item) * a.dim_p : q;
+    for (uint32_t c = l8; c < (a.qn ? a.dim_p : l.dim); c += 128) {
+        load8(x, c, l.dim, a.whole, v);
+        if (a.qn || c + 8 <= l.dim) ElemOps<T>::store8(un + c, v);
+        else
+            for (uint32_t i = 0; c + i < l.dim; ++i) un[c + i] = ElemOps<T>::from(x[c + i]);
     }
-    for (uint32_t c = lane; at + c < a.kp; c += 64) q[at + c] = ElemOps<T>::from(c < l.rot_dim ? rotated(l, x + l.dim, c, pos) : 0.0f);
+    const uint32_t at = a.qn ? a.rank_p : l.dim;
+    for (uint32_t c = lane & 15; at + c < a.kp; c += 16) q[at + c] = ElemOps<T>::from(c < l.rot_dim ? rotated(l, x + l.dim, c, pos) : 0.0f);
 }
 
 template <typename T>
@@ -114,9 +117,17 @@ template <typename T> __global__ __launch_bounds__(256) void latent_values_kerne
     T* const xs = reinterpret_cast<T*>(smem);
     const LatentShape& l = a.l;
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, head = blockIdx.x / a.slices, slice = blockIdx.x % a.slices;
-    for (uint32_t c = threadIdx.x * 4; c < a.rank_p; c += 1024) {
-        const f32x4 s = partials_sum4(a.parts, head, c);
-        ElemOps<T>::store4(xs + c, s.x, s.y, s.z, s.w);
+    if (a.parts.part) {
+        __shared__ float wz[LATENT_PARTS];
+        partials_weights(a.parts, head, 1, threadIdx.x, 256, wz);
+        __syncthreads();
+        for (uint32_t c = threadIdx.x * 4; c < a.rank_p; c += 1024) {
+            const f32x4 s = partials_sum4(a.parts, wz, head, c);
+            ElemOps<T>::store4(xs + c, s.x, s.y, s.z, s.w);
+        }
+    } else {
+        const T* const x = static_cast<const T*>(a.q) + static_cast<uint64_t>(head) * a.rank_p;
+        for (uint32_t c = threadIdx.x; c < a.rank_p; c += 256) xs[c] = x[c];
     }
     __syncthreads();
     const uint32_t r0 = slice * a.rows, r1 = min(r0 + a.rows, l.vdim);
@@ -146,7 +157,8 @@ cera_hip_status cera_launch_latent_prep(cera_hip_ctx* ctx, const LatentShape& l,
                                         uint32_t start, void* cache, void* q, uint32_t kp, void* qn, bool f32) {
     LArgs a = fill(l, absorbed);
     a.x = x; a.ld = ld; a.n = n; a.start = start; a.cache = cache; a.q = q; a.qn = qn; a.kp = kp;
-    const dim3 grid((l.heads + 1 + 3) / 4, n);
+    a.whole = l.dim % 8 == 0 && l.rot_dim % 4 == 0 && ld % 4 == 0;
+    const dim3 grid((l.heads + 15) / 16 + 1, n);
     if (f32) hipLaunchKernelGGL(latent_prep_kernel<float>, grid, dim3(256), 0, ctx->stream, a);
     else hipLaunchKernelGGL(latent_prep_kernel<__bf16>, grid, dim3(256), 0, ctx->stream, a);
     HIP_TRY(ctx, hipGetLastError());
@@ -182,10 +194,12 @@ cera_hip_status cera_launch_latent_step(cera_hip_ctx* ctx, const LatentShape& l,
     return CERA_HIP_OK;
 }
 
-cera_hip_status cera_launch_latent_values(cera_hip_ctx* ctx, const LatentShape& l, const DenseMat& wv, const SAttnPartials& parts, void* out, bool f32) {
+cera_hip_status cera_launch_latent_values(cera_hip_ctx* ctx, const LatentShape& l, const DenseMat& wv, const SAttnPartials& parts, const void* merged,
+                                          void* out, bool f32) {
     LArgs a{};
-    a.l = l; a.rank_p = l.rank_p(); a.parts = parts; a.out = out; a.w = static_cast<const __bf16*>(wv.w);
-    if (wv.rows != l.heads * l.vdim || wv.kp != a.rank_p || !parts.part || parts.vdim_p != a.rank_p || parts.heads != l.heads)
+    a.l = l; a.rank_p = l.rank_p(); a.parts = parts; a.q = const_cast<void*>(merged); a.out = out; a.w = static_cast<const __bf16*>(wv.w);
+    if (wv.rows != l.heads * l.vdim || wv.kp != a.rank_p ||
+        (parts.part ? parts.vdim_p != a.rank_p || parts.heads != l.heads || parts.splits > LATENT_PARTS : !merged))
         return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "latent values: matrix or partial results do not fit");
     slice_rows(ctx, a, l.heads, l.vdim);
     const dim3 grid(l.heads * a.slices);

@@ -78,7 +78,7 @@ struct CeraLayered {
     // sequential blocks: x holds all streams; the next sublayer's input, feed-forward activations, first mixing layer's values
     float u_scale = 1.0f;              // what the first sublayer reads of the embedding
     float *u = nullptr, *v_first = nullptr, *bu = nullptr, *bv_first = nullptr;
-    void *act = nullptr, *bqn = nullptr, *bo = nullptr;
+    void *act = nullptr, *lat = nullptr, *bqn = nullptr, *bo = nullptr;
 };
 
 // ---- shared between the two forms (layered.hip) ----

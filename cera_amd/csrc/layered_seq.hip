@@ -71,14 +71,18 @@ cera_hip_status seq_decode(cera_hip_model* m, uint32_t token, uint32_t pos, bool
         if (W.latent) {
             CERA_TRY(cera_launch_latent_step(ctx, W.lat, W.attn, W.k_up_t, g.qkvg, pos, W.kv, g.q, g.f32));
             SAttnPartials parts;
-            CERA_TRY(cera_launch_fattn(ctx, W.attn, p, &parts, g.f32));
-            CERA_TRY(cera_launch_latent_values(ctx, W.lat, W.v_up, parts, g.cat, g.f32));
+            p.out = g.lat; p.out_head = W.lat.rank_p(); p.out_ld = 0;
+            CERA_TRY(cera_launch_fattn(ctx, W.attn, p, &parts, LATENT_PARTS, g.f32));
+            CERA_TRY(cera_launch_latent_values(ctx, W.lat, W.v_up, parts, g.lat, g.cat, g.f32));
         } else {
             FAttnPrep prep = W.prep;
             prep.qkv = g.qkvg; prep.ld = W.in.rows; prep.v_first = W.v_mix ? g.v_first : nullptr;
             CERA_TRY(cera_launch_fattn_prep(ctx, W.attn, p, prep, g.f32));
-            CERA_TRY(cera_launch_fattn(ctx, W.attn, p, &raw.merge, g.f32));
-            raw.kind = DenseIn::MERGE;
+            p.out = g.cat; p.out_head = W.vdim; p.out_ld = W.o.kp;
+            // every workgroup of the output product reads all parts: 64 KB of them at the most
+            const uint32_t most = std::min(8u, std::max(1u, 16384u / (W.attn.heads * W.attn.vp)));
+            CERA_TRY(cera_launch_fattn(ctx, W.attn, p, &raw.merge, most, g.f32));
+            if (raw.merge.part) raw.kind = DenseIn::MERGE;
         }
         CERA_TRY(gemv(raw, W.o, streams(W.st_mixer)));
         if (!W.ff) continue;
@@ -166,7 +170,7 @@ cera_hip_status latent_pass(cera_hip_model* m, SeqLayer& W, FAttnPass p) {
         CERA_TRY(cera_launch_dense_gemm(ctx, W.v_up, W.kv, W.attn.row, total, to, g.f32, heads));
         CERA_TRY(cera_launch_latent_spread(ctx, l, W.attn, W.wide, W.kv, total, rows, cap, g.f32));
         p.kv = rows; p.cap = cap;
-        return cera_launch_fattn(ctx, W.wide, p, nullptr, g.f32);
+        return cera_launch_fattn(ctx, W.wide, p, nullptr, 0, g.f32);
     }
     CERA_TRY(cera_launch_latent_prep(ctx, l, W.attn, g.bqkvg, ld, p.n, p.start, W.kv, g.bq, W.attn.kp, g.bqn, g.f32));
     heads.x_stride = l.dim_p(); heads.out_stride = W.attn.kp;
@@ -174,7 +178,7 @@ cera_hip_status latent_pass(cera_hip_model* m, SeqLayer& W, FAttnPass p) {
     CERA_TRY(cera_launch_dense_gemm(ctx, W.k_up_t, g.bqn, static_cast<uint64_t>(l.heads) * l.dim_p(), p.n, to, g.f32, heads));
     const FAttnPass direct = p;
     p.out = g.bo; p.out_head = l.rank_p(); p.out_ld = static_cast<uint64_t>(l.heads) * l.rank_p();
-    CERA_TRY(cera_launch_fattn(ctx, W.attn, p, nullptr, g.f32));
+    CERA_TRY(cera_launch_fattn(ctx, W.attn, p, nullptr, 0, g.f32));
     heads.x_stride = l.rank_p(); heads.out_stride = l.vdim;
     to.out = direct.out; to.ld = direct.out_ld; to.rows = l.vdim;
     return cera_launch_dense_gemm(ctx, W.v_up, g.bo, p.out_ld, p.n, to, g.f32, heads);
@@ -211,7 +215,7 @@ cera_hip_status seq_pass(cera_hip_model* m, const uint32_t* tokens, uint32_t n, 
             FAttnPrep prep = W.prep;
             prep.qkv = g.bqkvg; prep.ld = proj.ld; prep.v_first = W.v_mix ? g.bv_first : nullptr;
             CERA_TRY(cera_launch_fattn_prep(ctx, W.attn, p, prep, g.f32));
-            CERA_TRY(cera_launch_fattn(ctx, W.attn, p, nullptr, g.f32));
+            CERA_TRY(cera_launch_fattn(ctx, W.attn, p, nullptr, 0, g.f32));
         }
         CERA_TRY(cera_launch_dense_gemm(ctx, W.o, g.bcat, W.o.kp, n, streams(W.st_mixer), g.f32));
         if (!W.ff) continue;
@@ -360,7 +364,7 @@ cera_hip_status layered_seq_build(cera_hip_model* m, const cera_hip_layered_conf
     const uint32_t S = c.streams;
     RotationTables tables;
     std::map<std::pair<double, double>, float*> temps;   // factors per position, by their constants
-    uint64_t proj = 0, att = 0, q = 0, ff = 0, first = 0, widest = ld;
+    uint64_t proj = 0, att = 0, q = 0, ff = 0, first = 0, lat = 0, widest = ld;
     auto pack = [&](const cera_hip_tensor& t, DenseMat* out) {
         Packer p(t.m, dense_pad(t.k));
         p.rows(0, 0, t);
@@ -446,6 +450,7 @@ cera_hip_status layered_seq_build(cera_hip_model* m, const cera_hip_layered_conf
         att = std::max<uint64_t>(att, W.o.kp);
         q = std::max<uint64_t>(q, static_cast<uint64_t>(a.heads) * W.attn.kp);
         ff = std::max<uint64_t>(ff, W.down.kp);
+        if (W.latent) lat = std::max<uint64_t>(lat, static_cast<uint64_t>(a.heads) * W.attn.vp);
         widest = std::max({widest, att, ff});
     }
     std::fill(before->next, before->next + S, 1.0f);   // the sum of the streams leaves the last layer
@@ -456,6 +461,7 @@ cera_hip_status layered_seq_build(cera_hip_model* m, const cera_hip_layered_conf
     CERA_TRY(layered_alloc(m, q * g.esz, &g.q, true));
     CERA_TRY(layered_alloc(m, att * g.esz, &g.cat, true));
     if (ff) CERA_TRY(layered_alloc(m, ff * g.esz, &g.act, true));
+    if (lat) CERA_TRY(layered_alloc(m, lat * g.esz, &g.lat, true));
     m->hidden = g.u;
     g.step_fits = cera_dense_gemv_fits(widest, g.f32);
     return CERA_HIP_OK;

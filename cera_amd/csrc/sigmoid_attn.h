@@ -59,6 +59,7 @@ struct ConvHist {
 // merge (nullable): receives partial results over key ranges that the consumer of the output adds up and gates
 // itself -- or part == nullptr when the launch has already written p.out.
 constexpr uint32_t SATTN_MERGE_SPLITS = 8;
+constexpr uint32_t PARTIALS_MAX = 2048;   // heads * splits a consumer takes
 struct SAttnPartials {
     const float* part = nullptr;   // [splits][heads][vdim_p]
     const float* gate = nullptr;   // sigmoid weights: [heads], before the sigmoid

@@ -497,7 +497,7 @@ cera_hip_status run_split(cera_hip_ctx* ctx, AArgs& a, bool f32, bool fused, SAt
     if (merge) {
         *merge = SAttnPartials{};
         const uint32_t fine = std::min((nb + SPLIT_WAVES - 1) / SPLIT_WAVES, SATTN_MERGE_SPLITS);
-        if (nb <= SATTN_MERGE_SPLITS * SPLIT_WAVES * 2) a.splits = fine;   // one block per wavefront, two at the most
+        if (nb <= SATTN_MERGE_SPLITS * SPLIT_WAVES * 2 && a.heads * fine <= PARTIALS_MAX) a.splits = fine;   // one block per wavefront, two at the most
         else merge = nullptr;
     }
     if (a.splits > 1 || merge) {

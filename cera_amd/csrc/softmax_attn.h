@@ -42,8 +42,9 @@ struct FAttnPass {
     uint32_t out_head = 0;
 };
 bool cera_fattn_fits(const FAttnShape& s);
-// merge (nullable, n == 1): receives partial results over key ranges that the consumer adds up itself
-cera_hip_status cera_launch_fattn(cera_hip_ctx* ctx, const FAttnShape& s, const FAttnPass& p, SAttnPartials* merge, bool f32);
+// merge (nullable, n == 1): receives partial results over at most `most` key ranges that the consumer adds up itself --
+// or part == nullptr when the launch has already written p.out, as it does beyond that
+cera_hip_status cera_launch_fattn(cera_hip_ctx* ctx, const FAttnShape& s, const FAttnPass& p, SAttnPartials* merge, uint32_t most, bool f32);
 
 // What stands between the projections and attention in a layer with separate keys and values: norms over the
 // entries of each query and key head, a factor per position on the queries, values mixed with another layer's

@@ -355,82 +355,102 @@ __global__ __launch_bounds__(FW * 64, WPE) void fattn_kernel(FArgs a) {
     }
 }
 
-// One workgroup per (query, head): a thread holds four value columns of every `groups`-th partial result.
-template <typename T> __global__ __launch_bounds__(256) void fattn_merge_kernel(FArgs a) {
+// `threads` consecutive threads per (query, head), `quads` of them with four value columns each for every one of their
+// `groups` shares of the parts; a workgroup holds 256 / threads such pairs.
+template <typename T> __global__ __launch_bounds__(256) void fattn_merge_kernel(FArgs a, uint32_t threads, uint32_t groups) {
     __shared__ __align__(16) f32x4 red[256];
-    __shared__ float wz[256];
-    const uint32_t query = blockIdx.x / a.heads, head = blockIdx.x % a.heads, quads = a.vp / 4, groups = 256 / quads;
-    const uint64_t at = static_cast<uint64_t>(query) * a.heads + head, slice = static_cast<uint64_t>(a.n) * a.heads;
-    // weights of the key ranges, by every wavefront alike
-    const uint32_t lane = threadIdx.x & 63;
-    const float sink2 = a.sink[head] * LOG2E;
-    float m = sink2;
-    for (uint32_t z = lane; z < a.splits; z += 64) m = fmaxf(m, a.ml[(at + z * slice) * 2]);
-    m = wave_max(m);
-    float l = 0.0f;
-    for (uint32_t z = lane; z < a.splits; z += 64) {
-        const float c = __builtin_amdgcn_exp2f(a.ml[(at + z * slice) * 2] - m);
-        l = fmaf(a.ml[(at + z * slice) * 2 + 1], c, l);
-        if (threadIdx.x < 64) wz[z] = c;
-    }
-    const float inv = 1.0f / (wave_sum(l) + __builtin_amdgcn_exp2f(sink2 - m));
-    __syncthreads();
-    const uint32_t q = threadIdx.x % quads, grp = threadIdx.x / quads;
+    const uint32_t quads = a.vp / 4, local = threadIdx.x % threads, q = local % quads, grp = local / quads;
+    const uint64_t rows = static_cast<uint64_t>(a.n) * a.heads, at = static_cast<uint64_t>(blockIdx.x) * (256 / threads) + threadIdx.x / threads;
+    const bool live = threadIdx.x / threads < 256 / threads && at < rows && grp < groups;
+    const uint32_t query = static_cast<uint32_t>(at / a.heads), head = static_cast<uint32_t>(at % a.heads);
     f32x4 s{0.f, 0.f, 0.f, 0.f};
-    if (grp < groups)
+    float inv = 0.0f;
+    if (live) {
+        const float2* const ml = reinterpret_cast<const float2*>(a.ml) + at;
+        const float sink2 = a.sink[head] * LOG2E;
+        float m = sink2;
+#pragma unroll 8
+        for (uint32_t z = 0; z < a.splits; ++z) m = fmaxf(m, ml[z * rows].x);
+        float l = __builtin_amdgcn_exp2f(sink2 - m);
+#pragma unroll 4
+        for (uint32_t z = 0; z < a.splits; ++z) l = fmaf(ml[z * rows].y, __builtin_amdgcn_exp2f(ml[z * rows].x - m), l);
+        inv = 1.0f / l;
+#pragma unroll 4
         for (uint32_t z = grp; z < a.splits; z += groups) {
-            const f32x4 v = *reinterpret_cast<const f32x4*>(a.part + (at + z * slice) * a.vp + q * 4);
+            const f32x4 v = *reinterpret_cast<const f32x4*>(a.part + (at + z * rows) * a.vp + q * 4);
+            const float w = __builtin_amdgcn_exp2f(ml[z * rows].x - m);
 #pragma unroll
-            for (int i = 0; i < 4; ++i) s[i] = fmaf(v[i], wz[z], s[i]);
+            for (int i = 0; i < 4; ++i) s[i] = fmaf(v[i], w, s[i]);
         }
-    red[threadIdx.x] = s;
-    __syncthreads();
-    if (grp != 0) return;
-    for (uint32_t i = 1; i < groups; ++i) s += red[i * quads + q];
+    }
+    if (groups > 1) {
+        red[threadIdx.x] = s;
+        __syncthreads();
+        if (live && grp == 0)
+            for (uint32_t i = 1; i < groups; ++i) s += red[threadIdx.x + i * quads];
+    }
+    if (!live || grp != 0 || q * 4 >= a.vdim) return;
     s.x *= inv; s.y *= inv; s.z *= inv; s.w *= inv;
-    if (q * 4 < a.vdim) finish4<T>(a, query, head, q * 4, s);
+    finish4<T>(a, query, head, q * 4, s);
 }
 
-// ---- preparation: a wavefront per head of q, k or v --------------------------------------------------
+// ---- preparation: sixteen lanes per head of q, k or v, eight entries each at a time -------------------
 struct PrepArgs {
     FAttnPrep p;
-    uint32_t n, start, heads, kv_heads, kp, v_off, vdim, row;
+    uint32_t n, start, heads, kv_heads, kp, v_off, vp, vdim, row;
     uint64_t head_stride;
     void *q, *kv;
+    bool whole_k, whole_v;   // heads start 16-byte aligned and come in whole eights
 };
 template <typename T> __global__ __launch_bounds__(256) void fattn_prep_kernel(PrepArgs a) {
-    const uint32_t lane = threadIdx.x & 63, item = blockIdx.x * 4 + (threadIdx.x >> 6), tok = blockIdx.y, dim = a.p.dim;
+    const uint32_t l8 = (threadIdx.x & 15) * 8, item = blockIdx.x * 16 + (threadIdx.x >> 4), tok = blockIdx.y, dim = a.p.dim;
     if (item >= a.heads + 2 * a.kv_heads) return;
     const uint32_t pos = a.start + tok;
     const float* const src = a.p.qkv + tok * a.p.ld;
+    float v[8];
     if (item < a.heads + a.kv_heads) {   // q | k heads stand back to back
         const bool is_q = item < a.heads;
         const float* const x = src + item * dim;
         const float* const w = is_q ? a.p.q_norm : a.p.k_norm;
         float ss = 0.0f;
-        for (uint32_t c = lane; c < dim; c += 64) ss = fmaf(x[c], x[c], ss);
-        float f = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(dim) + a.p.eps);
-        T* dst;
-        if (is_q) {
-            dst = static_cast<T*>(a.q) + (static_cast<uint64_t>(tok) * a.heads + item) * a.kp;
-        } else {
-            dst = static_cast<T*>(a.kv) + (item - a.heads) * a.head_stride + static_cast<uint64_t>(pos) * a.row;
+        for (uint32_t c = l8; c < dim; c += 128) {
+            load8(x, c, dim, a.whole_k, v);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) ss = fmaf(v[i], v[i], ss);
         }
+        const float f = 1.0f / sqrtf(wave_row_sum(ss) / static_cast<float>(dim) + a.p.eps);
         const float temp = is_q && a.p.q_mult ? a.p.q_mult[pos] : 1.0f;
-        for (uint32_t c = lane; c < a.kp; c += 64) dst[c] = ElemOps<T>::from(c < dim ? x[c] * f * w[c] * temp : 0.0f);
+        T* const dst = is_q ? static_cast<T*>(a.q) + (static_cast<uint64_t>(tok) * a.heads + item) * a.kp
+                            : static_cast<T*>(a.kv) + (item - a.heads) * a.head_stride + static_cast<uint64_t>(pos) * a.row;
+        for (uint32_t c = l8; c < a.kp; c += 128) {   // the pads become zero
+            float wv[8];
+            load8(x, c, dim, a.whole_k, v);
+            load8(w, c, dim, a.whole_k, wv);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) v[i] = v[i] * f * wv[i] * temp;
+            ElemOps<T>::store8(dst + c, v);
+        }
         return;
     }
     const uint32_t h = item - a.heads - a.kv_heads;
     const float* const x = src + (a.heads + a.kv_heads) * dim + h * a.vdim;
     T* const dst = static_cast<T*>(a.kv) + h * a.head_stride + static_cast<uint64_t>(pos) * a.row + a.v_off;
     float* const first = a.p.v_first ? a.p.v_first + (static_cast<uint64_t>(tok) * a.kv_heads + h) * a.vdim : nullptr;
-    for (uint32_t c = lane; c < a.vdim; c += 64) {
-        float v = x[c];
-        if (first) {
-            if (a.p.v_store) first[c] = v;
-            else v = (1.0f - a.p.v_lambda) * v + a.p.v_lambda * first[c];
+    for (uint32_t c = l8; c < a.vp; c += 128) {
+        load8(x, c, a.vdim, a.whole_v, v);
+        if (first && a.p.v_store) {
+            if (a.whole_v && c < a.vdim) ElemOps<float>::store8(first + c, v);
+            else
+#pragma unroll
+                for (int i = 0; i < 8; ++i)
+                    if (c + i < a.vdim) first[c + i] = v[i];
+        } else if (first) {
+            float u[8];
+            load8(first, c, a.vdim, a.whole_v, u);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) v[i] = (1.0f - a.p.v_lambda) * v[i] + a.p.v_lambda * u[i];
         }
-        dst[c] = ElemOps<T>::from(v);
+        ElemOps<T>::store8(dst + c, v);
     }
 }
 
@@ -476,7 +496,7 @@ static cera_hip_status fattn_check(cera_hip_ctx* ctx, const FAttnShape& s, const
     return CERA_HIP_OK;
 }
 
-cera_hip_status cera_launch_fattn(cera_hip_ctx* ctx, const FAttnShape& s, const FAttnPass& p, SAttnPartials* merge, bool f32) {
+cera_hip_status cera_launch_fattn(cera_hip_ctx* ctx, const FAttnShape& s, const FAttnPass& p, SAttnPartials* merge, uint32_t most, bool f32) {
     if (merge) *merge = SAttnPartials{};
     CERA_TRY(fattn_check(ctx, s, p));
     if (merge && p.n != 1) return cera_fail(ctx, CERA_HIP_ERR_SHAPE, "softmax attention: partial results are for one token");
@@ -510,9 +530,12 @@ cera_hip_status cera_launch_fattn(cera_hip_ctx* ctx, const FAttnShape& s, const 
         // share the keys out where the column tiles do not fill the chip: at least two steps of a workgroup each,
         // one for a single token (its launch is all latency)
         const uint32_t wgs = a.tiles * s.kv_heads, steps = (nb + a.kg - 1) / a.kg, least = p.n == 1 ? 1 : 2;
-        const uint32_t room = std::max(1u, 2 * ctx->n_cu / wgs);
-        a.splits = std::max(1u, std::min({room, steps / least, 64u}));
-        if (merge) a.splits = std::min(a.splits, 2 * SATTN_MERGE_SPLITS);
+        a.splits = std::max(1u, std::min({std::max(1u, 2 * ctx->n_cu / wgs), steps / least, p.n == 1 ? 128u : 16u}));
+        if (merge) {
+            most = std::min(most, PARTIALS_MAX / s.heads);
+            if (a.splits > most && steps <= 2 * most) a.splits = most;   // two steps cost less than a launch
+            if (a.splits > most) merge = nullptr;
+        }
         if (a.splits > 1 || merge) {
             void* part;
             const uint64_t rows = static_cast<uint64_t>(a.splits) * a.n * a.heads;
@@ -533,9 +556,12 @@ cera_hip_status cera_launch_fattn(cera_hip_ctx* ctx, const FAttnShape& s, const 
         merge->part = a.part; merge->ml = a.ml; merge->sink = s.sink; merge->splits = a.splits; merge->heads = s.heads;
         merge->vdim = s.vdim; merge->vdim_p = s.vp;
     } else if (a.splits > 1) {
-        const dim3 grid(p.n * s.heads);
-        if (f32) hipLaunchKernelGGL(fattn_merge_kernel<float>, grid, dim3(256), 0, ctx->stream, a);
-        else hipLaunchKernelGGL(fattn_merge_kernel<__bf16>, grid, dim3(256), 0, ctx->stream, a);
+        const uint32_t quads = s.vp / 4, pairs = p.n * s.heads;
+        // one pair per workgroup shares its parts out; many pairs take as few threads each as there are columns
+        const uint32_t groups = pairs < 4 * ctx->n_cu ? 256 / quads : 1, threads = groups > 1 ? 256 : quads;
+        const dim3 grid((pairs + 256 / threads - 1) / (256 / threads));
+        if (f32) hipLaunchKernelGGL(fattn_merge_kernel<float>, grid, dim3(256), 0, ctx->stream, a, threads, groups);
+        else hipLaunchKernelGGL(fattn_merge_kernel<__bf16>, grid, dim3(256), 0, ctx->stream, a, threads, groups);
         HIP_TRY(ctx, hipGetLastError());
     }
     return CERA_HIP_OK;
@@ -545,10 +571,12 @@ cera_hip_status cera_launch_fattn_prep(cera_hip_ctx* ctx, const FAttnShape& s, c
     CERA_TRY(fattn_check(ctx, s, p));
     PrepArgs a{};
     a.p = prep;
-    a.n = p.n; a.start = p.start; a.heads = s.heads; a.kv_heads = s.kv_heads; a.kp = s.kp; a.v_off = s.v_off; a.vdim = s.vdim; a.row = s.row;
+    a.n = p.n; a.start = p.start; a.heads = s.heads; a.kv_heads = s.kv_heads; a.kp = s.kp; a.v_off = s.v_off; a.vp = s.vp; a.vdim = s.vdim; a.row = s.row;
+    a.whole_k = prep.dim % 8 == 0 && (p.n == 1 || prep.ld % 4 == 0);
+    a.whole_v = a.whole_k && s.vdim % 8 == 0;
     a.head_stride = static_cast<uint64_t>(p.cap) * s.row;
     a.q = const_cast<void*>(p.q); a.kv = p.kv;
-    const dim3 grid((s.heads + 2 * s.kv_heads + 3) / 4, p.n);
+    const dim3 grid((s.heads + 2 * s.kv_heads + 15) / 16, p.n);
     if (f32) hipLaunchKernelGGL(fattn_prep_kernel<float>, grid, dim3(256), 0, ctx->stream, a);
     else hipLaunchKernelGGL(fattn_prep_kernel<__bf16>, grid, dim3(256), 0, ctx->stream, a);
     HIP_TRY(ctx, hipGetLastError());
