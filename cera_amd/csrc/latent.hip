@@ -64,16 +64,40 @@ template <typename T> __global__ __launch_bounds__(256) void latent_prep_kernel(
     for (uint32_t c = lane & 15; at + c < a.kp; c += 16) q[at + c] = ElemOps<T>::from(c < l.rot_dim ? rotated(l, x + l.dim, c, pos) : 0.0f);
 }
 
-template <typename T>
-__global__ __launch_bounds__(256) void latent_spread_kernel(const T* __restrict__ cache, uint32_t cache_row, uint32_t rank_p, uint32_t rot_dim, uint32_t dim,
-                                                            uint32_t vdim, uint32_t v_off, uint32_t row, uint32_t total, uint32_t cap, T* __restrict__ rows) {
-    const uint32_t pos = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    T* const dst = rows + (static_cast<uint64_t>(blockIdx.y) * cap + pos) * row;
-    const T* const kr = cache + static_cast<uint64_t>(pos) * cache_row + rank_p;
-    const bool live = pos < total;
-    for (uint32_t c = lane; c < row; c += 64) {
-        if (live && (c < dim || (c >= v_off && c < v_off + vdim))) continue;   // the products' columns
-        dst[c] = live && c >= dim && c < dim + rot_dim ? kr[c - dim] : ElemOps<T>::from(0.0f);
+// What the products leave open of the expanded rows, eight columns per thread: from `dim` (c0 eights) to the values, from
+// the values' end (c1 eights) to the row's end, and whole rows behind the last position.
+struct SpreadArgs {
+    const void* cache;
+    void* rows;
+    uint32_t cache_row, rank_p, rot_dim, dim, vdim, v_off, row, total, to, cap;
+    uint32_t c0, c1, open;    // open: eights per live row
+    bool whole;               // dim and rot_dim come in whole eights
+};
+template <typename T> __global__ __launch_bounds__(256) void latent_spread_kernel(SpreadArgs a) {
+    const uint32_t i = blockIdx.x * 256 + threadIdx.x, live = a.total * a.open, eights = a.row / 8;
+    uint32_t pos, c;
+    if (i < live) {
+        pos = i / a.open;
+        const uint32_t e = i - pos * a.open, front = a.v_off / 8 - a.c0;
+        c = (e < front ? a.c0 + e : a.c1 + e - front) * 8;
+    } else {
+        pos = a.total + (i - live) / eights;
+        c = (i - live) % eights * 8;
+    }
+    if (pos >= a.to) return;
+    T* const dst = static_cast<T*>(a.rows) + (static_cast<uint64_t>(blockIdx.y) * a.cap + pos) * a.row + c;
+    const T* const kr = static_cast<const T*>(a.cache) + static_cast<uint64_t>(pos) * a.cache_row + a.rank_p;
+    float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (i < live && a.whole && c < a.dim + a.rot_dim) {
+        typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+        const u32x4* const from = reinterpret_cast<const u32x4*>(kr + (c - a.dim));
+#pragma unroll
+        for (uint32_t k = 0; k < sizeof(T) / 2; ++k) reinterpret_cast<u32x4*>(dst)[k] = from[k];
+    } else if (i < live && (c < a.dim + a.rot_dim || (c >= a.v_off && c < a.v_off + a.vdim))) {   // beside or among the products' columns
+        for (uint32_t k = c; k < c + 8; ++k)
+            if (k >= a.dim && (k < a.v_off || k >= a.v_off + a.vdim)) dst[k - c] = k < a.dim + a.rot_dim ? kr[k - a.dim] : ElemOps<T>::from(0.0f);
+    } else {
+        ElemOps<T>::store8(dst, v);
     }
 }
 
@@ -169,12 +193,15 @@ cera_hip_status cera_launch_latent_spread(cera_hip_ctx* ctx, const LatentShape& 
                                           const void* cache, uint32_t total, void* rows, uint32_t cap, bool f32) {
     const uint32_t to = fattn_pad(total, FATTN_CAP_STEP);
     if (to > cap) return cera_fail(ctx, CERA_HIP_ERR_POSITION, "latent attention: positions beyond the expanded rows");
-    const dim3 grid(to / 4, l.heads);
-    auto go = [&](auto tag) {
-        using T = decltype(tag);
-        hipLaunchKernelGGL(latent_spread_kernel<T>, grid, dim3(256), 0, ctx->stream, static_cast<const T*>(cache), absorbed.row, l.rank_p(), l.rot_dim, l.dim,
-                           l.vdim, expanded.v_off, expanded.row, total, cap, static_cast<T*>(rows));
-    };
+    SpreadArgs a{};
+    a.cache = cache; a.rows = rows; a.cache_row = absorbed.row; a.rank_p = l.rank_p(); a.rot_dim = l.rot_dim; a.dim = l.dim; a.vdim = l.vdim;
+    a.v_off = expanded.v_off; a.row = expanded.row; a.total = total; a.to = to; a.cap = cap;
+    a.c0 = l.dim / 8; a.c1 = (expanded.v_off + l.vdim) / 8; a.open = expanded.v_off / 8 - a.c0 + expanded.row / 8 - a.c1;
+    a.whole = l.dim % 8 == 0 && l.rot_dim % 8 == 0;
+    const uint64_t threads = static_cast<uint64_t>(total) * a.open + static_cast<uint64_t>(to - total) * (a.row / 8);
+    if (threads > UINT32_MAX - 256) return cera_fail(ctx, CERA_HIP_ERR_POSITION, "latent attention: too many positions to expand");
+    const dim3 grid(static_cast<uint32_t>((threads + 255) / 256), l.heads);
+    auto go = [&](auto tag) { hipLaunchKernelGGL(latent_spread_kernel<decltype(tag)>, grid, dim3(256), 0, ctx->stream, a); };
     if (f32) go(float{});
     else go(static_cast<__bf16>(0.0f));
     HIP_TRY(ctx, hipGetLastError());

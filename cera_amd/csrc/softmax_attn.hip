@@ -2,8 +2,9 @@
 //
 // A workgroup of four wavefronts walks the keys in blocks of 32 rows that it stages in LDS by direct
 // global-to-LDS loads (16-byte chunk c of row k sits in slot c ^ swz(k) of its group of eight).  Wavefronts are
-// `cg` column groups times `kg` key groups: a column is one (query, query head of the kv head) pair, 16 * CT of
-// them per wavefront; key groups take blocks in turn and add up through LDS at the end.  Scores are K . q with the
+// `cg` column groups times `kg` key groups times VG value groups: a column is one (query, query head of the kv head)
+// pair, 16 * CT of them per wavefront; key groups take blocks in turn and add up through LDS at the end; value groups
+// compute the same scores and a share of the value columns each.  Scores are K . q with the
 // keys as matrix rows; a lane then holds, for its one column, the scores of exactly the keys whose values it must
 // supply for the second product -- for bf16 the two 16-key tiles take keys 8 (r / 4) + r % 4 and that plus 4 as
 // their row r, which leaves lane group g with keys 8 g .. 8 g + 7, the operand layout of
@@ -225,15 +226,17 @@ template <typename T> __device__ __forceinline__ void finish4(const FArgs& a, ui
     }
 }
 
-template <typename T, int MK, int MV, int CT, bool EXACT, int WPE>
+template <typename T, int MK, int MV, int CT, int VG, bool EXACT, int WPE>
 __global__ __launch_bounds__(FW * 64, WPE) void fattn_kernel(FArgs a) {
+    static_assert(VG == 1 || (EXACT && MV / VG % 4 == 0), "value groups start at whole 64 columns");
+    constexpr int MW = MV / VG;
     extern __shared__ __align__(16) unsigned char smem[];
     const uint32_t lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    const uint32_t cgi = wave % a.cg, kgi = wave / a.cg;
+    const uint32_t cgi = wave % a.cg, kgi = wave / a.cg % a.kg, vgi = VG > 1 ? wave / a.cg / a.kg : 0;
     // launch index: kv heads (consecutive ones on different XCDs), column tiles with the longest key ranges first, splits
     const uint32_t kvh = blockIdx.x % a.kv_heads, tile = a.tiles - 1 - blockIdx.x / a.kv_heads % a.tiles, split = blockIdx.x / a.kv_heads / a.tiles;
     const uint32_t cols = a.n * a.per, wg_c0 = tile * a.cg * 16 * CT, wg_c1 = min(wg_c0 + a.cg * 16 * CT, cols);
-    const int nk = EXACT ? MK : static_cast<int>(a.kp / 32), nv = EXACT ? MV : static_cast<int>(a.vp / 16);
+    const int nk = EXACT ? MK : static_cast<int>(a.kp / 32), nv = EXACT ? MW : static_cast<int>(a.vp / 16);
     // this workgroup's key blocks
     const uint32_t nb = (a.start + (wg_c1 - 1) / a.per) / 32 + 1;
     const uint32_t share = ((nb + a.splits - 1) / a.splits + a.kg - 1) / a.kg * a.kg;
@@ -260,7 +263,7 @@ __global__ __launch_bounds__(FW * 64, WPE) void fattn_kernel(FArgs a) {
     auto stage = [&](uint32_t b, uint32_t buf) {
         unsigned char* const dst = smem + (buf * a.kg + kgi) * block_bytes;
         const T* const src = kv + static_cast<uint64_t>(b) * 32 * a.row;
-        for (uint32_t s = cgi; s < segs; s += a.cg) {
+        for (uint32_t s = cgi + vgi * a.cg; s < segs; s += a.cg * VG) {
             const uint32_t i = s * 64 + lane, key = (i * a.row_magic) >> 20, slot = i - key * cpr;
             __builtin_amdgcn_global_load_lds(
                 reinterpret_cast<const __attribute__((address_space(1))) void*>(reinterpret_cast<uintptr_t>(src + key * a.row + (slot ^ swz(key)) * E)),
@@ -269,15 +272,16 @@ __global__ __launch_bounds__(FW * 64, WPE) void fattn_kernel(FArgs a) {
     };
     uint32_t b = first + kgi;
     if (b < last) stage(b, 0);
-    Block<T, MK, MV, CT, EXACT> t;
-    Column<MV> col[CT];
+    Block<T, MK, MW, CT, EXACT> t;
+    Column<MW> col[CT];
+    const uint32_t vc0 = vgi * MW * 16;   // this wavefront's first value column
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
         t.load_q(ct, static_cast<const T*>(a.q) + (static_cast<uint64_t>(query[ct]) * a.heads + head[ct]) * a.kp, live[ct], nk, lane);
         col[ct].m = a.sink[head[ct]] * LOG2E;
         col[ct].l = 0.0f;
 #pragma unroll
-        for (int vt = 0; vt < MV; ++vt) col[ct].o[vt] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int vt = 0; vt < MW; ++vt) col[ct].o[vt] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
     uint32_t buf = 0;
     for (uint32_t b0 = first; b0 < last; b0 += a.kg, b += a.kg) {
@@ -286,7 +290,7 @@ __global__ __launch_bounds__(FW * 64, WPE) void fattn_kernel(FArgs a) {
         __syncthreads();
         if (a.stages == 2 && b + a.kg < last) stage(b + a.kg, buf ^ 1);
         if (b < last && wave_live && b * 32 <= hi_max)
-            t.run(reinterpret_cast<const T*>(smem + (buf * a.kg + kgi) * block_bytes), a.row, a.v_off, b * 32, nk, nv, hi, b * 32 + 31 <= hi_min,
+            t.run(reinterpret_cast<const T*>(smem + (buf * a.kg + kgi) * block_bytes), a.row, a.v_off + vc0, b * 32, nk, nv, hi, b * 32 + 31 <= hi_min,
                   a.scale2, col, lane);
         if (a.stages == 2) {
             buf ^= 1;
@@ -299,16 +303,16 @@ __global__ __launch_bounds__(FW * 64, WPE) void fattn_kernel(FArgs a) {
     for (int ct = 0; ct < CT; ++ct) col[ct].l = rows_sum(col[ct].l);
     // key groups: the upper ones hand their columns to the first through LDS, one after the other
     for (uint32_t k = 1; k < a.kg; ++k) {
-        float* const red = reinterpret_cast<float*>(smem) + cgi * (CT * (MV * 256 + 128));
+        float* const red = reinterpret_cast<float*>(smem) + (cgi + vgi * a.cg) * (CT * (MW * 256 + 128));
         __syncthreads();
         if (kgi == k) {
 #pragma unroll
             for (int ct = 0; ct < CT; ++ct) {
-                float* const p = red + ct * (MV * 256 + 128);
+                float* const p = red + ct * (MW * 256 + 128);
                 p[lane] = col[ct].m;
                 p[64 + lane] = col[ct].l;
 #pragma unroll
-                for (int vt = 0; vt < MV; ++vt)
+                for (int vt = 0; vt < MW; ++vt)
                     if (vt < nv) *reinterpret_cast<f32x4*>(p + 128 + (vt * 64 + lane) * 4) = col[ct].o[vt];
             }
         }
@@ -316,12 +320,12 @@ __global__ __launch_bounds__(FW * 64, WPE) void fattn_kernel(FArgs a) {
         if (kgi == 0) {
 #pragma unroll
             for (int ct = 0; ct < CT; ++ct) {
-                const float* const p = red + ct * (MV * 256 + 128);
+                const float* const p = red + ct * (MW * 256 + 128);
                 const float m2 = p[lane], mn = fmaxf(col[ct].m, m2), c1 = __builtin_amdgcn_exp2f(col[ct].m - mn), c2 = __builtin_amdgcn_exp2f(m2 - mn);
                 col[ct].m = mn;
                 col[ct].l = col[ct].l * c1 + p[64 + lane] * c2;
 #pragma unroll
-                for (int vt = 0; vt < MV; ++vt)
+                for (int vt = 0; vt < MW; ++vt)
                     if (vt < nv) {
                         const f32x4 o2 = *reinterpret_cast<const f32x4*>(p + 128 + (vt * 64 + lane) * 4);
 #pragma unroll
@@ -336,60 +340,85 @@ __global__ __launch_bounds__(FW * 64, WPE) void fattn_kernel(FArgs a) {
         if (!live[ct]) continue;
         const uint64_t at = (static_cast<uint64_t>(split) * a.n + query[ct]) * a.heads + head[ct];
         if (a.part) {
-            if (lane < 16) {
+            if (vgi == 0 && lane < 16) {
                 a.ml[at * 2] = col[ct].m;
                 a.ml[at * 2 + 1] = col[ct].l;
             }
         } else {
             const float inv = 1.0f / (col[ct].l + __builtin_amdgcn_exp2f(a.sink[head[ct]] * LOG2E - col[ct].m));
 #pragma unroll
-            for (int vt = 0; vt < MV; ++vt) { col[ct].o[vt].x *= inv; col[ct].o[vt].y *= inv; col[ct].o[vt].z *= inv; col[ct].o[vt].w *= inv; }
+            for (int vt = 0; vt < MW; ++vt) { col[ct].o[vt].x *= inv; col[ct].o[vt].y *= inv; col[ct].o[vt].z *= inv; col[ct].o[vt].w *= inv; }
         }
 #pragma unroll
-        for (int vt = 0; vt < MV; ++vt)
+        for (int vt = 0; vt < MW; ++vt)
             if (vt < nv) {
-                const uint32_t v = vt * 16 + (lane >> 4) * 4;
+                const uint32_t v = vc0 + vt * 16 + (lane >> 4) * 4;
                 if (a.part) *reinterpret_cast<f32x4*>(a.part + at * a.vp + v) = col[ct].o[vt];
                 else finish4<T>(a, query[ct], head[ct], v, col[ct].o[vt]);
             }
     }
 }
 
-// `threads` consecutive threads per (query, head), `quads` of them with four value columns each for every one of their
-// `groups` shares of the parts; a workgroup holds 256 / threads such pairs.
-template <typename T> __global__ __launch_bounds__(256) void fattn_merge_kernel(FArgs a, uint32_t threads, uint32_t groups) {
-    __shared__ __align__(16) f32x4 red[256];
-    const uint32_t quads = a.vp / 4, local = threadIdx.x % threads, q = local % quads, grp = local / quads;
-    const uint64_t rows = static_cast<uint64_t>(a.n) * a.heads, at = static_cast<uint64_t>(blockIdx.x) * (256 / threads) + threadIdx.x / threads;
-    const bool live = threadIdx.x / threads < 256 / threads && at < rows && grp < groups;
+// Many pairs with few parts: a.vp / 4 threads per (query, head), four value columns each.
+template <typename T> __global__ __launch_bounds__(256) void fattn_merge_kernel(FArgs a) {
+    const uint32_t threads = a.vp / 4, q = threadIdx.x % threads, slot = threadIdx.x / threads;
+    const uint64_t rows = static_cast<uint64_t>(a.n) * a.heads, at = static_cast<uint64_t>(blockIdx.x) * (256 / threads) + slot;
+    if (slot >= 256 / threads || at >= rows || q * 4 >= a.vdim) return;
     const uint32_t query = static_cast<uint32_t>(at / a.heads), head = static_cast<uint32_t>(at % a.heads);
-    f32x4 s{0.f, 0.f, 0.f, 0.f};
-    float inv = 0.0f;
-    if (live) {
-        const float2* const ml = reinterpret_cast<const float2*>(a.ml) + at;
-        const float sink2 = a.sink[head] * LOG2E;
-        float m = sink2;
+    const float2* const ml = reinterpret_cast<const float2*>(a.ml) + at;
+    const float sink2 = a.sink[head] * LOG2E;
+    float m = sink2;
 #pragma unroll 8
-        for (uint32_t z = 0; z < a.splits; ++z) m = fmaxf(m, ml[z * rows].x);
-        float l = __builtin_amdgcn_exp2f(sink2 - m);
+    for (uint32_t z = 0; z < a.splits; ++z) m = fmaxf(m, ml[z * rows].x);
+    float l = __builtin_amdgcn_exp2f(sink2 - m);
+    f32x4 s{0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
-        for (uint32_t z = 0; z < a.splits; ++z) l = fmaf(ml[z * rows].y, __builtin_amdgcn_exp2f(ml[z * rows].x - m), l);
-        inv = 1.0f / l;
-#pragma unroll 4
-        for (uint32_t z = grp; z < a.splits; z += groups) {
-            const f32x4 v = *reinterpret_cast<const f32x4*>(a.part + (at + z * rows) * a.vp + q * 4);
-            const float w = __builtin_amdgcn_exp2f(ml[z * rows].x - m);
+    for (uint32_t z = 0; z < a.splits; ++z) {
+        const float2 e = ml[z * rows];
+        const f32x4 v = *reinterpret_cast<const f32x4*>(a.part + (at + z * rows) * a.vp + q * 4);
+        const float w = __builtin_amdgcn_exp2f(e.x - m);
+        l = fmaf(e.y, w, l);
 #pragma unroll
-            for (int i = 0; i < 4; ++i) s[i] = fmaf(v[i], w, s[i]);
-        }
+        for (int i = 0; i < 4; ++i) s[i] = fmaf(v[i], w, s[i]);
     }
-    if (groups > 1) {
-        red[threadIdx.x] = s;
-        __syncthreads();
-        if (live && grp == 0)
-            for (uint32_t i = 1; i < groups; ++i) s += red[threadIdx.x + i * quads];
+    const float inv = 1.0f / l;
+    s.x *= inv; s.y *= inv; s.z *= inv; s.w *= inv;
+    finish4<T>(a, query, head, q * 4, s);
+}
+// Few pairs with many parts (at most 256): a workgroup per (query, head) and 32 value columns, the parts shared out
+// over 32 groups of eight threads.
+template <typename T> __global__ __launch_bounds__(256) void fattn_merge_few_kernel(FArgs a) {
+    __shared__ float wz[256], red[8];
+    __shared__ __align__(16) f32x4 sums[4][8];
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, slices = a.vp / 32, q = blockIdx.x % slices * 8 + (tid & 7), grp = tid >> 3;
+    const uint32_t pair = blockIdx.x / slices, query = pair / a.heads, head = pair % a.heads;
+    const uint64_t rows = static_cast<uint64_t>(a.n) * a.heads;
+    const float sink2 = a.sink[head] * LOG2E;
+    const float2 e = tid < a.splits ? reinterpret_cast<const float2*>(a.ml)[pair + tid * rows] : make_float2(sink2, 0.0f);
+    float m = wave_max(e.x);
+    if (lane == 0) red[wave] = m;
+    __syncthreads();
+    m = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), sink2);
+    const float w = __builtin_amdgcn_exp2f(e.x - m), part = wave_sum(e.y * w);
+    wz[tid] = w;
+    if (lane == 0) red[4 + wave] = part;
+    __syncthreads();
+    const float inv = 1.0f / (red[4] + red[5] + red[6] + red[7] + __builtin_amdgcn_exp2f(sink2 - m));
+    f32x4 s{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (uint32_t z = grp; z < a.splits; z += 32) {
+        const f32x4 v = *reinterpret_cast<const f32x4*>(a.part + (pair + z * rows) * a.vp + q * 4);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) s[i] = fmaf(v[i], wz[z], s[i]);
     }
-    if (!live || grp != 0 || q * 4 >= a.vdim) return;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int d = 8; d <= 32; d <<= 1) s[i] += __shfl_xor(s[i], d);
+    if (lane < 8) sums[wave][lane] = s;
+    __syncthreads();
+    if (tid >= 8 || q * 4 >= a.vdim) return;
+    s = sums[0][tid] + sums[1][tid] + sums[2][tid] + sums[3][tid];
     s.x *= inv; s.y *= inv; s.z *= inv; s.w *= inv;
     finish4<T>(a, query, head, q * 4, s);
 }
@@ -470,10 +499,10 @@ template <class F> void by_size(const FArgs& a, bool f32, F&& f) {
     return f(Int<18>{}, Int<32>{}, std::false_type{});
 }
 
-template <typename T, int MK, int MV, int CT, bool EXACT>
+constexpr int wavefronts_per_simd(int mk) { return mk <= 6 ? 2 : 1; }   // what the registers leave room for
+template <typename T, int MK, int MV, int CT, int VG, bool EXACT>
 cera_hip_status launch(cera_hip_ctx* ctx, const FArgs& a, uint32_t grid, uint64_t lds) {
-    constexpr int WPE = MK <= 6 ? 2 : 1;   // wavefronts per SIMD the register budget leaves room for
-    auto* const fn = fattn_kernel<T, MK, MV, CT, EXACT, WPE>;
+    auto* const fn = fattn_kernel<T, MK, MV, CT, VG, EXACT, wavefronts_per_simd(MK)>;
     if (lds > 64 * 1024) {
         static const hipError_t allowed = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, FATTN_LDS_MAX);
         HIP_TRY(ctx, allowed);
@@ -517,16 +546,19 @@ cera_hip_status cera_launch_fattn(cera_hip_ctx* ctx, const FAttnShape& s, const 
         // two column tiles per wavefront where that still fills the chip
         const bool two = CAN2 && !f32 && static_cast<uint64_t>(col_tiles + 7) / 8 * s.kv_heads >= ctx->n_cu;
         const uint32_t tiles = two ? (col_tiles + 1) / 2 : col_tiles;
-        a.cg = tiles >= 3 ? 4 : tiles;
-        a.kg = FW / a.cg;
+        // a row so large that two blocks of it take all LDS: two wavefronts share a column instead of the keys
+        constexpr bool CAN_SHARE = EX && MK > 8 && MV % 8 == 0;
+        const bool share = CAN_SHARE && tiles <= 2;
+        a.cg = share ? 2 : tiles >= 3 ? 4 : tiles;
+        a.kg = share ? 1 : FW / a.cg;
         a.tiles = (tiles + a.cg - 1) / a.cg;
         const uint64_t block = 32ull * s.row * esz, red = a.kg > 1 ? static_cast<uint64_t>(a.cg) * (two ? 2 : 1) * (MV * 256 + 128) * 4 : 0;
         while (a.kg > 1 && a.kg * block > FATTN_LDS_MAX) a.kg /= 2;
-        if (a.cg * a.kg != FW) {   // wavefronts without a key group take columns that do not exist: they only help staging
+        if (!share && a.cg * a.kg != FW) {   // wavefronts without a key group take columns that do not exist: they only help staging
             a.cg = FW / a.kg;
             a.tiles = (tiles + a.cg - 1) / a.cg;
         }
-        a.stages = 2 * a.kg * block <= 64 * 1024 ? 2 : 1;
+        a.stages = 2 * a.kg * block <= (wavefronts_per_simd(MK) == 1 ? FATTN_LDS_MAX : 64 * 1024) ? 2 : 1;
         // share the keys out where the column tiles do not fill the chip: at least two steps of a workgroup each,
         // one for a single token (its launch is all latency)
         const uint32_t wgs = a.tiles * s.kv_heads, steps = (nb + a.kg - 1) / a.kg, least = p.n == 1 ? 1 : 2;
@@ -547,9 +579,13 @@ cera_hip_status cera_launch_fattn(cera_hip_ctx* ctx, const FAttnShape& s, const 
         const uint32_t grid = wgs * a.splits;
         const uint64_t lds = std::max(a.stages * a.kg * block, red);
         if constexpr (!EX) {
-            st = f32 ? launch<float, MK, MV, 1, EX>(ctx, a, grid, lds) : launch<__bf16, MK, MV, 1, EX>(ctx, a, grid, lds);
-        } else if constexpr (CAN2) st = two ? launch<__bf16, MK, MV, 2, EX>(ctx, a, grid, lds) : launch<__bf16, MK, MV, 1, EX>(ctx, a, grid, lds);
-        else st = launch<__bf16, MK, MV, 1, EX>(ctx, a, grid, lds);
+            st = f32 ? launch<float, MK, MV, 1, 1, EX>(ctx, a, grid, lds) : launch<__bf16, MK, MV, 1, 1, EX>(ctx, a, grid, lds);
+        } else {
+            st = CERA_HIP_ERR_SHAPE;
+            if constexpr (CAN2) { if (two) st = launch<__bf16, MK, MV, 2, 1, EX>(ctx, a, grid, lds); }
+            if constexpr (CAN_SHARE) { if (share) st = launch<__bf16, MK, MV, 1, 2, EX>(ctx, a, grid, lds); }
+            if (!two && !share) st = launch<__bf16, MK, MV, 1, 1, EX>(ctx, a, grid, lds);
+        }
     });
     CERA_TRY(st);
     if (merge) {
@@ -557,11 +593,11 @@ cera_hip_status cera_launch_fattn(cera_hip_ctx* ctx, const FAttnShape& s, const 
         merge->vdim = s.vdim; merge->vdim_p = s.vp;
     } else if (a.splits > 1) {
         const uint32_t quads = s.vp / 4, pairs = p.n * s.heads;
-        // one pair per workgroup shares its parts out; many pairs take as few threads each as there are columns
-        const uint32_t groups = pairs < 4 * ctx->n_cu ? 256 / quads : 1, threads = groups > 1 ? 256 : quads;
-        const dim3 grid((pairs + 256 / threads - 1) / (256 / threads));
-        if (f32) hipLaunchKernelGGL(fattn_merge_kernel<float>, grid, dim3(256), 0, ctx->stream, a, threads, groups);
-        else hipLaunchKernelGGL(fattn_merge_kernel<__bf16>, grid, dim3(256), 0, ctx->stream, a, threads, groups);
+        const bool few = pairs < 4 * ctx->n_cu;
+        const dim3 grid(few ? pairs * (s.vp / 32) : (pairs + 256 / quads - 1) / (256 / quads));
+        auto go = [&](auto* fn) { hipLaunchKernelGGL(fn, grid, dim3(256), 0, ctx->stream, a); };
+        if (few) go(f32 ? fattn_merge_few_kernel<float> : fattn_merge_few_kernel<__bf16>);
+        else go(f32 ? fattn_merge_kernel<float> : fattn_merge_kernel<__bf16>);
         HIP_TRY(ctx, hipGetLastError());
     }
     return CERA_HIP_OK;

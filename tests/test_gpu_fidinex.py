@@ -324,8 +324,8 @@ def test_long_prompts_take_the_large_tiles(tmp_path, f32):
 @DTYPES
 def test_steps_behind_a_very_long_context(tmp_path, f32):
     """Thousands of visible keys: decode steps and short portions split them over many workgroups."""
-    cfg = U.config([U.attention(4, 2, 64, 64, (0.1, 1000), True, ff=48), U.latent(2, 24, 8, 36, 68, 900.0), U.attention(2, 1, 24, 64, None, False)],
-                   width=48, vocab=30, streams=2)
+    cfg = U.config([U.attention(4, 2, 64, 64, (0.1, 1000), True, ff=48), U.latent(2, 24, 8, 36, 68, 900.0), U.attention(2, 1, 24, 64, None, False),
+                    U.latent(4, 24, 64, 36, 512, 5000.0)], width=48, vocab=30, streams=2)
     w = U.random_model(cfg, 43)
     m = _open(U.save(tmp_path / "m", cfg, w), f32, 4400)
     toks = U.tokens(cfg, 4330, 3)
