@@ -562,7 +562,7 @@ cera_hip_status cera_launch_fattn(cera_hip_ctx* ctx, const FAttnShape& s, const 
         // share the keys out where the column tiles do not fill the chip: at least two steps of a workgroup each,
         // one for a single token (its launch is all latency)
         const uint32_t wgs = a.tiles * s.kv_heads, steps = (nb + a.kg - 1) / a.kg, least = p.n == 1 ? 1 : 2;
-        a.splits = std::max(1u, std::min({std::max(1u, 2 * ctx->n_cu / wgs), steps / least, p.n == 1 ? 128u : 16u}));
+        a.splits = std::max(1u, std::min({std::max(1u, 2 * ctx->n_cu / wgs), steps / least, p.n == 1 ? 256u : 16u}));
         if (merge) {
             most = std::min(most, PARTIALS_MAX / s.heads);
             if (a.splits > most && steps <= 2 * most) a.splits = most;   // two steps cost less than a launch
